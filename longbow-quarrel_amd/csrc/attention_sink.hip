@@ -19,6 +19,12 @@
 // holds their keys side by side, K[block][value head][offset][map][key size], V[block][value head][...]: key head j
 // reads map j % maps of value head j / maps (differential attention: two score maps over the same values).
 // `out_f32`: out is 32-bit whatever the dtype of q and the cache.
+//
+// A score may be shaped on its way to the softmax, each step where it is asked for (`ScoreShape`), all in 32-bit:
+//   s = q . k * scale * temp[h];   s = cap tanh(s / cap);   s -= r1[h] ln(1 + r2[h] (p - t));
+//   s += dist[h][min(p - t, dist_n - 1)]   (a bias looked up by distance, the last entry for all that is farther).
+// The sink's score is not shaped.  `wide_gate`: a logit for every entry of the result, [rows, nh * value size] in
+// 32-bit, whose sigmoid multiplies it.
 #include "common.h"
 
 namespace {
@@ -36,6 +42,13 @@ __device__ inline f32x4 ld4(const bf16_t* p) {
   return r;
 }
 
+struct ScoreShape {
+  float cap;                       // 0: no cap
+  const float *temp, *r1, *r2;     // a number a query head each, or null (r1 and r2 together)
+  const float* dist;               // [nh][dist_n], or null
+  int dist_n;
+};
+
 struct SinkArgs {
   int ldq, ldo, ldg, rows, rows_per_tile, heads_per_tile, nh, nkv, KD, VD;
   const int *row_pos, *row_seq, *seq_slot, *block_table;
@@ -49,7 +62,51 @@ struct SinkArgs {
   float* part;
   int maps, out_f32;
   const float* sinks;  // null: the sink's score is 0
+  ScoreShape shape;
+  const float* wide_gate;
+  int ldwg;
 };
+
+// What a lane needs of its query head to shape a score.
+struct HeadShape {
+  float mul, cap, inv_cap, r1, r2;
+  const float* dist;
+  int last;
+  bool log_bias;
+};
+
+__device__ inline HeadShape head_shape(const SinkArgs& a, int h) {
+  HeadShape s;
+  s.mul = a.shape.temp != nullptr ? a.scale * a.shape.temp[h] : a.scale;
+  s.cap = a.shape.cap, s.inv_cap = a.shape.cap > 0.f ? 1.f / a.shape.cap : 0.f;
+  s.r1 = a.shape.r1 != nullptr ? a.shape.r1[h] : 0.f, s.r2 = a.shape.r1 != nullptr ? a.shape.r2[h] : 0.f;
+  s.log_bias = a.shape.r1 != nullptr;
+  s.last = a.shape.dist_n - 1;
+  s.dist = a.shape.dist != nullptr ? a.shape.dist + (long long)h * a.shape.dist_n : nullptr;
+  return s;
+}
+
+// The score of a key `d` positions back (d >= 0).  EXACT: the library's tanh and logarithm (32-bit runs); else the
+// hardware's exponential and logarithm, whose absolute error is that of a 32-bit rounding of 1.
+template <bool EXACT>
+__device__ inline float shaped(float dot, int d, const HeadShape& s) {
+  float v = dot * s.mul;
+  if (s.cap > 0.f) {
+    const float y = v * s.inv_cap;
+    if constexpr (EXACT) {
+      v = s.cap * tanhf(y);
+    } else {
+      const float e = __expf(-2.f * fabsf(y));
+      v = copysignf(s.cap * (1.f - e) * __builtin_amdgcn_rcpf(1.f + e), y);
+    }
+  }
+  if (s.log_bias) {
+    if constexpr (EXACT) v -= s.r1 * log1pf(s.r2 * (float)d);
+    else v -= s.r1 * __logf(fmaf(s.r2, (float)d, 1.f));
+  }
+  if (s.dist != nullptr) v += s.dist[min(d, s.last)];
+  return v;
+}
 
 template <typename T>
 __device__ inline void put_out(T* out, long long at, float v, int out_f32) {
@@ -73,7 +130,7 @@ constexpr int MAX_KD = 256;
 constexpr int SPLIT = 4;
 typedef short bf16x4 __attribute__((ext_vector_type(4)));
 
-template <typename T, int HSV>  // HSV: value size / 16
+template <typename T, int HSV, bool SHAPED>  // HSV: value size / 16
 __global__ __launch_bounds__(64 * SPLIT) void sink_tiles_kernel(const T* __restrict__ q, T* __restrict__ out,
                                                                 const T* __restrict__ gate,
                                                                 const T* __restrict__ kcache,
@@ -96,6 +153,8 @@ __global__ __launch_bounds__(64 * SPLIT) void sink_tiles_kernel(const T* __restr
   const int my_row = r0 + min(c / GH, n_rows - 1), h = hbase + c % GH;
   const int my_pos = a.row_pos[my_row], my_seq = a.row_seq[my_row];
   const int my_lo = (a.window > 0 && my_pos >= a.window) ? my_pos - a.window + 1 : 0;
+  HeadShape hs;
+  if constexpr (SHAPED) hs = head_shape(a, h);
   float* myq = smem + (g * 16 + c) * QROW;
   if (wave == 0) {
     for (int sl = 0; sl < HS; ++sl) {
@@ -162,7 +221,10 @@ __global__ __launch_bounds__(64 * SPLIT) void sink_tiles_kernel(const T* __restr
           for (int e = 0; e < 4; ++e) {
             const int t = t0 + 16 * kt + 4 * g + e;
             const bool valid = mine && t <= my_pos && (t >= my_lo || t < a.keep_first);
-            st[kt][e] = valid ? st[kt][e] * a.scale : -INFINITY;
+            float score;
+            if constexpr (SHAPED) score = shaped<!HALF>(st[kt][e], max(my_pos - t, 0), hs);
+            else score = st[kt][e] * a.scale;
+            st[kt][e] = valid ? score : -INFINITY;
             cmax = fmaxf(cmax, st[kt][e]);
           }
         cmax = fmaxf(cmax, __shfl_xor(cmax, 16, 64));
@@ -256,8 +318,14 @@ __global__ __launch_bounds__(64 * SPLIT) void sink_tiles_kernel(const T* __restr
       float f = inv4[e];
       if (gate != nullptr) f /= 1.f + expf(-to_f32(gate[(long long)(r0 + row) * a.ldg + hh]));
       const long long orow = (long long)(r0 + row) * a.ldo + hh * (HSV * 16) + c;
+      if (a.wide_gate != nullptr) {
+        const float* wg = a.wide_gate + (long long)(r0 + row) * a.ldwg + hh * (HSV * 16) + c;
 #pragma unroll
-      for (int dt = 0; dt < HSV; ++dt) put_out(out, orow + dt * 16, o[dt][e] * f, a.out_f32);
+        for (int dt = 0; dt < HSV; ++dt) put_out(out, orow + dt * 16, o[dt][e] * f / (1.f + expf(-wg[dt * 16])), a.out_f32);
+      } else {
+#pragma unroll
+        for (int dt = 0; dt < HSV; ++dt) put_out(out, orow + dt * 16, o[dt][e] * f, a.out_f32);
+      }
     }
   }
 }
@@ -306,8 +374,14 @@ __global__ __launch_bounds__(64) void sink_merge_kernel(T* __restrict__ out, con
       float f = inv4[e];
       if (gate != nullptr) f /= 1.f + expf(-to_f32(gate[(long long)(r0 + row) * a.ldg + hh]));
       const long long orow = (long long)(r0 + row) * a.ldo + hh * (HSV * 16) + c;
+      if (a.wide_gate != nullptr) {
+        const float* wg = a.wide_gate + (long long)(r0 + row) * a.ldwg + hh * (HSV * 16) + c;
 #pragma unroll
-      for (int dt = 0; dt < HSV; ++dt) put_out(out, orow + dt * 16, o[dt][e] * f, a.out_f32);
+        for (int dt = 0; dt < HSV; ++dt) put_out(out, orow + dt * 16, o[dt][e] * f / (1.f + expf(-wg[dt * 16])), a.out_f32);
+      } else {
+#pragma unroll
+        for (int dt = 0; dt < HSV; ++dt) put_out(out, orow + dt * 16, o[dt][e] * f, a.out_f32);
+      }
     }
   }
 }
@@ -316,7 +390,7 @@ __global__ __launch_bounds__(64) void sink_merge_kernel(T* __restrict__ out, con
 // several) for the sums.
 constexpr int MAX_DIM = 1024;
 
-template <typename T>
+template <typename T, bool SHAPED>
 __global__ __launch_bounds__(64) void sink_rows_kernel(const T* __restrict__ q, T* __restrict__ out,
                                                        const T* __restrict__ gate, const T* __restrict__ kcache,
                                                        const T* __restrict__ vcache, SinkArgs a) {
@@ -330,6 +404,8 @@ __global__ __launch_bounds__(64) void sink_rows_kernel(const T* __restrict__ q, 
   const int lo = (a.window > 0 && p >= a.window) ? p - a.window + 1 : 0;
   const int* table = a.block_table + (long long)a.seq_slot[a.row_seq[r]] * a.bt_stride;
   for (int d = lane; d < KD; d += 64) qs[d] = to_f32(q[(long long)r * a.ldq + h * KD + d]);
+  HeadShape hs;
+  if constexpr (SHAPED) hs = head_shape(a, h);
   float m = a.sink ? (a.sinks != nullptr ? a.sinks[h] : 0.f) : -INFINITY, l = a.sink ? 1.f : 0.f;
   float acc[MAX_DIM / 64];
 #pragma unroll
@@ -348,7 +424,8 @@ __global__ __launch_bounds__(64) void sink_rows_kernel(const T* __restrict__ q, 
       const T* kr = kcache + ((blk * nvh + g) * BS + off) * (long long)a.maps * KD + kmap * KD;
       float dot = 0.f;
       for (int d = 0; d < KD; ++d) dot = fmaf(qs[d], to_f32(kr[d]), dot);
-      s = dot * a.scale;
+      if constexpr (SHAPED) s = shaped<sizeof(T) == 4>(dot, p - t, hs);
+      else s = dot * a.scale;
     }
     const float m_new = fmaxf(m, wave_max(s));
     const bool none = m_new == -INFINITY;
@@ -380,7 +457,10 @@ __global__ __launch_bounds__(64) void sink_rows_kernel(const T* __restrict__ q, 
 #pragma unroll
   for (int j = 0; j < MAX_DIM / 64; ++j) {
     const int d = lane + 64 * j;
-    if (d < VD) put_out(out, (long long)r * a.ldo + h * VD + d, acc[j] * f, a.out_f32);
+    if (d < VD) {
+      const float open = a.wide_gate != nullptr ? 1.f / (1.f + expf(-a.wide_gate[(long long)r * a.ldwg + h * VD + d])) : 1.f;
+      put_out(out, (long long)r * a.ldo + h * VD + d, acc[j] * f * open, a.out_f32);
+    }
   }
 }
 
@@ -442,6 +522,10 @@ TileShape tile_shape(int el, int rows, int batch, int nh, int nkv, int KD, int V
   return t;
 }
 
+bool scores_shaped(const ScoreShape& s) {
+  return s.cap > 0.f || s.temp != nullptr || s.r1 != nullptr || s.dist != nullptr;
+}
+
 template <typename T>
 bool launch_tiles(const void* q, void* out, const void* gate, const void* kcache, const void* vcache, const SinkArgs& a,
                   int batch, int max_len, float* part, long long part_floats, hipStream_t stream) {
@@ -457,10 +541,15 @@ bool launch_tiles(const void* q, void* out, const void* gate, const void* kcache
   b.ksplit = t.part_floats > 0 && t.part_floats <= part_floats ? t.ksplit : 1;
   b.part = part;
   dim3 grid(t.grid_x, t.grid_y, b.ksplit);
+  const bool shaped_scores = scores_shaped(a.shape);
 #define LQ_SINK(HSV)                                                                                                  \
   case HSV:                                                                                                           \
-    sink_tiles_kernel<T, HSV><<<grid, 64 * SPLIT, 0, stream>>>((const T*)q, (T*)out, (const T*)gate, (const T*)kcache,        \
-                                                       (const T*)vcache, b);                                          \
+    if (shaped_scores)                                                                                                \
+      sink_tiles_kernel<T, HSV, true><<<grid, 64 * SPLIT, 0, stream>>>((const T*)q, (T*)out, (const T*)gate,           \
+                                                                       (const T*)kcache, (const T*)vcache, b);        \
+    else                                                                                                              \
+      sink_tiles_kernel<T, HSV, false><<<grid, 64 * SPLIT, 0, stream>>>((const T*)q, (T*)out, (const T*)gate,          \
+                                                                        (const T*)kcache, (const T*)vcache, b);       \
     if (b.ksplit > 1) sink_merge_kernel<T, HSV><<<dim3(t.grid_x, t.grid_y), 64, 0, stream>>>((T*)out, (const T*)gate, b);   \
     return true;
   switch (a.VD / 16) {
@@ -501,13 +590,18 @@ extern "C" long long lq_sink_attention_workspace(int dtype, int rows, int batch,
 }
 
 // `gate`: null, or [rows, nh] logits (stride ldg) in the dtype of q.  `rows == batch` means single tokens.  `part`:
-// lq_sink_attention_workspace(...) floats for `max_len`, or null.
+// lq_sink_attention_workspace(...) floats for `max_len`, or null.  `cap` to `dist_n`: how a score is shaped (see the
+// top of the file; 0 and null: not), `wide_gate` [rows, nh * VD] 32-bit logits (stride ldwg) or null.
 extern "C" int lq_sink_attention(const void* q, int ldq, void* out, int ldo, const void* gate, int ldg, int dtype, int rows,
                                  int batch, int nh, int nkv, int KD, int VD, const int* row_pos, const int* row_seq,
                                  const int* seq_slot, const int* block_table, int bt_stride, const void* kcache,
                                  const void* vcache, int block_size, float scale, int window, int keep_first, int sink,
                                  int force_rows, int max_len, float* part, long long part_floats, const float* sinks,
-                                 int maps, int out_f32, hipStream_t stream) {
+                                 int maps, int out_f32, float cap, const float* temp, const float* r1, const float* r2,
+                                 const float* dist, int dist_n, const float* wide_gate, int ldwg, hipStream_t stream) {
+  LQ_REQUIRE(cap >= 0.f && (r1 == nullptr) == (r2 == nullptr) && (dist == nullptr || dist_n > 0),
+             "sink_attention: a cap of %g, a table by distance of %d entries", (double)cap, dist_n);
+  LQ_REQUIRE(wide_gate == nullptr || ldwg >= nh * VD, "sink_attention: the wide gate's stride is smaller than its row");
   LQ_REQUIRE(maps >= 1 && nkv % maps == 0, "sink_attention: %d key heads in runs of %d that share a value head", nkv, maps);
   LQ_REQUIRE(sinks == nullptr || sink, "sink_attention: learned sink scores without a sink");
   LQ_REQUIRE(rows > 0 && batch > 0 && rows >= batch, "sink_attention: rows %d and sequences %d", rows, batch);
@@ -523,6 +617,8 @@ extern "C" int lq_sink_attention(const void* q, int ldq, void* out, int ldo, con
   a.bt_stride = bt_stride, a.BS = block_size, a.scale = scale, a.window = window, a.keep_first = keep_first, a.sink = sink;
   a.ksplit = 1, a.part = nullptr;
   a.maps = maps, a.out_f32 = out_f32 || dtype == LQ_F32, a.sinks = sinks;
+  a.shape = {cap, temp, r1, r2, dist, dist_n};
+  a.wide_gate = wide_gate, a.ldwg = ldwg;
   if (!force_rows) {
     const bool done = dtype == LQ_F32
                           ? launch_tiles<float>(q, out, gate, kcache, vcache, a, batch, max_len, part, part_floats, stream)
@@ -534,12 +630,14 @@ extern "C" int lq_sink_attention(const void* q, int ldq, void* out, int ldo, con
   }
   LQ_REQUIRE(rows <= 0x7fffffff, "sink_attention: too many rows");
   dim3 grid(rows, nh);
-  if (dtype == LQ_F32)
-    sink_rows_kernel<float><<<grid, 64, 0, stream>>>((const float*)q, (float*)out, (const float*)gate, (const float*)kcache,
-                                                     (const float*)vcache, a);
-  else
-    sink_rows_kernel<bf16_t><<<grid, 64, 0, stream>>>((const bf16_t*)q, (bf16_t*)out, (const bf16_t*)gate,
-                                                      (const bf16_t*)kcache, (const bf16_t*)vcache, a);
+#define LQ_SINK_ROWS(T, SHAPED)                                                                                     \
+  sink_rows_kernel<T, SHAPED><<<grid, 64, 0, stream>>>((const T*)q, (T*)out, (const T*)gate, (const T*)kcache,      \
+                                                       (const T*)vcache, a)
+  if (dtype == LQ_F32 && scores_shaped(a.shape)) LQ_SINK_ROWS(float, true);
+  else if (dtype == LQ_F32) LQ_SINK_ROWS(float, false);
+  else if (scores_shaped(a.shape)) LQ_SINK_ROWS(bf16_t, true);
+  else LQ_SINK_ROWS(bf16_t, false);
+#undef LQ_SINK_ROWS
   LQ_CHECK_LAUNCH("sink_attention(rows)");
   return 0;
 }

@@ -5,22 +5,42 @@
 #include <algorithm>
 
 // ---------------------------------------------------------------- embedding
+// Sine and cosine of position * frequency, the angle reduced in double.
+__device__ inline float2 sinusoid_of(double pos, double freq) {
+  const double a = pos * freq;
+  const double n = rint(a * 0.15915494309189533577);
+  double rem = fma(-n, 6.283185307179586232, a);
+  rem = fma(-n, 2.4492935982947064e-16, rem);
+  float2 r;
+  sincosf((float)rem, &r.x, &r.y);
+  return r;
+}
+
 // out[r, :] = float(table[token[r], :])   (row copy, internal/device/kernels.metal:465-467)
 // A token that is no row of the table (a replayed step can be handed the sampler's "no token" before the
 // host has seen it) gives a row of zeros: nothing outside the table is read.
 // A packed table (the layout of lq_pack_weight, for a table that is also the head's weight) keeps 8 rows'
 // slabs of 64 elements side by side: element k of row n lies at (n / 8) 8 D + (k / 64) 512 + (n % 8) 64 + k % 64.
+// With `freqs` ([(D + 1) / 2], double) a position vector is added: column 2 i takes the sine, column 2 i + 1 the cosine of
+// row_pos[r] * freqs[i].
 template <typename T>
 __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict__ tokens,
-                             float* __restrict__ out, int D, int vocab, int packed, float scale) {
+                             float* __restrict__ out, int D, int vocab, int packed, float scale,
+                             const int* __restrict__ row_pos, const double* __restrict__ freqs) {
   const int r = blockIdx.x;
   const long long tok = tokens[r];
   const bool known = tok >= 0 && tok < vocab;
   const long long row = known ? tok : 0;
   const T* src = packed ? table + (row >> 3) * 8 * (long long)D + (row & 7) * 64 : table + row * (long long)D;
   float* dst = out + (long long)r * D;
-  for (int j = threadIdx.x; j < D; j += blockDim.x)
-    dst[j] = known ? to_f32(src[packed ? ((j >> 6) << 9) + (j & 63) : j]) * scale : 0.0f;
+  for (int j = threadIdx.x; j < D; j += blockDim.x) {
+    float v = known ? to_f32(src[packed ? ((j >> 6) << 9) + (j & 63) : j]) * scale : 0.0f;
+    if (freqs != nullptr) {
+      const float2 sc = sinusoid_of((double)row_pos[r], freqs[j >> 1]);
+      v += (j & 1) ? sc.y : sc.x;
+    }
+    dst[j] = v;
+  }
 }
 
 // A bfloat16 row of a width that is a multiple of 8, 16 bytes a lane and load: all of a thread's loads are on
@@ -31,7 +51,9 @@ typedef float embed_f32x4 __attribute__((ext_vector_type(4)));
 template <int PER_THREAD>
 __global__ __launch_bounds__(256) void embed_bf16_vec_kernel(const bf16_t* __restrict__ table,
                                                              const int* __restrict__ tokens, float* __restrict__ out,
-                                                             int D, int vocab, int packed, float scale) {
+                                                             int D, int vocab, int packed, float scale,
+                                                             const int* __restrict__ row_pos,
+                                                             const double* __restrict__ freqs) {
   const int r = blockIdx.x;
   const long long tok = tokens[r];
   const bool known = tok >= 0 && tok < vocab;
@@ -51,35 +73,46 @@ __global__ __launch_bounds__(256) void embed_bf16_vec_kernel(const bf16_t* __res
   for (int i = 0; i < PER_THREAD; ++i) {
     const int c = threadIdx.x + i * 256;
     if (c < chunks) {
-      dst[2 * c] = (embed_f32x4){__uint_as_float(v[i][0] << 16) * scale, __uint_as_float(v[i][0] & 0xffff0000u) * scale,
-                                 __uint_as_float(v[i][1] << 16) * scale, __uint_as_float(v[i][1] & 0xffff0000u) * scale};
-      dst[2 * c + 1] = (embed_f32x4){__uint_as_float(v[i][2] << 16) * scale, __uint_as_float(v[i][2] & 0xffff0000u) * scale,
-                                     __uint_as_float(v[i][3] << 16) * scale, __uint_as_float(v[i][3] & 0xffff0000u) * scale};
+      embed_f32x4 lo = {__uint_as_float(v[i][0] << 16) * scale, __uint_as_float(v[i][0] & 0xffff0000u) * scale,
+                        __uint_as_float(v[i][1] << 16) * scale, __uint_as_float(v[i][1] & 0xffff0000u) * scale};
+      embed_f32x4 hi = {__uint_as_float(v[i][2] << 16) * scale, __uint_as_float(v[i][2] & 0xffff0000u) * scale,
+                        __uint_as_float(v[i][3] << 16) * scale, __uint_as_float(v[i][3] & 0xffff0000u) * scale};
+      if (freqs != nullptr) {
+        const double pos = (double)row_pos[r];
+        const float2 s0 = sinusoid_of(pos, freqs[4 * c]), s1 = sinusoid_of(pos, freqs[4 * c + 1]);
+        const float2 s2 = sinusoid_of(pos, freqs[4 * c + 2]), s3 = sinusoid_of(pos, freqs[4 * c + 3]);
+        lo += (embed_f32x4){s0.x, s0.y, s1.x, s1.y};
+        hi += (embed_f32x4){s2.x, s2.y, s3.x, s3.y};
+      }
+      dst[2 * c] = lo, dst[2 * c + 1] = hi;
     }
   }
 }
 
-// out[r, :] = scale * table[tokens[r], :] (a model's own constant; 1 for most)
+// out[r, :] = scale * table[tokens[r], :] (a model's own constant; 1 for most), plus the sinusoids of the rows'
+// positions where `freqs` is given
 extern "C" int lq_embed(const void* table, int table_dtype, const int* tokens, float* out, int rows,
-                        int D, int vocab, int packed, float scale, hipStream_t stream) {
+                        int D, int vocab, int packed, float scale, const int* row_pos, const double* freqs,
+                        hipStream_t stream) {
+  LQ_REQUIRE(freqs == nullptr || row_pos != nullptr, "embed: sinusoids need the rows' positions");
   LQ_REQUIRE(rows > 0 && D > 0 && vocab > 0, "embed: rows %d, width %d and table rows %d must be positive", rows, D, vocab);
   LQ_REQUIRE(!packed || (D % 64 == 0 && vocab % 8 == 0), "embed: a packed table has rows in eights and a width in 64s");
   const int threads = D >= 1024 ? 256 : 64;
   if (table_dtype == LQ_BF16 && D % 8 == 0 && D >= 2048 && D <= 8 * 256 * 8 && (uintptr_t)table % 16 == 0 &&
       (uintptr_t)out % 16 == 0) {
     if (D <= 8 * 256 * 2)
-      embed_bf16_vec_kernel<2><<<rows, 256, 0, stream>>>((const bf16_t*)table, tokens, out, D, vocab, packed, scale);
+      embed_bf16_vec_kernel<2><<<rows, 256, 0, stream>>>((const bf16_t*)table, tokens, out, D, vocab, packed, scale, row_pos, freqs);
     else if (D <= 8 * 256 * 4)
-      embed_bf16_vec_kernel<4><<<rows, 256, 0, stream>>>((const bf16_t*)table, tokens, out, D, vocab, packed, scale);
+      embed_bf16_vec_kernel<4><<<rows, 256, 0, stream>>>((const bf16_t*)table, tokens, out, D, vocab, packed, scale, row_pos, freqs);
     else
-      embed_bf16_vec_kernel<8><<<rows, 256, 0, stream>>>((const bf16_t*)table, tokens, out, D, vocab, packed, scale);
+      embed_bf16_vec_kernel<8><<<rows, 256, 0, stream>>>((const bf16_t*)table, tokens, out, D, vocab, packed, scale, row_pos, freqs);
     LQ_CHECK_LAUNCH("embed");
     return 0;
   }
   if (table_dtype == LQ_F32)
-    embed_kernel<float><<<rows, threads, 0, stream>>>((const float*)table, tokens, out, D, vocab, packed, scale);
+    embed_kernel<float><<<rows, threads, 0, stream>>>((const float*)table, tokens, out, D, vocab, packed, scale, row_pos, freqs);
   else if (table_dtype == LQ_BF16)
-    embed_kernel<bf16_t><<<rows, threads, 0, stream>>>((const bf16_t*)table, tokens, out, D, vocab, packed, scale);
+    embed_kernel<bf16_t><<<rows, threads, 0, stream>>>((const bf16_t*)table, tokens, out, D, vocab, packed, scale, row_pos, freqs);
   else
     LQ_REQUIRE(false, "embed: unknown table dtype %d", table_dtype);
   LQ_CHECK_LAUNCH("embed");
@@ -957,6 +990,83 @@ __global__ __launch_bounds__(256) void rmsnorm_residual_kernel(float* __restrict
     if (rounded != nullptr) rounded[base + i] = from_f32<T>(v);
   }
 }
+
+// x[r, :] += N(y[r, :]) with N(y) = y / sqrt(mean(y^2) + eps) * w; rounded as above; a row is read once and kept in
+// registers (PER runs of four columns a thread).  With `n_in` branches that have weights of their own, y is their mean,
+// each normed first: y = (1 / n) sum_i N_i(y_i + b_i), with branch_eps (mixers side by side whose result is normed again).
+struct Branches {
+  const float* y[4];
+  const float* w[4];  // (null: one branch, taken as it is)
+  const float* b[4];  // null: no bias
+};
+
+template <typename T, int PER>
+__global__ __launch_bounds__(256) void branches_residual_kernel(float* __restrict__ x, Branches in, int n_in, float branch_eps,
+                                                                const float* __restrict__ w, float eps,
+                                                                T* __restrict__ rounded, int width) {
+  __shared__ float red[16];
+  const long long base = (long long)blockIdx.x * width;
+  const int quads = width / 4;
+  embed_f32x4 xv[PER], y[PER], one[PER];
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int q = threadIdx.x + i * 256;
+    one[i] = q < quads ? ((const embed_f32x4*)(in.y[0] + base))[q] : (embed_f32x4){0.f, 0.f, 0.f, 0.f};
+  }
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int q = threadIdx.x + i * 256;
+    xv[i] = q < quads ? ((const embed_f32x4*)(x + base))[q] : (embed_f32x4){0.f, 0.f, 0.f, 0.f};
+    y[i] = one[i];
+  }
+  if (in.w[0] != nullptr) {
+    const float share = 1.f / (float)n_in;
+    for (int p = 0; p < n_in; ++p) {
+      float ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < PER; ++i) {
+        const int q = threadIdx.x + i * 256;
+        if (p > 0) one[i] = q < quads ? ((const embed_f32x4*)(in.y[p] + base))[q] : (embed_f32x4){0.f, 0.f, 0.f, 0.f};
+        if (in.b[p] != nullptr && q < quads) one[i] += ((const embed_f32x4*)in.b[p])[q];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss = fmaf(one[i][e], one[i][e], ss);
+      }
+      const float inv = share / sqrtf(block_sum(ss, red) / (float)width + branch_eps);
+#pragma unroll
+      for (int i = 0; i < PER; ++i) {
+        const int q = threadIdx.x + i * 256;
+        if (q < quads) {
+          const embed_f32x4 wv = ((const embed_f32x4*)in.w[p])[q];
+          y[i] = p == 0 ? one[i] * inv * wv : y[i] + one[i] * inv * wv;
+        }
+      }
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < PER; ++i)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss = fmaf(y[i][e], y[i][e], ss);
+  const float inv = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int q = threadIdx.x + i * 256;
+    if (q >= quads) continue;
+    const embed_f32x4 v = xv[i] + y[i] * inv * ((const embed_f32x4*)w)[q];
+    ((embed_f32x4*)(x + base))[q] = v;
+    if (rounded != nullptr) {
+      if constexpr (sizeof(T) == 2) {
+        uint2 packed;
+        packed.x = (uint32_t)f32_to_bf16(v[0]).bits | ((uint32_t)f32_to_bf16(v[1]).bits << 16);
+        packed.y = (uint32_t)f32_to_bf16(v[2]).bits | ((uint32_t)f32_to_bf16(v[3]).bits << 16);
+        ((uint2*)(rounded + base))[q] = packed;
+      } else {
+        ((embed_f32x4*)(rounded + base))[q] = v;
+      }
+    }
+  }
+}
+
 // The norm on a sublayer's result and the norm ahead of the next sublayer in one pass over a row:
 //   y = sum_i scale_i piece_i;   x += y / sqrt(mean(y^2) + eps) * w;   (x += extra;)
 //   (h = x / sqrt(mean(x^2) + next_eps) * next_w, in the next reader's dtype.)
@@ -1084,10 +1194,79 @@ extern "C" int lq_bigram_add(float* x, const void* table, int table_dtype, const
   return 0;
 }
 
+__global__ __launch_bounds__(256) void add_bias_kernel(float* __restrict__ x, const float* __restrict__ b, int width) {
+  float* row = x + (long long)blockIdx.x * width;
+  for (int i = threadIdx.x; i < width; i += 256) row[i] += b[i];
+}
+
+// x [rows, width] dense: x[r, :] += b
+extern "C" int lq_add_bias(float* x, const float* b, int rows, int width, hipStream_t stream) {
+  LQ_REQUIRE(x && b && rows > 0 && width > 0, "add_bias: rows %d, width %d", rows, width);
+  add_bias_kernel<<<rows, 256, 0, stream>>>(x, b, width);
+  LQ_CHECK_LAUNCH("add_bias");
+  return 0;
+}
+
+// Rows that `branches_residual_kernel` takes: their columns in fours on 16 bytes, up to 8 192 of them.
+static bool branches_fit(const float* x, const void* rounded, int rounded_dtype, int width) {
+  return width % 4 == 0 && width <= 8192 && (uintptr_t)x % 16 == 0 &&
+         (uintptr_t)rounded % (rounded_dtype == LQ_F32 ? 16 : 8) == 0;
+}
+
+static int launch_branches(float* x, const Branches& in, int n_in, float branch_eps, const float* w, float eps, void* rounded,
+                           int rounded_dtype, int rows, int width, hipStream_t stream) {
+  const int per = lq_ceil_div(width / 4, 256);
+#define LQ_BRANCHES(T, PER)                                                                                                \
+  branches_residual_kernel<T, PER><<<rows, 256, 0, stream>>>(x, in, n_in, branch_eps, w, eps, (T*)rounded, width)
+#define LQ_BRANCHES_T(T)                          \
+  do {                                            \
+    if (per <= 1) LQ_BRANCHES(T, 1);              \
+    else if (per <= 2) LQ_BRANCHES(T, 2);         \
+    else if (per <= 4) LQ_BRANCHES(T, 4);         \
+    else LQ_BRANCHES(T, 8);                       \
+  } while (0)
+  if (rounded == nullptr || rounded_dtype == LQ_F32) LQ_BRANCHES_T(float);
+  else if (rounded_dtype == LQ_BF16) LQ_BRANCHES_T(bf16_t);
+  else LQ_REQUIRE(false, "rmsnorm_residual: unknown dtype %d", rounded_dtype);
+#undef LQ_BRANCHES_T
+#undef LQ_BRANCHES
+  LQ_CHECK_LAUNCH("rmsnorm_residual");
+  return 0;
+}
+
+// stack [n_in, rows, width] dense float32; x += N(mean of the normed branches), see the kernel.  Widths the kernel does
+// not take are refused (the caller runs lq_rmsnorm_mean and lq_rmsnorm_residual).
+extern "C" int lq_mean_residual_accepts(int width) { return width % 4 == 0 && width <= 8192; }
+
+extern "C" int lq_mean_residual(float* x, const float* stack, int n_in, const float* w0, const float* w1, const float* w2,
+                                const float* w3, const float* b0, const float* b1, const float* b2, const float* b3,
+                                float branch_eps, const float* w, float eps, void* rounded, int rounded_dtype, int rows,
+                                int width, hipStream_t stream) {
+  LQ_REQUIRE(rows > 0 && n_in >= 1 && n_in <= 4 && width > 0, "mean_residual: %d branches of %d x %d", n_in, rows, width);
+  LQ_REQUIRE(x && stack && w, "mean_residual: null pointer");
+  const float* ws[4] = {w0, w1, w2, w3};
+  const float* bs[4] = {b0, b1, b2, b3};
+  Branches in;
+  for (int i = 0; i < 4; ++i) {
+    in.y[i] = i < n_in ? stack + (long long)i * rows * width : nullptr;
+    in.w[i] = i < n_in ? ws[i] : nullptr, in.b[i] = i < n_in ? bs[i] : nullptr;
+    LQ_REQUIRE(i >= n_in || (ws[i] != nullptr && (uintptr_t)ws[i] % 16 == 0 && (uintptr_t)bs[i] % 16 == 0),
+               "mean_residual: branch %d has no weight, or one off 16 bytes", i);
+  }
+  LQ_REQUIRE(branches_fit(x, rounded, rounded_dtype, width) && (uintptr_t)stack % 16 == 0 && (uintptr_t)w % 16 == 0,
+             "mean_residual: columns in fours on 16 bytes, at most 8192 of them");
+  return launch_branches(x, in, n_in, branch_eps, w, eps, rounded, rounded_dtype, rows, width, stream);
+}
+
 extern "C" int lq_rmsnorm_residual(float* x, const float* y, const float* w, float eps, void* rounded, int rounded_dtype,
                                    int rows, int width, hipStream_t stream) {
   LQ_REQUIRE(rows > 0 && width > 0, "rmsnorm_residual: rows %d and width %d must be positive", rows, width);
   LQ_REQUIRE(x && y && w, "rmsnorm_residual: null pointer");
+  if (branches_fit(x, rounded, rounded_dtype, width) && (uintptr_t)y % 16 == 0 && (uintptr_t)w % 16 == 0) {
+    Branches in = {};
+    in.y[0] = y;
+    return launch_branches(x, in, 1, 0.f, w, eps, rounded, rounded_dtype, rows, width, stream);
+  }
   if (rounded == nullptr || rounded_dtype == LQ_F32)
     rmsnorm_residual_kernel<float><<<rows, 256, 0, stream>>>(x, y, w, eps, (float*)rounded, width);
   else if (rounded_dtype == LQ_BF16)

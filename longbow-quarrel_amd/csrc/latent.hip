@@ -118,6 +118,75 @@ __global__ __launch_bounds__(256) void rotary_qkv_kernel(const float* __restrict
   for (int e = blockIdx.y * blockDim.x + threadIdx.x; e < VW; e += blockDim.x * gridDim.y) vo[e] = from_f32<T>(vs[e]);
 }
 
+// Queries, keys and values of a step's rows without a rotation, from the 32-bit result of their one product to what the
+// attention kernel reads and straight into the paged cache.  src [rows, H D + G D (+ G V)]; `bias` (a number a column, or
+// null) is added first.  q and k are normed in units of `unit_q` and `unit_k` entries (a head each, or the whole row of
+// all heads; units divided by their root mean square, eps inside the root, times a weight of the unit's size), values in
+// units of a head without a weight (`norm_v`) or not at all; `v_from_k`: there are no value columns, the values are the
+// keys as they are before their norm.  k and v go to the row's position in the cache (K [block][G][BS][D],
+// V [block][G][V][BS]); kcache null: q alone is wanted.  A wavefront takes a unit (WIDE: a workgroup), so a unit's sum of
+// squares is one fixed tree whatever else is in the launch.
+struct QkvUnits {
+  int lds, ldq, H, G, D, V, unit_q, unit_k, norm_qk, norm_v, v_from_k;
+  float eps;
+  const float *bias, *wq, *wk;
+  const int *row_pos, *row_seq, *seq_slot, *block_table;
+  int bt_stride, BS;
+};
+
+template <typename T, bool WIDE>
+__global__ __launch_bounds__(256) void qkv_norm_store_kernel(const float* __restrict__ src, T* __restrict__ q_out,
+                                                             T* __restrict__ kcache, T* __restrict__ vcache, QkvUnits a) {
+  __shared__ float red[16];
+  const int r = blockIdx.x;
+  const int i0 = WIDE ? threadIdx.x : threadIdx.x & 63;
+  constexpr int STEP = WIDE ? 256 : 64;
+  int u = WIDE ? (int)blockIdx.y : (int)blockIdx.y * 4 + (int)(threadIdx.x >> 6);
+  const int QW = a.H * a.D, KW = a.G * a.D, VW = a.G * a.V, unit_v = a.norm_v ? a.V : VW;
+  const int nq = QW / a.unit_q, nk = kcache != nullptr ? KW / a.unit_k : 0, nv = kcache != nullptr ? VW / unit_v : 0;
+  if (u >= nq + nk + nv) return;  // (WIDE: the whole workgroup)
+  const int which = u < nq ? 0 : u < nq + nk ? 1 : 2;
+  int n, at, col;  // the unit's entries, its first entry among its kind, its first column in src
+  const float* w = nullptr;
+  bool norm = a.norm_qk != 0;
+  if (which == 0) n = a.unit_q, at = u * n, col = at, w = a.wq;
+  else if (which == 1) n = a.unit_k, at = (u - nq) * n, col = QW + at, w = a.wk;
+  else n = unit_v, at = (u - nq - nk) * n, col = (a.v_from_k ? QW : QW + KW) + at, norm = a.norm_v != 0;
+  const float* s = src + (long long)r * a.lds + col;
+  const float* b = a.bias != nullptr ? a.bias + col : nullptr;
+  float inv = 1.f;
+  if (norm) {
+    float ss = 0.f;
+    for (int i = i0; i < n; i += STEP) {
+      const float v = b != nullptr ? s[i] + b[i] : s[i];
+      ss = fmaf(v, v, ss);
+    }
+    inv = 1.f / sqrtf((WIDE ? block_sum(ss, red) : wave_sum(ss)) / (float)n + a.eps);
+  }
+  long long blk = 0;
+  int off = 0;
+  if (which != 0) {
+    const int p = a.row_pos[r];
+    blk = a.block_table[(long long)a.seq_slot[a.row_seq[r]] * a.bt_stride + p / a.BS];
+    off = p % a.BS;
+  }
+  for (int i = i0; i < n; i += STEP) {
+    float v = b != nullptr ? s[i] + b[i] : s[i];
+    if (norm) v *= inv;
+    if (w != nullptr) v *= w[i];
+    const int e = at + i;
+    if (which == 0) {
+      q_out[(long long)r * a.ldq + e] = from_f32<T>(v);
+    } else if (which == 1) {
+      const int g = e / a.D;
+      kcache[((blk * a.G + g) * a.BS + off) * (long long)a.D + e - g * a.D] = from_f32<T>(v);
+    } else {
+      const int g = e / a.V;
+      vcache[((blk * a.G + g) * (long long)a.V + e - g * a.V) * a.BS + off] = from_f32<T>(v);
+    }
+  }
+}
+
 // A product a head: out[r, h ohs + n] = sum_k x[r, h K + k] w[h, n, k], bfloat16 operands on
 // v_mfma_f32_16x16x16_bf16 (exact products, 32-bit sums).  A workgroup of four wavefronts takes 64 rows by 64
 // columns of one head; a wavefront 16 rows by the 64 columns, its operands straight from memory (a head's weight
@@ -222,6 +291,43 @@ extern "C" int lq_rotary_qkv(const float* src, int lds_, void* q_out, int ldq, v
                                                                 interleaved, freqs, magnitude, norm_eps, row_pos);
   else LQ_REQUIRE(false, "rotary_qkv: unknown dtype %d", out_dtype);
   LQ_CHECK_LAUNCH("rotary_qkv");
+  return 0;
+}
+
+// bias: null or a number for every column of src; wq, wk: weights of unit_q and unit_k entries, or null (with
+// `norm_qk` off: no norm of q and k); kcache and vcache null: q alone.
+extern "C" int lq_qkv_norm_store(const float* src, int lds_, const float* bias, const float* wq, const float* wk, int unit_q,
+                                 int unit_k, int norm_qk, int norm_v, int v_from_k, float eps, void* q_out, int ldq, int dtype,
+                                 int rows, int heads, int kv_heads, int key_dim, int value_dim, const int* row_pos,
+                                 const int* row_seq, const int* seq_slot, const int* block_table, int bt_stride, void* kcache,
+                                 void* vcache, int block_size, hipStream_t stream) {
+  LQ_REQUIRE(rows > 0 && rows <= 0x7fffffff && heads > 0 && kv_heads > 0 && key_dim > 0 && value_dim > 0,
+             "qkv_norm_store: rows %d, heads %d and %d, sizes %d and %d", rows, heads, kv_heads, key_dim, value_dim);
+  LQ_REQUIRE(!v_from_k || key_dim == value_dim, "qkv_norm_store: values that are the keys have their size (%d, %d)", key_dim, value_dim);
+  const int QW = heads * key_dim, KW = kv_heads * key_dim, VW = kv_heads * value_dim;
+  LQ_REQUIRE(unit_q > 0 && unit_k > 0 && QW % unit_q == 0 && KW % unit_k == 0, "qkv_norm_store: units of %d and %d entries", unit_q, unit_k);
+  LQ_REQUIRE(lds_ >= QW + KW + (v_from_k ? 0 : VW) && ldq >= QW, "qkv_norm_store: a row stride is smaller than its row");
+  LQ_REQUIRE(src && q_out && (kcache == nullptr) == (vcache == nullptr), "qkv_norm_store: null pointer");
+  LQ_REQUIRE(kcache == nullptr || (row_pos && row_seq && seq_slot && block_table && block_size > 0 && bt_stride > 0),
+             "qkv_norm_store: the cache needs the rows' places");
+  LQ_REQUIRE(norm_qk || (wq == nullptr && wk == nullptr), "qkv_norm_store: weights without a norm");
+  QkvUnits a = {lds_, ldq, heads, kv_heads, key_dim, value_dim, unit_q, unit_k, norm_qk, norm_v, v_from_k,
+                eps, bias, wq, wk, row_pos, row_seq, seq_slot, block_table, bt_stride, block_size};
+  const int units = QW / unit_q + (kcache ? KW / unit_k + (norm_v ? kv_heads : 1) : 0);
+  const bool wide = unit_q > 512 || unit_k > 512 || (kcache && !norm_v && VW > 512);
+  const int gy = wide ? units : lq_ceil_div(units, 4);
+  LQ_REQUIRE(gy <= 65535, "qkv_norm_store: too many heads");
+  const dim3 grid(rows, gy);
+#define LQ_QKV(T)                                                                                                    \
+  do {                                                                                                               \
+    if (wide) qkv_norm_store_kernel<T, true><<<grid, 256, 0, stream>>>(src, (T*)q_out, (T*)kcache, (T*)vcache, a);   \
+    else qkv_norm_store_kernel<T, false><<<grid, 256, 0, stream>>>(src, (T*)q_out, (T*)kcache, (T*)vcache, a);       \
+  } while (0)
+  if (dtype == LQ_F32) LQ_QKV(float);
+  else if (dtype == LQ_BF16) LQ_QKV(bf16_t);
+  else LQ_REQUIRE(false, "qkv_norm_store: unknown dtype %d", dtype);
+#undef LQ_QKV
+  LQ_CHECK_LAUNCH("qkv_norm_store");
   return 0;
 }
 

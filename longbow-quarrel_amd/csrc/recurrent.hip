@@ -7,37 +7,9 @@
 // The scans walk a sequence's tokens in order, one workgroup a (sequence, head, slice of the head's columns),
 // the state in registers, and are the same kernel for a prompt and for single tokens: a token's result is made of
 // the same operations in the same order however the sequence was cut into steps and whatever else is in the batch.
-#include "common.h"
+#include "device_math.h"
 
 namespace {
-
-__device__ inline float softplus_f(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
-__device__ inline float silu_f(float z) { return z / (1.f + expf(-z)); }
-__device__ inline float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
-__device__ inline float gelu_tanh_f(float z) {
-  return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-}
-
-__device__ inline float gelu_erf_f(float z) { return 0.5f * z * (1.f + erff(z * 0.70710678118654752f)); }
-
-enum { ACT_NONE = 0, ACT_SILU = 1, ACT_RELU = 2, ACT_GELU_TANH = 3, ACT_GELU_ERF = 4 };
-
-__device__ inline float activate(float z, int act) {
-  switch (act) {
-    case ACT_SILU: return silu_f(z);
-    case ACT_RELU: return fmaxf(z, 0.f);
-    case ACT_GELU_TANH: return gelu_tanh_f(z);
-    case ACT_GELU_ERF: return gelu_erf_f(z);
-    default: return z;
-  }
-}
-
-template <typename T>
-__device__ inline void store_as(T* p, float v);
-template <>
-__device__ inline void store_as<float>(float* p, float v) { *p = v; }
-template <>
-__device__ inline void store_as<bf16_t>(bf16_t* p, float v) { *p = f32_to_bf16(v); }
 
 // ---------------------------------------------------------------- Dynamic Tanh and the scaled add
 // (x += scale * (piece 0 + piece 1 + ...);)  out = tanh(alpha x) w + b
@@ -114,9 +86,10 @@ __global__ __launch_bounds__(256) void activation4_kernel(const float* __restric
 // ---------------------------------------------------------------- short causal convolution
 // y[t, c] = act(bias[c] + sum_j w[c, j] x[t - (taps - 1) + j, c]); inputs before this step's rows come from
 // the sequence's state (its last taps - 1 inputs, zeros at the start of a sequence).
-__global__ __launch_bounds__(256) void causal_conv_kernel(const float* __restrict__ x, int ldx,
+template <typename T>
+__global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ x, int ldx,
                                                           const float* __restrict__ w, const float* __restrict__ bias,
-                                                          const float* __restrict__ state, float* __restrict__ out,
+                                                          const float* __restrict__ state, T* __restrict__ out,
                                                           int ldo, int C, int taps, const int* __restrict__ row_seq,
                                                           const int* __restrict__ row_pos,
                                                           const int* __restrict__ seq_slot,
@@ -132,15 +105,16 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const float* __restric
   float acc = 0.f;
   for (int j = 0; j < taps; ++j) {
     const int back = taps - 1 - j;  // how many tokens before this one
-    const float v = back <= since ? x[(first + since - back) * ldx + c] : st[(long long)(taps - 1 - (back - since)) * C + c];
+    const float v = back <= since ? to_f32(x[(first + since - back) * ldx + c]) : st[(long long)(taps - 1 - (back - since)) * C + c];
     acc = fmaf(w[(long long)c * taps + j], v, acc);
   }
   if (bias != nullptr) acc += bias[c];
-  out[(long long)r * ldo + c] = activate(acc, act);
+  store_as<T>(out + (long long)r * ldo + c, activate(acc, act));
 }
 
 // The state after the step: the last taps - 1 inputs of each sequence (old ones move up where the step brought fewer).
-__global__ __launch_bounds__(256) void conv_state_kernel(const float* __restrict__ x, int ldx, float* __restrict__ state,
+template <typename T>
+__global__ __launch_bounds__(256) void conv_state_kernel(const T* __restrict__ x, int ldx, float* __restrict__ state,
                                                          int C, int taps, const int* __restrict__ seq_slot,
                                                          const int* __restrict__ cu_rows) {
   const int b = blockIdx.y;
@@ -151,7 +125,7 @@ __global__ __launch_bounds__(256) void conv_state_kernel(const float* __restrict
   float* st = state + (long long)seq_slot[b] * (taps - 1) * C;
   for (int j = 0; j < taps - 1; ++j) {  // ascending: entry j is written after entry j + n_new was read
     const int src = j + n_new;
-    st[(long long)j * C + c] = src < taps - 1 ? st[(long long)src * C + c] : x[(first + src - (taps - 1)) * ldx + c];
+    st[(long long)j * C + c] = src < taps - 1 ? st[(long long)src * C + c] : to_f32(x[(first + src - (taps - 1)) * ldx + c]);
   }
 }
 
@@ -164,23 +138,6 @@ __global__ __launch_bounds__(256) void conv_state_kernel(const float* __restrict
 // buffers taking turns: the next chunk's loads are in flight while this chunk is computed.
 constexpr int PRE = 16;        // registers a thread lends to a chunk's loads of the shared rows
 constexpr int MAX_CHUNK = 16;  // tokens a chunk at most
-
-template <int CTRL>
-__device__ inline float dpp_swap(float v) {
-  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, false));
-}
-
-// the sum over the LN lanes of a column; every lane gets it
-template <int LN>
-__device__ inline float group_sum(float v) {
-  if (LN >= 2) v += dpp_swap<0xB1>(v);    // lanes 1 apart (quad_perm [1,0,3,2])
-  if (LN >= 4) v += dpp_swap<0x4E>(v);    // 2 apart (quad_perm [2,3,0,1])
-  if (LN >= 8) v += dpp_swap<0x141>(v);   // the other quad of eight lanes (row_half_mirror)
-  if (LN >= 16) v += dpp_swap<0x140>(v);  // the other half of sixteen (row_mirror)
-  if (LN >= 32) v += __shfl_xor(v, 16, LQ_WAVE);
-  if (LN >= 64) v += __shfl_xor(v, 32, LQ_WAVE);
-  return v;
-}
 
 // A launch of the state-space scan in segments, for few long sequences that would leave most of the chip idle: a
 // sequence of SEG_MIN_ROWS rows or more is cut into `nseg` segments (whole chunks), one workgroup each.  Pass 1: segment
@@ -198,6 +155,10 @@ struct SegArgs {
 struct ScanShape {
   int heads, groups, P, N;  // groups: of the shared rows (state-space groups, q/k heads)
   const int *seq_slot, *cu_rows;
+  // the state-space scan alone: a token's decay and step are given ([rows, heads] each: `decay`, and dt as it is), not
+  // made of a logit; `ones`: the head's last column is not in x ([rows, heads * (P - 1)]), its input is one
+  const float* decay = nullptr;
+  int lddecay = 0, ones = 0;
 };
 
 // The chunk-wise staging that both scans share.  `a`, `b`: the two shared rows of a token ([rows, groups * N] each),
@@ -223,7 +184,7 @@ __global__ __launch_bounds__(TH) void ssd_scan_kernel(const float* __restrict__ 
                                                        const float* __restrict__ d_skip, float* __restrict__ state,
                                                        float* __restrict__ y, int ldy, ScanShape sh, SegArgs sg) {
   extern __shared__ float lds[];
-  const int heads = sh.heads, P = sh.P, N = sh.N;
+  const int heads = sh.heads, P = sh.P, N = sh.N, Px = P - sh.ones;
   constexpr int TT = Stage<LN, SLAB, TH>::TT, PER = Stage<LN, SLAB, TH>::PER;
   const int b = blockIdx.x / heads, h = blockIdx.x % heads, g = h / (heads / sh.groups);
   const int threads = blockDim.x, cols = threads / LN, tid = threadIdx.x;
@@ -256,7 +217,8 @@ __global__ __launch_bounds__(TH) void ssd_scan_kernel(const float* __restrict__ 
     const int n = i * LN + l;
     S[i] = (live && !from_zero && i < slab && n < N) ? from[n] : 0.f;
   }
-  const float A = -expf(a_log[h]), bias = dt_bias[h], D = d_skip[h];
+  const bool given = sh.decay != nullptr;
+  const float A = given ? 0.f : -expf(a_log[h]), bias = given ? 0.f : dt_bias[h], D = given ? 0.f : d_skip[h];
   Stage<LN, SLAB, TH> st;
 
   auto fetch = [&](long long c0, int nt) {  // the chunk's loads, into registers
@@ -273,10 +235,13 @@ __global__ __launch_bounds__(TH) void ssd_scan_kernel(const float* __restrict__ 
       const int e = tid + i * threads;
       if (e < nt * cols) {
         const int t = e / cols, c = e - t * cols;
-        st.xs[i] = p0 + c < P ? x[(c0 + t) * ldx + h * P + p0 + c] : 0.f;
+        st.xs[i] = p0 + c < Px ? x[(c0 + t) * ldx + h * Px + p0 + c] : p0 + c < P ? 1.f : 0.f;
       }
     }
-    if (tid < nt) st.s0 = dt[(c0 + tid) * lddt + h];
+    if (tid < nt) {
+      st.s0 = dt[(c0 + tid) * lddt + h];
+      if (given) st.s1 = sh.decay[(c0 + tid) * sh.lddecay + h];
+    }
   };
   auto stash = [&](float* buf, int nt) {  // registers to LDS
 #pragma unroll
@@ -292,8 +257,8 @@ __global__ __launch_bounds__(TH) void ssd_scan_kernel(const float* __restrict__ 
       if (e < nt * cols) buf[TT * 2 * NP + e] = st.xs[i];
     }
     if (tid < nt) {
-      const float step = softplus_f(st.s0 + bias);
-      buf[TT * (2 * NP + cols) + 2 * tid] = expf(A * step);
+      const float step = given ? st.s0 : softplus_f(st.s0 + bias);
+      buf[TT * (2 * NP + cols) + 2 * tid] = given ? st.s1 : expf(A * step);
       buf[TT * (2 * NP + cols) + 2 * tid + 1] = step;
     }
   };
@@ -932,9 +897,10 @@ __global__ void gated_rmsnorm_kernel(const float* __restrict__ y, int ldy, const
 struct MeanInputs {
   const float* x[4];
   const float* w[4];
+  const float* b[4];  // null: none
 };
 
-// out = (1 / n) sum_i x_i / rms(x_i) w_i, row by row.  The branches' sums of squares are taken in one pass (their
+// out = (1 / n) sum_i x_i / rms(x_i) w_i, row by row (a branch with a bias: x_i + b_i in the place of x_i).  The branches' sums of squares are taken in one pass (their
 // loads are in flight together), each with the block's fixed tree.
 __global__ void rmsnorm_mean_kernel(MeanInputs in, int n_in, float eps, float* __restrict__ out, int width) {
   __shared__ float red[16];
@@ -943,7 +909,8 @@ __global__ void rmsnorm_mean_kernel(MeanInputs in, int n_in, float eps, float* _
   for (int c = threadIdx.x; c < width; c += blockDim.x) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const float v = i < n_in ? in.x[i][r * width + c] : 0.f;
+      float v = i < n_in ? in.x[i][r * width + c] : 0.f;
+      if (i < n_in && in.b[i] != nullptr) v += in.b[i][c];
       ss[i] = fmaf(v, v, ss[i]);
     }
   }
@@ -955,7 +922,7 @@ __global__ void rmsnorm_mean_kernel(MeanInputs in, int n_in, float eps, float* _
     float acc = 0.f;
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-      if (i < n_in) acc += in.x[i][r * width + c] * inv[i] * in.w[i][c];
+      if (i < n_in) acc += (in.b[i] != nullptr ? in.x[i][r * width + c] + in.b[i][c] : in.x[i][r * width + c]) * inv[i] * in.w[i][c];
     out[r * width + c] = acc * share;
   }
 }
@@ -1060,12 +1027,30 @@ extern "C" int lq_glu(const void* gu, int in_dtype, int ld, void* out, int out_d
   return 0;
 }
 
-// x [rows, C] (stride ldx), w [C, taps], bias [C] or null, state [slots, taps - 1, C]; out [rows, C] (stride ldo).
-// The state is read for the step's outputs and then moved on by a second launch.
-extern "C" int lq_causal_conv(const float* x, int ldx, const float* w, const float* bias, float* state, float* out,
+template <typename T>
+static int launch_causal_conv(const T* x, int ldx, const float* w, const float* bias, float* state, T* out, int ldo, int rows,
+                              int C, int taps, const int* row_seq, const int* row_pos, const int* seq_slot,
+                              const int* seq_start, const int* cu_rows, int batch, int act, hipStream_t stream) {
+  for (int r0 = 0; r0 < rows; r0 += 65535) {
+    const int nr = rows - r0 < 65535 ? rows - r0 : 65535;
+    causal_conv_kernel<T><<<dim3(lq_ceil_div(C, 256), nr), 256, 0, stream>>>(
+        x, ldx, w, bias, state, out + (long long)r0 * ldo, ldo, C, taps, row_seq + r0, row_pos + r0, seq_slot, seq_start,
+        cu_rows, act);
+  }
+  LQ_CHECK_LAUNCH("causal_conv");
+  if (taps > 1) {
+    conv_state_kernel<T><<<dim3(lq_ceil_div(C, 256), batch), 256, 0, stream>>>(x, ldx, state, C, taps, seq_slot, cu_rows);
+    LQ_CHECK_LAUNCH("causal_conv(state)");
+  }
+  return 0;
+}
+
+// x [rows, C] (stride ldx), w [C, taps], bias [C] or null, state [slots, taps - 1, C] (32-bit); out [rows, C] (stride
+// ldo); x and out of one dtype.  The state is read for the step's outputs and then moved on by a second launch.
+extern "C" int lq_causal_conv(const void* x, int ldx, const float* w, const float* bias, float* state, void* out,
                               int ldo, int rows, int C, int taps, const int* row_seq, const int* row_pos,
                               const int* seq_slot, const int* seq_start, const int* cu_rows, int batch, int act,
-                              hipStream_t stream) {
+                              int dtype, hipStream_t stream) {
   LQ_REQUIRE(rows > 0 && C > 0 && taps >= 1 && batch > 0, "causal_conv: rows %d, channels %d, taps %d, sequences %d", rows, C,
              taps, batch);
   LQ_REQUIRE(ldx >= C && ldo >= C, "causal_conv: a row stride is smaller than its row");
@@ -1073,18 +1058,12 @@ extern "C" int lq_causal_conv(const float* x, int ldx, const float* w, const flo
              "causal_conv: null pointer");
   LQ_REQUIRE(act >= ACT_NONE && act <= ACT_GELU_TANH, "causal_conv: unknown activation %d", act);
   LQ_REQUIRE(batch <= 65535, "causal_conv: too many sequences");
-  for (int r0 = 0; r0 < rows; r0 += 65535) {
-    const int nr = rows - r0 < 65535 ? rows - r0 : 65535;
-    causal_conv_kernel<<<dim3(lq_ceil_div(C, 256), nr), 256, 0, stream>>>(
-        x, ldx, w, bias, state, out + (long long)r0 * ldo, ldo, C, taps, row_seq + r0, row_pos + r0, seq_slot, seq_start,
-        cu_rows, act);
-  }
-  LQ_CHECK_LAUNCH("causal_conv");
-  if (taps > 1) {
-    conv_state_kernel<<<dim3(lq_ceil_div(C, 256), batch), 256, 0, stream>>>(x, ldx, state, C, taps, seq_slot, cu_rows);
-    LQ_CHECK_LAUNCH("causal_conv(state)");
-  }
-  return 0;
+  LQ_REQUIRE(dtype == LQ_F32 || dtype == LQ_BF16, "causal_conv: unknown dtype %d", dtype);
+  if (dtype == LQ_F32)
+    return launch_causal_conv<float>((const float*)x, ldx, w, bias, state, (float*)out, ldo, rows, C, taps, row_seq, row_pos,
+                                     seq_slot, seq_start, cu_rows, batch, act, stream);
+  return launch_causal_conv<bf16_t>((const bf16_t*)x, ldx, w, bias, state, (bf16_t*)out, ldo, rows, C, taps, row_seq, row_pos,
+                                    seq_slot, seq_start, cu_rows, batch, act, stream);
 }
 
 #define LQ_SCAN_TH(LAUNCH, LN, SL)                                 \
@@ -1120,14 +1099,20 @@ extern "C" long long lq_ssd_scan_workspace(int batch, int heads, int P, int N, i
 // x [rows, heads * P], B and C [rows, groups * N], dt [rows, heads] (before its softplus), state
 // [slots, heads, P, N], y [rows, heads * P]; rows lie sequence by sequence (cu_rows).  `max_rows`: the most rows a
 // sequence brings (0: unknown); `scratch`: lq_ssd_scan_workspace(...) floats, or null (then no segments).
+// `decay` [rows, heads] (or null): a token's decay and step are given, S <- decay S + dt B x^T, y = S^T C; dt_bias, a_log
+// and d_skip are then null.  `ones`: x is [rows, heads * (P - 1)], and a head's last column has the input one.
 extern "C" int lq_ssd_scan(const float* x, int ldx, const float* Bm, int ldb, const float* Cm, int ldc, const float* dt,
                            int lddt, const float* dt_bias, const float* a_log, const float* d_skip, float* state, float* y,
                            int ldy, int heads, int P, int N, int groups, const int* seq_slot, const int* cu_rows, int batch,
-                           int max_rows, float* scratch, long long scratch_floats, hipStream_t stream) {
+                           int max_rows, float* scratch, long long scratch_floats, const float* decay, int lddecay, int ones,
+                           hipStream_t stream) {
   LQ_REQUIRE(heads > 0 && P > 0 && N > 0 && groups > 0 && heads % groups == 0 && batch > 0, "ssd_scan: bad sizes");
-  LQ_REQUIRE(ldx >= heads * P && ldy >= heads * P && ldb >= groups * N && ldc >= groups * N && lddt >= heads,
+  LQ_REQUIRE(ones == 0 || (ones == 1 && P > 1), "ssd_scan: a column of ones beside %d columns", P - 1);
+  LQ_REQUIRE(ldx >= heads * (P - ones) && ldy >= heads * P && ldb >= groups * N && ldc >= groups * N && lddt >= heads &&
+                 (decay == nullptr || lddecay >= heads),
              "ssd_scan: a row stride is smaller than its row");
-  LQ_REQUIRE(x && Bm && Cm && dt && dt_bias && a_log && d_skip && state && y && seq_slot && cu_rows, "ssd_scan: null pointer");
+  LQ_REQUIRE(x && Bm && Cm && dt && state && y && seq_slot && cu_rows, "ssd_scan: null pointer");
+  LQ_REQUIRE(decay != nullptr || (dt_bias && a_log && d_skip), "ssd_scan: neither decays nor what makes them");
   const long long need = scratch != nullptr ? ssd_segment_floats(batch, heads, P, N, max_rows) : 0;
   ScanLaunch cfg;
   LQ_REQUIRE(scan_launch(N, P, (long long)batch * heads * (need > 0 ? SEG_COUNT : 1), cfg),
@@ -1139,7 +1124,7 @@ extern "C" int lq_ssd_scan(const float* x, int ldx, const float* Bm, int ldb, co
     sg.state = scratch;
     sg.decay = scratch + (long long)batch * heads * SEG_COUNT * P * N;
   }
-  ScanShape sh = {heads, groups, P, N, seq_slot, cu_rows};
+  ScanShape sh = {heads, groups, P, N, seq_slot, cu_rows, decay, lddecay, ones};
 #define LQ_SSD(LN, SL, TH)                                                                                              \
   ssd_scan_kernel<LN, SL, TH><<<grid, cfg.threads, cfg.lds, stream>>>(x, ldx, Bm, ldb, Cm, ldc, dt, lddt, dt_bias, a_log, \
                                                                   d_skip, state, y, ldy, sh, sg)
@@ -1230,15 +1215,17 @@ extern "C" int lq_gated_rmsnorm(const float* y, int ldy, const float* z, int ldz
   return 0;
 }
 
-// stack [n_in, rows, width] dense float32; w0..w3 the branches' weights [width]
+// stack [n_in, rows, width] dense float32; w0..w3 the branches' weights [width], b0..b3 their biases [width] or null
 extern "C" int lq_rmsnorm_mean(const float* stack, int n_in, const float* w0, const float* w1, const float* w2,
-                               const float* w3, float eps, float* out, int rows, int width, hipStream_t stream) {
+                               const float* w3, const float* b0, const float* b1, const float* b2, const float* b3,
+                               float eps, float* out, int rows, int width, hipStream_t stream) {
   LQ_REQUIRE(rows > 0 && width > 0 && n_in >= 1 && n_in <= 4, "rmsnorm_mean: %d branches of %d x %d", n_in, rows, width);
   const float* ws[4] = {w0, w1, w2, w3};
+  const float* bs[4] = {b0, b1, b2, b3};
   MeanInputs in;
   for (int i = 0; i < 4; ++i) {
     in.x[i] = i < n_in ? stack + (long long)i * rows * width : nullptr;
-    in.w[i] = ws[i];
+    in.w[i] = ws[i], in.b[i] = bs[i];
     LQ_REQUIRE(i >= n_in || ws[i] != nullptr, "rmsnorm_mean: branch %d has no weight", i);
   }
   LQ_REQUIRE(stack && out, "rmsnorm_mean: null pointer");

@@ -20,7 +20,7 @@ from .. import build as _build
 from .dry import query
 
 F32, BF16 = 0, 1
-ABI_VERSION = 10  # lq_abi_version() of the library these wrappers were written for
+ABI_VERSION = 11  # lq_abi_version() of the library these wrappers were written for
 _DTYPE_CODE = {torch.float32: F32, torch.bfloat16: BF16}
 
 
@@ -224,8 +224,11 @@ class HipKernels:
         self._check(self.lib.lq_pack_weight(_ptr(w), _ptr(out), c_int(n), c_int(k), self.stream))
         return PackedWeight(out, n, k)
 
-    def embed(self, table: torch.Tensor, tokens: torch.Tensor, out: torch.Tensor, scale: float = 1.0) -> None:
-        """out[r, :] = scale * float32(table[tokens[r], :]); zeros where tokens[r] is no row of the table"""
+    def embed(self, table: torch.Tensor, tokens: torch.Tensor, out: torch.Tensor, scale: float = 1.0,
+              row_pos: Optional[torch.Tensor] = None, freqs: Optional[torch.Tensor] = None) -> None:
+        """out[r, :] = scale * float32(table[tokens[r], :]); zeros where tokens[r] is no row of the table.  With `freqs`
+        (float64 [(width + 1) / 2]) a row's position vector is added: column 2 i is the sine, column 2 i + 1 the cosine
+        of row_pos[r] * freqs[i]."""
         self._dev(table, tokens, out)
         rows, width = out.shape
         self._i32(tokens, "embed tokens", rows)
@@ -233,9 +236,15 @@ class HipKernels:
             raise KernelLibraryError("embed: out must be dense float32, the table dense")
         if table.dim() != 2 or table.shape[1] != width:
             raise KernelLibraryError(f"embed: table {tuple(table.shape)} does not match width {width}")
+        if freqs is not None:
+            self._dev(row_pos, freqs)
+            self._i32(row_pos, "embed row_pos", rows)
+            if freqs.dtype != torch.float64 or not freqs.is_contiguous() or freqs.numel() != (width + 1) // 2:
+                raise KernelLibraryError(f"embed: {(width + 1) // 2} float64 frequencies")
         self._check(self.lib.lq_embed(_ptr(table), c_int(_code(table)), _ptr(tokens), _ptr(out),
                                       c_int(rows), c_int(width), c_int(table.shape[0]), c_int(_packed(table)),
-                                      c_float(scale), self.stream))
+                                      c_float(scale), _ptr(row_pos if freqs is not None else None), _ptr(freqs),
+                                      self.stream))
 
     @staticmethod
     def _pieces(delta: Optional[torch.Tensor], like: torch.Tensor, what: str):
@@ -724,7 +733,9 @@ class HipKernels:
                        scale: float, window: int = 0, keep_first: int = 0, sink: bool = True,
                        gate: Optional[torch.Tensor] = None, decode: bool = False, max_len: int = 0,
                        workspace: Optional[torch.Tensor] = None, sink_values: Optional[torch.Tensor] = None,
-                       maps: int = 1) -> None:
+                       maps: int = 1, softcap: float = 0.0, temp: Optional[torch.Tensor] = None,
+                       log_bias: Optional[tuple] = None, distance_bias: Optional[torch.Tensor] = None,
+                       wide_gate: Optional[torch.Tensor] = None) -> None:
         """Attention of the step's rows over their slots' cached keys: row at position p sees t <= p with
         p - t < window (0: all) or t < keep_first; with `sink` the softmax's denominator has one more term e^0;
         `gate` [rows, heads]: every head's result times the sigmoid of its entry.  Scores and probabilities
@@ -734,8 +745,15 @@ class HipKernels:
         e^(its entry) for every query head, not e^0.  `maps` > 1: `kv_heads` counts key heads of which every `maps`
         neighbours share a value head; the cache is K [blocks, kv_heads / maps, block_size, maps * key_dim] (a row
         holds the neighbours' keys side by side) and V [blocks, kv_heads / maps, value_dim, block_size].  out may be
-        float32 in a bfloat16 run."""
-        self._dev(q, out, gate, row_pos, row_seq, seq_slot, block_table, kcache, vcache, sink_values)
+        float32 in a bfloat16 run.
+
+        A score q . k * scale is shaped on its way to the softmax, each step where it is asked for: times `temp`
+        (float32 [heads]); softcap * tanh(score / softcap); minus r1 ln(1 + r2 n) with `log_bias` = (r1, r2) (float32
+        [heads] each), n the distance p - t; plus `distance_bias` [heads, entries] at column min(n, entries - 1).  The
+        sink's score is not shaped.  `wide_gate` float32 [rows, heads * value_dim]: every entry of the result times the
+        sigmoid of its own."""
+        self._dev(q, out, gate, row_pos, row_seq, seq_slot, block_table, kcache, vcache, sink_values, temp, distance_bias,
+                  wide_gate)
         rows, batch = q.shape[0], seq_slot.numel()
         self._i32(row_pos, "row_pos", rows)
         self._i32(row_seq, "row_seq", rows)
@@ -754,6 +772,18 @@ class HipKernels:
             raise KernelLibraryError("sink_attention: the gate is [rows, heads] in the dtype of q")
         if decode and rows != batch:
             raise KernelLibraryError("sink_attention: decode means one row per sequence")
+        r1, r2 = log_bias if log_bias is not None else (None, None)
+        for t, what in ((temp, "temp"), (r1, "r1"), (r2, "r2")):
+            if t is not None:
+                self._f32(t, "sink_attention: " + what, heads)
+        if log_bias is not None and (r1 is None or r2 is None):
+            raise KernelLibraryError("sink_attention: r1 and r2 come together")
+        if distance_bias is not None and (distance_bias.dtype != torch.float32 or not distance_bias.is_contiguous()
+                                          or distance_bias.dim() != 2 or distance_bias.shape[0] != heads
+                                          or distance_bias.shape[1] < 1):
+            raise KernelLibraryError("sink_attention: the bias by distance is dense float32 [heads, entries]")
+        if wide_gate is not None and (tuple(wide_gate.shape) != (rows, heads * value_dim) or wide_gate.dtype != torch.float32):
+            raise KernelLibraryError("sink_attention: the wide gate is float32 [rows, heads * value_dim]")
         if workspace is not None:
             self._f32(workspace, "sink_attention: workspace", workspace.numel())
         self._check(self.lib.lq_sink_attention(
@@ -764,7 +794,9 @@ class HipKernels:
             c_int(block_size), c_float(scale), c_int(window), c_int(keep_first), c_int(1 if sink else 0),
             c_int(1 if self.force_generic else 0), c_int(max_len if workspace is not None else 0), _ptr(workspace),
             c_longlong(0 if workspace is None else workspace.numel()), _ptr(sink_values), c_int(maps),
-            c_int(1 if out.dtype == torch.float32 else 0), self.stream))
+            c_int(1 if out.dtype == torch.float32 else 0), c_float(softcap), _ptr(temp), _ptr(r1), _ptr(r2),
+            _ptr(distance_bias), c_int(0 if distance_bias is None else int(distance_bias.shape[1])), _ptr(wide_gate),
+            c_int(0 if wide_gate is None else self._rows2d(wide_gate, "wide_gate")), self.stream))
 
     def diff_combine(self, both: torch.Tensor, out: torch.Tensor, heads: int, kv_heads: int, value_dim: int, lam: float,
                      eps: float, gain: float) -> None:
@@ -855,12 +887,14 @@ class HipKernels:
                     activation: str = "silu") -> None:
         """out[t, c] = act(bias[c] + sum_j weight[c, j] x[t - (taps - 1) + j, c]) along every sequence of the step;
         what lies before the step's rows comes from state [slots, taps - 1, channels] (a sequence's last inputs,
-        zeros at its start), which is then moved on to the step's end.  All float32."""
+        zeros at its start), which is then moved on to the step's end.  x and out of one dtype, the rest float32."""
         rows, ch, ldx = self._mat(x, "causal_conv: x")
         ro, co, ldo = self._mat(out, "causal_conv: out")
         taps = weight.shape[1] if weight.dim() == 2 else 0
-        for t, what in ((x, "x"), (out, "out"), (state, "state")):
-            self._f32(t, "causal_conv: " + what)
+        self._dev(x, out)
+        self._f32(state, "causal_conv: state")
+        if x.dtype != out.dtype:
+            raise KernelLibraryError("causal_conv: x and out in one dtype")
         self._f32(weight, "causal_conv: weight", ch * max(1, taps))
         if bias is not None:
             self._f32(bias, "causal_conv: bias", ch)
@@ -876,7 +910,7 @@ class HipKernels:
         self._check(self.lib.lq_causal_conv(_ptr(x), c_int(ldx), _ptr(weight), _ptr(bias), _ptr(state), _ptr(out),
                                             c_int(ldo), c_int(rows), c_int(ch), c_int(taps), _ptr(row_seq), _ptr(row_pos),
                                             _ptr(seq_slot), _ptr(seq_start), _ptr(cu_rows), c_int(batch),
-                                            c_int(self._ACTIVATIONS[activation]), self.stream))
+                                            c_int(self._ACTIVATIONS[activation]), c_int(_code(x)), self.stream))
 
     @query
     def ssd_scan_workspace(self, batch: int, heads: int, head_dim: int, n_state: int, max_rows: int) -> int:
@@ -888,19 +922,28 @@ class HipKernels:
     def ssd_scan(self, x: torch.Tensor, b_in: torch.Tensor, c_in: torch.Tensor, dt: torch.Tensor, dt_bias: torch.Tensor,
                  a_log: torch.Tensor, d_skip: torch.Tensor, state: torch.Tensor, y: torch.Tensor, heads: int,
                  head_dim: int, n_state: int, groups: int, seq_slot: torch.Tensor, cu_rows: torch.Tensor,
-                 batch: int, max_rows: int = 0, workspace: Optional[torch.Tensor] = None) -> None:
+                 batch: int, max_rows: int = 0, workspace: Optional[torch.Tensor] = None,
+                 decay: Optional[torch.Tensor] = None, ones: bool = False) -> None:
         """The Mamba-2 recurrence along every sequence of the step, token by token: with dt = softplus(dt + dt_bias),
         S <- exp(-exp(a_log) dt) S + dt B x^T and y = S^T C + d_skip x per head; state [slots, heads, head_dim,
         n_state] is read and left at the step's end.  All float32.  `max_rows` (the most rows a sequence brings)
-        and `workspace` (`ssd_scan_workspace(...)` floats) let a launch of few long sequences run in segments."""
+        and `workspace` (`ssd_scan_workspace(...)` floats) let a launch of few long sequences run in segments.
+        `decay` [rows, heads]: a token's decay and step (`dt` as it is) are given, S <- decay S + dt B x^T, y = S^T C;
+        dt_bias, a_log and d_skip are then None.  `ones`: head_dim counts one column more than x has for a head, the
+        last, whose input is one (its result is the sum of the steps' B under the same decays, times C)."""
         rows = x.shape[0]
-        for t, what, cols in ((x, "x", heads * head_dim), (b_in, "B", groups * n_state), (c_in, "C", groups * n_state),
+        for t, what, cols in ((x, "x", heads * (head_dim - (1 if ones else 0))), (b_in, "B", groups * n_state), (c_in, "C", groups * n_state),
                               (dt, "dt", heads), (y, "y", heads * head_dim)):
             self._f32(t, "ssd_scan: " + what)
             if self._mat(t, "ssd_scan: " + what)[:2] != (rows, cols):
                 raise KernelLibraryError(f"ssd_scan: {what} must be [{rows}, {cols}], found {tuple(t.shape)}")
-        for t, what in ((dt_bias, "dt_bias"), (a_log, "a_log"), (d_skip, "d_skip")):
-            self._f32(t, "ssd_scan: " + what, heads)
+        if decay is not None:
+            self._f32(decay, "ssd_scan: decay")
+            if self._mat(decay, "ssd_scan: decay")[:2] != (rows, heads) or any(t is not None for t in (dt_bias, a_log, d_skip)):
+                raise KernelLibraryError("ssd_scan: given decays [rows, heads] stand in the place of dt_bias, a_log and d_skip")
+        else:
+            for t, what in ((dt_bias, "dt_bias"), (a_log, "a_log"), (d_skip, "d_skip")):
+                self._f32(t, "ssd_scan: " + what, heads)
         self._f32(state, "ssd_scan: state")
         if state.dim() != 4 or tuple(state.shape[1:]) != (heads, head_dim, n_state) or not state.is_contiguous():
             raise KernelLibraryError("ssd_scan: state must be dense [slots, heads, head_dim, n_state]")
@@ -914,7 +957,94 @@ class HipKernels:
                                          _ptr(d_skip), _ptr(state), _ptr(y), c_int(ld(y, "y")), c_int(heads),
                                          c_int(head_dim), c_int(n_state), c_int(groups), _ptr(seq_slot), _ptr(cu_rows),
                                          c_int(batch), c_int(max_rows if workspace is not None else 0), _ptr(workspace),
-                                         c_longlong(0 if workspace is None else workspace.numel()), self.stream))
+                                         c_longlong(0 if workspace is None else workspace.numel()), _ptr(decay),
+                                         c_int(0 if decay is None else ld(decay, "decay")), c_int(1 if ones else 0),
+                                         self.stream))
+
+    @query
+    def selective_scan_workspace(self, batch: int, channels: int, n_state: int, max_rows: int) -> int:
+        """Float32 entries of scratch with which `selective_scan` runs this launch in segments (0: it does not)."""
+        self.lib.lq_selective_scan_workspace.restype = c_longlong
+        return int(self.lib.lq_selective_scan_workspace(c_int(batch), c_int(channels), c_int(n_state), c_int(max_rows)))
+
+    def selective_scan(self, x: torch.Tensor, dt: torch.Tensor, b_in: torch.Tensor, c_in: torch.Tensor, z: torch.Tensor,
+                       dt_bias: torch.Tensor, a_log: torch.Tensor, d_skip: torch.Tensor, state: torch.Tensor,
+                       out: torch.Tensor, seq_slot: torch.Tensor, cu_rows: torch.Tensor, batch: int, max_rows: int = 0,
+                       workspace: Optional[torch.Tensor] = None) -> None:
+        """The selective scan along every sequence of the step, token by token: with dt = softplus(dt + dt_bias) a number
+        a channel and A = -exp(a_log) [channels, n_state], S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n and
+        y_c = sum_n S[c, n] C_n + d_skip_c x_c; out = y silu(z).  x, z, out [rows, channels], B and C [rows, n_state] in
+        one dtype, dt float32; state [slots, channels, n_state] float32 is read and left at the step's end.  `max_rows`
+        and `workspace` (`selective_scan_workspace(...)` floats) let a launch of few long sequences run in segments."""
+        rows, ch = x.shape
+        n = a_log.shape[1] if a_log.dim() == 2 else 0
+        self._dev(x, dt, b_in, c_in, z, out)
+        for t, what, cols in ((x, "x", ch), (dt, "dt", ch), (b_in, "B", n), (c_in, "C", n), (z, "z", ch), (out, "out", ch)):
+            if self._mat(t, "selective_scan: " + what)[:2] != (rows, cols):
+                raise KernelLibraryError(f"selective_scan: {what} must be [{rows}, {cols}], found {tuple(t.shape)}")
+        if not x.dtype == b_in.dtype == c_in.dtype == z.dtype == out.dtype:
+            raise KernelLibraryError("selective_scan: x, B, C, z and out in one dtype")
+        self._f32(dt, "selective_scan: dt")
+        self._f32(a_log, "selective_scan: a_log", ch * n)
+        self._f32(dt_bias, "selective_scan: dt_bias", ch)
+        self._f32(d_skip, "selective_scan: d_skip", ch)
+        self._f32(state, "selective_scan: state")
+        if state.dim() != 3 or tuple(state.shape[1:]) != (ch, n) or not state.is_contiguous():
+            raise KernelLibraryError("selective_scan: state must be dense [slots, channels, n_state]")
+        self._i32(seq_slot, "seq_slot", batch)
+        self._i32(cu_rows, "cu_rows", batch + 1)
+        if workspace is not None:
+            self._f32(workspace, "selective_scan: workspace", workspace.numel())
+        ld = self._rows2d
+        self._check(self.lib.lq_selective_scan(
+            _ptr(x), c_int(ld(x, "x")), _ptr(dt), c_int(ld(dt, "dt")), _ptr(b_in), c_int(ld(b_in, "B")), _ptr(c_in),
+            c_int(ld(c_in, "C")), _ptr(z), c_int(ld(z, "z")), _ptr(dt_bias), _ptr(a_log), _ptr(d_skip), _ptr(state), _ptr(out),
+            c_int(ld(out, "out")), c_int(_code(x)), c_int(ch), c_int(n), _ptr(seq_slot), _ptr(cu_rows), c_int(batch),
+            c_int(max_rows if workspace is not None else 0), _ptr(workspace),
+            c_longlong(0 if workspace is None else workspace.numel()), self.stream))
+
+    def memory_gates(self, i_in: torch.Tensor, f_in: torch.Tensor, i_bias: torch.Tensor, f_bias: torch.Tensor, cap: float,
+                     m_state: torch.Tensor, decay: torch.Tensor, take: torch.Tensor, floor: torch.Tensor,
+                     seq_slot: torch.Tensor, cu_rows: torch.Tensor, batch: int) -> None:
+        """Gates of a matrix memory along every sequence of the step, all float32: with i = cap tanh((i_in + i_bias) / cap),
+        f = log sigmoid(cap tanh((f_in + f_bias) / cap)) and a running maximum m (m_state [slots, heads], zero before the
+        first token): m <- max(f + m_before, i), decay = exp(f + m_before - m), take = exp(i - m), floor = exp(-m)."""
+        rows, heads = i_in.shape
+        for t, what in ((i_in, "i"), (f_in, "f"), (decay, "decay"), (take, "take"), (floor, "floor")):
+            self._f32(t, "memory_gates: " + what)
+            if self._mat(t, "memory_gates: " + what)[:2] != (rows, heads):
+                raise KernelLibraryError(f"memory_gates: {what} must be [{rows}, {heads}], found {tuple(t.shape)}")
+        if not (decay.is_contiguous() and take.is_contiguous() and floor.is_contiguous()):
+            raise KernelLibraryError("memory_gates: decay, take and floor must be dense")
+        self._f32(i_bias, "memory_gates: i_bias", heads)
+        self._f32(f_bias, "memory_gates: f_bias", heads)
+        self._f32(m_state, "memory_gates: m_state")
+        if m_state.dim() != 2 or m_state.shape[1] != heads or not m_state.is_contiguous():
+            raise KernelLibraryError("memory_gates: m_state must be dense [slots, heads]")
+        self._i32(seq_slot, "seq_slot", batch)
+        self._i32(cu_rows, "cu_rows", batch + 1)
+        self._check(self.lib.lq_memory_gates(
+            _ptr(i_in), c_int(self._rows2d(i_in, "i")), _ptr(f_in), c_int(self._rows2d(f_in, "f")), _ptr(i_bias), _ptr(f_bias),
+            c_float(cap), _ptr(m_state), _ptr(decay), _ptr(take), _ptr(floor), c_int(heads), _ptr(seq_slot), _ptr(cu_rows),
+            c_int(batch), self.stream))
+
+    def memory_out(self, y: torch.Tensor, floor: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, scale: float,
+                   den_eps: float, eps: float, out: torch.Tensor) -> None:
+        """y float32 [rows, heads * (P + 1)]: a head's S^T q and, behind it, n . q, both before q's scale.
+        o = scale y / (max(|scale n . q|, floor) + den_eps), divided by its root mean square over P (eps inside the
+        root), times weight [heads * P], times sigmoid(z); floor [rows, heads], z float32 [rows, heads * P]."""
+        rows, heads = floor.shape
+        ry, ny, ldy = self._mat(y, "memory_out: y")
+        rz, nz, ldz = self._mat(z, "memory_out: z")
+        ro, no, ldo = self._mat(out, "memory_out: out")
+        for t, what in ((y, "y"), (floor, "floor"), (z, "z")):
+            self._f32(t, "memory_out: " + what)
+        self._f32(weight, "memory_out: weight", nz)
+        if nz % heads or ny != nz + heads or (rz, ry) != (rows, rows) or (ro, no) != (rows, nz) or not floor.is_contiguous():
+            raise KernelLibraryError("memory_out: y [rows, heads (P + 1)], z and out [rows, heads P], dense floor [rows, heads]")
+        self._check(self.lib.lq_memory_out(_ptr(y), c_int(ldy), _ptr(floor), _ptr(z), c_int(ldz), _ptr(weight), c_float(scale),
+                                           c_float(den_eps), c_float(eps), _ptr(out), c_int(_code(out)), c_int(ldo),
+                                           c_int(rows), c_int(heads), c_int(nz // heads), self.stream))
 
     def delta_scan(self, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, beta: torch.Tensor, a: torch.Tensor,
                    dt_bias: torch.Tensor, a_log: torch.Tensor, state: torch.Tensor, out: torch.Tensor, heads: int,
@@ -971,19 +1101,57 @@ class HipKernels:
                                               c_int(1 if gate_first else 0), c_int(1 if gate == "sigmoid" else 0),
                                               self.stream))
 
-    def rmsnorm_mean(self, stack: torch.Tensor, weights, eps: float, out: torch.Tensor) -> None:
-        """out = mean over i of stack[i] / rms(stack[i]) * weights[i], row by row; stack [n, rows, width] float32."""
-        self._f32(stack, "rmsnorm_mean: stack")
+    def _branches(self, stack: torch.Tensor, weights, biases, what: str):
+        """The checked pointers of a stack of normed branches: weights and (None for none) biases, four of each."""
+        self._f32(stack, what + ": stack")
+        if stack.dim() != 3 or not stack.is_contiguous() or len(weights) != stack.shape[0] or not 1 <= len(weights) <= 4:
+            raise KernelLibraryError(f"{what}: a dense stack [n, rows, width] of 1 to 4 branches, a weight for each")
+        n, _, width = stack.shape
+        biases = list(biases) if biases is not None else [None] * n
+        if len(biases) != n:
+            raise KernelLibraryError(f"{what}: a bias (or None) for each branch")
+        for w in list(weights) + [b for b in biases if b is not None]:
+            self._f32(w, what + ": weight or bias", width)
+        none = [c_void_p(0)] * (4 - n)
+        return [_ptr(w) for w in weights] + none + [_ptr(b) for b in biases] + none
+
+    def rmsnorm_mean(self, stack: torch.Tensor, weights, eps: float, out: torch.Tensor, biases=None) -> None:
+        """out = mean over i of stack[i] / rms(stack[i]) * weights[i], row by row; stack [n, rows, width] float32.
+        `biases` (a vector or None for each branch): stack[i] + biases[i] in the place of stack[i]."""
+        ptrs = self._branches(stack, weights, biases, "rmsnorm_mean")
         self._f32(out, "rmsnorm_mean: out")
-        if stack.dim() != 3 or not stack.is_contiguous() or not out.is_contiguous() \
-                or tuple(out.shape) != tuple(stack.shape[1:]) or len(weights) != stack.shape[0] or not 1 <= len(weights) <= 4:
-            raise KernelLibraryError("rmsnorm_mean: a dense stack [n, rows, width] of 1 to 4 branches, a weight for each")
+        if not out.is_contiguous() or tuple(out.shape) != tuple(stack.shape[1:]):
+            raise KernelLibraryError("rmsnorm_mean: out must be dense and shaped like a branch")
         n, rows, width = stack.shape
-        for w in weights:
-            self._f32(w, "rmsnorm_mean: weight", width)
-        ws = [_ptr(w) for w in weights] + [c_void_p(0)] * (4 - n)
-        self._check(self.lib.lq_rmsnorm_mean(_ptr(stack), c_int(n), *ws, c_float(eps), _ptr(out), c_int(rows),
+        self._check(self.lib.lq_rmsnorm_mean(_ptr(stack), c_int(n), *ptrs, c_float(eps), _ptr(out), c_int(rows),
                                              c_int(width), self.stream))
+
+    @query
+    def mean_residual_takes(self, width: int) -> bool:
+        """Whether `mean_residual` takes rows of this width."""
+        return not self.force_generic and bool(self.lib.lq_mean_residual_accepts(c_int(width)))
+
+    def mean_residual(self, x: torch.Tensor, stack: torch.Tensor, weights, biases, branch_eps: float, weight: torch.Tensor,
+                      eps: float, rounded: Optional[torch.Tensor] = None) -> None:
+        """`rmsnorm_mean` and `rmsnorm_residual` in one pass: x += y / sqrt(mean(y^2) + eps) * weight with y the mean of
+        the normed branches; `rounded`, where given, takes the new x in its own dtype."""
+        ptrs = self._branches(stack, weights, biases, "mean_residual")
+        n, rows, width = stack.shape
+        self._f32(x, "mean_residual: x", rows * width)
+        self._f32(weight, "mean_residual: weight", width)
+        if tuple(x.shape) != (rows, width) or (rounded is not None and (tuple(rounded.shape) != (rows, width)
+                                                                        or not rounded.is_contiguous() or not rounded.is_cuda)):
+            raise KernelLibraryError("mean_residual: x and rounded must be dense and shaped like a branch")
+        self._check(self.lib.lq_mean_residual(_ptr(x), _ptr(stack), c_int(n), *ptrs, c_float(branch_eps), _ptr(weight),
+                                              c_float(eps), _ptr(rounded), c_int(_code(rounded) if rounded is not None else 0),
+                                              c_int(rows), c_int(width), self.stream))
+
+    def add_bias(self, x: torch.Tensor, bias: torch.Tensor) -> None:
+        """x[r, :] += bias (float32, x dense [rows, width])."""
+        rows, width = x.shape
+        self._f32(x, "add_bias: x", rows * width)
+        self._f32(bias, "add_bias: bias", width)
+        self._check(self.lib.lq_add_bias(_ptr(x), _ptr(bias), c_int(rows), c_int(width), self.stream))
 
     # ------------------------------------------------------------------ bigram embedding, norm on a sublayer's result,
     # ------------------------------------------------------------------ gated linear attention, latent attention, experts
@@ -1080,6 +1248,49 @@ class HipKernels:
                                            c_int(1 if interleaved else 0), _ptr(freqs if dims else None),
                                            c_float(magnitude), c_float(-1.0 if norm_eps is None else norm_eps),
                                            _ptr(row_pos), c_int(value_width), self.stream))
+
+    def qkv_norm_store(self, src: torch.Tensor, q_out: torch.Tensor, heads: int, kv_heads: int, key_dim: int, value_dim: int,
+                       eps: float, bias: Optional[torch.Tensor] = None, q_weight: Optional[torch.Tensor] = None,
+                       k_weight: Optional[torch.Tensor] = None, norm_qk: Optional[str] = None, norm_v: bool = False,
+                       v_from_k: bool = False, row_pos: Optional[torch.Tensor] = None, row_seq: Optional[torch.Tensor] = None,
+                       seq_slot: Optional[torch.Tensor] = None, block_table: Optional[torch.Tensor] = None,
+                       kcache: Optional[torch.Tensor] = None, vcache: Optional[torch.Tensor] = None,
+                       block_size: int = 0) -> None:
+        """src float32 [rows, queries | keys (| values)], `bias` (float32, a number a column) added first.  `norm_qk`:
+        None, "head" (every query and key head divided by its root mean square) or "row" (all heads of a row's queries
+        together, all of its keys together); q_weight and k_weight (of the normed run's size) multiply the result.
+        `norm_v`: every value head divided by its root mean square, no weight.  `v_from_k`: src has no values, they are
+        the keys with their bias, before their norm.  Queries go to q_out in its dtype; keys and values straight into
+        the paged cache (layout as `kv_store`) at the rows' positions, or nowhere when kcache is None."""
+        rows, ns, lds = self._mat(src, "qkv_norm_store: src")
+        rq, nq, ldq = self._mat(q_out, "qkv_norm_store: q")
+        kw, vw = kv_heads * key_dim, 0 if v_from_k else kv_heads * value_dim
+        if src.dtype != torch.float32 or ns != heads * key_dim + kw + vw or (rq, nq) != (rows, heads * key_dim) \
+                or norm_qk not in (None, "head", "row") or (v_from_k and key_dim != value_dim):
+            raise KernelLibraryError("qkv_norm_store: src float32 [rows, q | k | v], q_out [rows, q], norm_qk None, 'head' or 'row'")
+        uq, uk = (heads * key_dim, kw) if norm_qk == "row" else (key_dim, key_dim)
+        if bias is not None:
+            self._f32(bias, "qkv_norm_store: bias", ns)
+        for t, what, n in ((q_weight, "q_weight", uq), (k_weight, "k_weight", uk)):
+            if t is not None:
+                self._f32(t, "qkv_norm_store: " + what, n)
+        if norm_qk is None and (q_weight is not None or k_weight is not None):
+            raise KernelLibraryError("qkv_norm_store: weights without a norm")
+        stride = 0
+        if kcache is not None:
+            self._dev(kcache, vcache, row_pos, row_seq, seq_slot, block_table)
+            self._i32(row_pos, "row_pos", rows)
+            self._i32(row_seq, "row_seq", rows)
+            self._check_paged(kcache, vcache, kv_heads, key_dim, value_dim, block_size, block_table, seq_slot, "qkv_norm_store")
+            if kcache.dtype != q_out.dtype:
+                raise KernelLibraryError("qkv_norm_store: q_out in the cache's dtype")
+            stride = int(block_table.stride(0))
+        self._check(self.lib.lq_qkv_norm_store(
+            _ptr(src), c_int(lds), _ptr(bias), _ptr(q_weight), _ptr(k_weight), c_int(uq), c_int(uk),
+            c_int(0 if norm_qk is None else 1), c_int(1 if norm_v else 0), c_int(1 if v_from_k else 0), c_float(eps), _ptr(q_out),
+            c_int(ldq), c_int(_code(q_out)), c_int(rows), c_int(heads), c_int(kv_heads), c_int(key_dim), c_int(value_dim),
+            _ptr(row_pos), _ptr(row_seq), _ptr(seq_slot), _ptr(block_table), c_int(stride), _ptr(kcache), _ptr(vcache),
+            c_int(block_size), self.stream))
 
     def postnorm_residual(self, x: torch.Tensor, y: torch.Tensor, scales, weight: torch.Tensor, eps: float,
                           extra: Optional[torch.Tensor] = None, next_weight: Optional[torch.Tensor] = None,
