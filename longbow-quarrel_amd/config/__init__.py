@@ -2,8 +2,9 @@
 from .base import ConfigError, ModelConfig, read_config_json
 from .llama import LlamaConfig, RopeScaling
 from .mifidra import MifidraConfig
+from .puzonex import PuzonexConfig
 from .sofinex import SofinexConfig
 from .vafodra import VafodraConfig
 from .vupelorn import VupelornConfig
 
-__all__ = ["ConfigError", "ModelConfig", "read_config_json", "LlamaConfig", "MifidraConfig", "RopeScaling", "SofinexConfig", "VafodraConfig", "VupelornConfig"]
+__all__ = ["ConfigError", "ModelConfig", "read_config_json", "LlamaConfig", "MifidraConfig", "PuzonexConfig", "RopeScaling", "SofinexConfig", "VafodraConfig", "VupelornConfig"]

@@ -445,6 +445,9 @@ class Mixer(Part):
     takes_residual_sink = False
     #: forward has a keyword `out`, a float32 [rows, width] buffer of the caller's that the result is written to
     takes_out = False
+    #: a bias of the last projection (float32 [width]): forward then has a keyword `leave_bias`, with which the caller
+    #: says that it adds the bias itself on its way
+    out_bias: Optional[torch.Tensor] = None
 
     def cache_need(self):
         """KVNeed, StateNeed or None."""

@@ -176,7 +176,7 @@ class OutputNormBlock(Block):
     """Norms on the sublayers' results, none on their inputs: x += norm1(mixer(x)); x += norm2(ffn(x)).  The
     sublayers read the stream itself (rounded to the run's dtype where that is narrower).  The norms are RMS norms;
     one kernel normalises a sublayer's result, adds it to the 32-bit stream and leaves the stream's rounding for the
-    next reader.  The feed-forward may be absent (`feed_forward=None`; then there is no second norm either)."""
+    next reader; for mixers side by side it also norms their results and takes the mean.  The feed-forward may be absent (`feed_forward=None`; then there is no second norm either)."""
 
     def __init__(self, mixer: PartSpec, mixer_norm: PartSpec, feed_forward: Optional[PartSpec] = None,
                  ffn_norm: Optional[PartSpec] = None) -> None:
@@ -232,6 +232,18 @@ class OutputNormBlock(Block):
         ctx.kernels.rmsnorm_residual(x, y, norm.weight, norm.eps, rounded)
         return rounded if narrow else x
 
+    def _mixed(self, x: torch.Tensor, h: torch.Tensor, ctx: StepContext, cache) -> torch.Tensor:
+        """x += norm1(mixer(h)); -> x in the run's dtype."""
+        kn, norm = ctx.kernels, self.mixer_norm
+        branches = getattr(self.mixer, "forward_branches", None)
+        takes = getattr(kn, "mean_residual_takes", None)
+        if branches is None or self.mixer.weights is not None or takes is None or not takes(x.shape[1]):
+            return self._add_normed(x, self._run(self.mixer, (h, ctx, cache), ctx, x.shape[1]), norm, ctx)
+        stack, weights, biases = branches(h, ctx, cache)
+        rounded = ctx.ws.alloc(x.shape, ctx.dtype) if ctx.dtype != torch.float32 else None
+        kn.mean_residual(x, stack, weights, biases, self.mixer.eps, norm.weight, norm.eps, rounded)
+        return x if rounded is None else rounded
+
     def forward(self, x: torch.Tensor, pending, ctx: StepContext, cache: Optional[LayerCache]):
         kn = ctx.kernels
         if isinstance(pending, RoundedStream):
@@ -245,7 +257,7 @@ class OutputNormBlock(Block):
             if ctx.dtype != torch.float32:
                 h = ctx.ws.alloc(x.shape, ctx.dtype)
                 kn.cast(x, h)
-        h = self._add_normed(x, self._run(self.mixer, (h, ctx, cache), ctx, x.shape[1]), self.mixer_norm, ctx)
+        h = self._mixed(x, h, ctx, cache)
         if self.ffn is not None:
             h = self._add_normed(x, self._run(self.ffn, (h, ctx), ctx, x.shape[1]), self.ffn_norm, ctx)
         return RoundedStream(h) if h is not x else None

@@ -17,8 +17,12 @@ class TokenTable(Embedding):
     # form of it (`parts.base.product_weight`) in its place
     table_is_for_kernels = True
 
-    def __init__(self, name: str, vocab_size: int, width: int, scale: float = 1.0) -> None:
-        """`scale`: x = scale * E[token] (a model's own constant; the product is taken in 32-bit)."""
+    def __init__(self, name: str, vocab_size: int, width: int, scale: float = 1.0,
+                 sinusoids: Optional[float] = None) -> None:
+        """`scale`: x = scale * E[token] (a model's own constant; the product is taken in 32-bit).  `sinusoids`: a position
+        vector is added, entry 2 i the sine and entry 2 i + 1 the cosine of position * sinusoids^(-2 i / width)."""
+        self.sinusoids = None if sinusoids is None else float(sinusoids)
+        self.freqs: Optional[torch.Tensor] = None
         self.name, self.vocab_size, self.width, self.scale = name, int(vocab_size), int(width), float(scale)
         self.table: Optional[torch.Tensor] = None
 
@@ -28,10 +32,15 @@ class TokenTable(Embedding):
     def bind(self, tensors: Mapping[str, torch.Tensor], env: BuildEnv) -> None:
         super().bind(tensors, env)
         self.table = tensors[self.name].contiguous()
+        if self.sinusoids is not None:
+            self.freqs = torch.tensor([self.sinusoids ** (-2.0 * i / self.width) for i in range((self.width + 1) // 2)],
+                                      dtype=torch.float64, device=env.device)
 
     def forward(self, ctx: StepContext) -> torch.Tensor:
         x = ctx.ws.alloc((ctx.rows, self.width), torch.float32, keep=True)
-        if self.scale == 1.0:
+        if self.freqs is not None:
+            ctx.kernels.embed(self.table, ctx.tokens, x, scale=self.scale, row_pos=ctx.row_pos, freqs=self.freqs)
+        elif self.scale == 1.0:
             ctx.kernels.embed(self.table, ctx.tokens, x)
         else:
             ctx.kernels.embed(self.table, ctx.tokens, x, scale=self.scale)

@@ -1,6 +1,6 @@
-"""Mixers with a recurrent state of fixed size per sequence: the Mamba-2 state-space layer and the gated
-delta rule.  Both carry, for every sequence, a matrix state per head in 32-bit and the last inputs of a
-short causal convolution; both are computed token by token in the order of the sequence, by one kernel for
+"""Mixers with a recurrent state of fixed size per sequence: the Mamba-2 state-space layer, the selective scan, the
+gated delta rule, gated linear attention and a matrix memory with exponential gates.  They carry, for every sequence, a matrix state per head (or channel) in 32-bit and, where they have one, the last inputs of a
+short causal convolution; all are computed token by token in the order of the sequence, by one kernel for
 prompts and single tokens alike, so that the result does not depend on how a sequence is cut into steps.
 
 Everything that enters a recurrence is 32-bit (step sizes, decays, gates, unit norms, the state); the
@@ -27,7 +27,7 @@ class _Recurrent(Mixer):
     @staticmethod
     def _states(cache):
         if not isinstance(cache, MultiCache) or len(cache.parts) != 2:
-            raise RuntimeError("a recurrent mixer needs its state and its convolution's last inputs")
+            raise RuntimeError("a recurrent mixer needs its state and what it keeps beside it (a convolution's last inputs, a running maximum)")
         if not cache.write:
             raise RuntimeError("a recurrent state cannot be shared between runs of the schedule")
         return cache.parts[0].state, cache.parts[1].state
@@ -116,6 +116,171 @@ class Mamba2(_Recurrent):
                     ctx.seq_slot, ctx.cu_rows, ctx.batch, **more)
         normed = ctx.ws.alloc((rows, self.inner), ctx.dtype)
         kn.gated_rmsnorm(y, z, self.norm_w, self.eps, self.inner // self.norm_groups, normed, gate_first=True)
+        if out is None:
+            out = ctx.ws.alloc((rows, self.width), torch.float32)
+        project(kn, ctx, normed, self.w_o, out)
+        return out
+
+
+def _round8(n: int) -> int:
+    return (n + 7) // 8 * 8
+
+
+@MIXERS.register("mamba1")
+class Mamba1(_Recurrent):
+    """The selective scan of Gu and Dao, "Mamba: Linear-Time Sequence Modeling with Selective State Spaces".  One product
+    of the input gives [x | z] (`inner` columns each).  x passes a causal convolution per channel (`conv` taps, with bias)
+    and silu; a product of it gives [dt | B | C] (`dt_rank`, `state` and `state` columns), and a product of that dt a step
+    size for every channel, dt = softplus(Wdt dt + bias).  With A = -exp(A_log) [inner, state] and the state S starting
+    at zero, per channel c and entry n:
+
+        S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n,      y_c = sum_n S[c, n] C_n + D_c x_c.
+
+    Then y silu(z) and the output projection.  The step sizes, the decays and the state are 32-bit; the projections and
+    the convolution's result are in the run's dtype."""
+
+    def __init__(self, width: int, inner: int, state: int, dt_rank: int, conv: int, prefix: str,
+                 names: Optional[Mapping[str, str]] = None) -> None:
+        self.width, self.inner, self.state = int(width), int(inner), int(state)
+        self.dt_rank, self.taps = int(dt_rank), int(conv)
+        if min(self.inner, self.state, self.dt_rank, self.taps) < 1:
+            raise ValueError("channels, state, rank of the step sizes and taps must be positive")
+        n = {"in": "in", "conv": "conv", "conv_bias": "conv.b", "x": "x", "dt": "dt", "dt_bias": "dt.b", "A_log": "A_log",
+             "D": "D", "o": "o"}
+        n.update(names or {})
+        self.names: Dict[str, str] = {key: f"{prefix}.{val}" for key, val in n.items()}
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        nm = self.names
+        return [
+            TensorSpec(nm["in"], (2 * self.inner, self.width)),
+            TensorSpec(nm["conv"], (self.inner, self.taps), kind=VECTOR32),
+            TensorSpec(nm["conv_bias"], (self.inner,), kind=VECTOR32),
+            TensorSpec(nm["x"], (self.dt_rank + 2 * self.state, self.inner)),
+            TensorSpec(nm["dt"], (self.inner, self.dt_rank)),
+            TensorSpec(nm["dt_bias"], (self.inner,), kind=VECTOR32),
+            TensorSpec(nm["A_log"], (self.inner, self.state), kind=VECTOR32),
+            TensorSpec(nm["D"], (self.inner,), kind=VECTOR32, init="around_one"),
+            TensorSpec(nm["o"], (self.width, self.inner)),
+        ]
+
+    def bind(self, tensors: Mapping[str, torch.Tensor], env: BuildEnv) -> None:
+        super().bind(tensors, env)
+        nm = self.names
+        self.w_in, self.w_x, self.w_dt, self.w_o = (product_weight(env, tensors[nm[k]]) for k in ("in", "x", "dt", "o"))
+        self.conv_w, self.conv_b, self.dt_bias, self.a_log, self.d = (
+            tensors[nm[k]].contiguous() for k in ("conv", "conv_bias", "dt_bias", "A_log", "D"))
+
+    def cache_need(self) -> MultiNeed:
+        return MultiNeed((StateNeed((self.inner, self.state), torch.float32),
+                          StateNeed((max(1, self.taps - 1), self.inner), torch.float32)))
+
+    def forward(self, h: torch.Tensor, ctx: StepContext, cache, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        kn = ctx.kernels
+        state, conv_state = self._states(cache)
+        rows, c, r, n = h.shape[0], self.inner, self.dt_rank, self.state
+        u = ctx.ws.alloc((rows, _round8(2 * c)), ctx.dtype)[:, : 2 * c]
+        project(kn, ctx, h, self.w_in, u)
+        x = ctx.ws.alloc((rows, _round8(c)), ctx.dtype)[:, :c]
+        kn.causal_conv(u[:, :c], self.conv_w, self.conv_b, conv_state, x, ctx.row_pos, ctx.row_seq, ctx.seq_slot,
+                       ctx.seq_start, ctx.seq_len, ctx.cu_rows, ctx.batch, activation="silu")
+        low = ctx.ws.alloc((rows, _round8(r + 2 * n)), ctx.dtype)[:, : r + 2 * n]
+        project(kn, ctx, x, self.w_x, low)
+        dt = ctx.ws.alloc((rows, _round4(c)), torch.float32)[:, :c]
+        project(kn, ctx, low[:, :r], self.w_dt, dt)
+        y = ctx.ws.alloc((rows, _round8(c)), ctx.dtype)[:, :c]
+        # a few long prompts: the kernel may cut them into segments that run side by side, given scratch
+        ask = getattr(kn, "selective_scan_workspace", None)
+        need = ask(ctx.batch, c, n, ctx.max_new) if ask is not None else 0
+        more = dict(max_rows=ctx.max_new, workspace=ctx.ws.alloc((need,), torch.float32)) if need else {}
+        kn.selective_scan(x, dt, low[:, r : r + n], low[:, r + n :], u[:, c:], self.dt_bias, self.a_log, self.d, state, y,
+                          ctx.seq_slot, ctx.cu_rows, ctx.batch, **more)
+        if out is None:
+            out = ctx.ws.alloc((rows, self.width), torch.float32)
+        project(kn, ctx, y, self.w_o, out)
+        return out
+
+
+@MIXERS.register("matrix_memory")
+class MatrixMemory(_Recurrent):
+    """The matrix memory (mLSTM) of Beck, Poeppel, Spanring, Auer, Prudnikova, Kopp, Klambauer, Brandstetter, Hochreiter:
+    "xLSTM: Extended Long Short-Term Memory", with capped gates.  q and k are `heads` x `key_dim`, v is `heads` x
+    `value_dim`; q is scaled by key_dim^(-1/2).  Per head the logarithms of an input and a forget gate,
+    i = cap tanh((Wi h + bi) / cap) and f = log sigmoid(cap tanh((Wf h + bf) / cap)), a running maximum m, a memory S
+    [key_dim, value_dim] and a normaliser n [key_dim], all zero before the first token:
+
+        m' = max(f + m, i);   S <- exp(f + m - m') S + exp(i - m') k v^T;   n <- exp(f + m - m') n + exp(i - m') k;
+        o = S^T q / (max(|n . q|, exp(-m')) + den_eps).
+
+    Each head's o is divided by its root mean square; the heads side by side are multiplied by a weight (all heads'
+    entries) and by the sigmoid of one more projection of the input; then the output projection.
+
+    How it runs.  The gates of all tokens come first (`memory_gates`: a decay and a factor a token and head); the memory
+    is then the state-space scan with given decays, k and q in the place of B and C and v of x, and the normaliser is one
+    more column of the head's values whose input is one.  `memory_out` divides, norms and gates."""
+
+    def __init__(self, width: int, heads: int, key_dim: int, value_dim: int, gate_cap: float, eps: float, den_eps: float,
+                 prefix: str, names: Optional[Mapping[str, str]] = None) -> None:
+        self.width, self.heads, self.key_dim, self.value_dim = int(width), int(heads), int(key_dim), int(value_dim)
+        self.gate_cap, self.eps, self.den_eps = float(gate_cap), float(eps), float(den_eps)
+        if not self.gate_cap > 0:
+            raise ValueError("the gates' cap must be positive")
+        self.qk_width, self.v_width = self.heads * self.key_dim, self.heads * self.value_dim
+        n = {"q": "q", "k": "k", "v": "v", "gate": "g", "i": "i", "f": "f", "i_bias": "i.b", "f_bias": "f.b", "norm": "norm",
+             "o": "o"}
+        n.update(names or {})
+        self.names: Dict[str, str] = {key: f"{prefix}.{val}" for key, val in n.items()}
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        nm = self.names
+        return [
+            TensorSpec(nm["q"], (self.qk_width, self.width)),
+            TensorSpec(nm["k"], (self.qk_width, self.width)),
+            TensorSpec(nm["v"], (self.v_width, self.width)),
+            TensorSpec(nm["gate"], (self.v_width, self.width)),
+            TensorSpec(nm["o"], (self.width, self.v_width)),
+            TensorSpec(nm["norm"], (self.v_width,), kind=VECTOR32, init="around_one"),
+            TensorSpec(nm["i"], (self.heads, self.width)),
+            TensorSpec(nm["i_bias"], (self.heads,), kind=VECTOR32),
+            TensorSpec(nm["f"], (self.heads, self.width)),
+            TensorSpec(nm["f_bias"], (self.heads,), kind=VECTOR32),
+        ]
+
+    def bind(self, tensors: Mapping[str, torch.Tensor], env: BuildEnv) -> None:
+        super().bind(tensors, env)
+        nm = self.names
+        mats = [tensors[nm[k]] for k in ("q", "k", "v", "gate", "i", "f")]
+        if len({m.dtype for m in mats}) != 1:
+            raise ValueError(f"{nm['q']}: the projections of one input are stored in different dtypes")
+        self.w_in = product_weight(env, torch.cat(mats, dim=0))  # one product, 32-bit results for the gates and the scan
+        self.w_o = product_weight(env, tensors[nm["o"]])
+        self.norm_w, self.i_bias, self.f_bias = (tensors[nm[k]].contiguous() for k in ("norm", "i_bias", "f_bias"))
+
+    def cache_need(self) -> MultiNeed:
+        # held [head, value_dim + 1, key_dim]: the normaliser is the head's last column; beside it the running maximum
+        return MultiNeed((StateNeed((self.heads, self.value_dim + 1, self.key_dim), torch.float32),
+                          StateNeed((self.heads,), torch.float32)))
+
+    def forward(self, h: torch.Tensor, ctx: StepContext, cache, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        kn = ctx.kernels
+        state, top = self._states(cache)
+        rows, nh, qk, vw = h.shape[0], self.heads, self.qk_width, self.v_width
+        total = 2 * qk + 2 * vw + 2 * nh
+        u = ctx.ws.alloc((rows, _round4(total)), torch.float32)[:, :total]
+        project(kn, ctx, h, self.w_in, u)
+        at = 2 * qk + 2 * vw
+        decay, take, floor = (ctx.ws.alloc((rows, nh), torch.float32) for _ in range(3))
+        kn.memory_gates(u[:, at : at + nh], u[:, at + nh :], self.i_bias, self.f_bias, self.gate_cap, top, decay, take, floor,
+                        ctx.seq_slot, ctx.cu_rows, ctx.batch)
+        cols = self.value_dim + 1
+        y = ctx.ws.alloc((rows, nh * cols), torch.float32)
+        ask = getattr(kn, "ssd_scan_workspace", None)
+        need = ask(ctx.batch, nh, cols, self.key_dim, ctx.max_new) if ask is not None else 0
+        more = dict(max_rows=ctx.max_new, workspace=ctx.ws.alloc((need,), torch.float32)) if need else {}
+        kn.ssd_scan(u[:, 2 * qk : 2 * qk + vw], u[:, qk : 2 * qk], u[:, :qk], take, None, None, None, state, y, nh, cols,
+                    self.key_dim, nh, ctx.seq_slot, ctx.cu_rows, ctx.batch, decay=decay, ones=True, **more)
+        normed = ctx.ws.alloc((rows, vw), ctx.dtype)
+        kn.memory_out(y, floor, u[:, 2 * qk + vw : at], self.norm_w, self.key_dim ** -0.5, self.den_eps, self.eps, normed)
         if out is None:
             out = ctx.ws.alloc((rows, self.width), torch.float32)
         project(kn, ctx, normed, self.w_o, out)
@@ -308,7 +473,7 @@ class SideBySide(Mixer):
     def lengths_uneven(self, kernels, lengths) -> bool:
         return any(s.lengths_uneven(kernels, lengths) for s in self.sides)
 
-    def _results(self, h: torch.Tensor, ctx: StepContext, cache) -> torch.Tensor:
+    def _results(self, h: torch.Tensor, ctx: StepContext, cache, leave_bias: bool = False) -> torch.Tensor:
         if not isinstance(cache, MultiCache) or len(cache.parts) != len(self.sides):
             raise RuntimeError("mixers side by side need a cache for each side")
         rows = h.shape[0]
@@ -316,7 +481,8 @@ class SideBySide(Mixer):
         for i, (side, part) in enumerate(zip(self.sides, cache.parts)):
             part = None if isinstance(part, MultiCache) and not part.parts else part
             if side.takes_out:
-                side.forward(h, ctx, part, out=results[i])
+                more = {"leave_bias": True} if leave_bias and side.out_bias is not None else {}
+                side.forward(h, ctx, part, out=results[i], **more)
             else:
                 ctx.kernels.cast(side.forward(h, ctx, part), results[i])
         return results
@@ -327,12 +493,23 @@ class SideBySide(Mixer):
             return self.forward(h, ctx, cache), (1.0,)
         return self._results(h, ctx, cache), self.weights
 
+    def _biases(self):
+        """The biases that the mixers leave to whoever norms their outputs (None: there is none)."""
+        biases = [side.out_bias if side.takes_out else None for side in self.sides]
+        return biases if any(b is not None for b in biases) else None
+
+    def forward_branches(self, h: torch.Tensor, ctx: StepContext, cache):
+        """The normed mean's ingredients: the mixers' outputs [n, rows, width], their weights and the biases that are
+        still to be added to them (None: there is none)."""
+        return self._results(h, ctx, cache, leave_bias=True), self.out_w, self._biases()
+
     def forward(self, h: torch.Tensor, ctx: StepContext, cache, out: Optional[torch.Tensor] = None) -> torch.Tensor:
-        results = self._results(h, ctx, cache)
+        results = self._results(h, ctx, cache, leave_bias=self.weights is None)
         if out is None:
             out = ctx.ws.alloc((h.shape[0], self.width), torch.float32)
         if self.weights is None:
-            ctx.kernels.rmsnorm_mean(results, self.out_w, self.eps, out)
+            biases = self._biases()
+            ctx.kernels.rmsnorm_mean(results, self.out_w, self.eps, out, **({"biases": biases} if biases else {}))
             return out
         ctx.kernels.cast(results[0], out)
         ctx.kernels.scale(out, self.weights[0])

@@ -22,10 +22,27 @@ product with the values (the sums stay 32-bit): plain causal attention with keys
 a bfloat16 run, on the causal kernel of the matrix cores, several times as fast over a prompt.  The default keeps the
 weights 32-bit through that product.
 
+What a design may ask for beside these, each with a parameter (none of it together with a rotation or `qk_norm_eps`):
+* `qkv_bias`: biases on q, k and v (`<name>.b`); `out_bias`: one on the output projection (`<prefix>.o.b`).
+* `qk_norm` "head" or "row": RMS norm with a weight (`<prefix>.q.norm`, `<prefix>.k.norm`) on every head of q and k (the
+  weight is shared by the heads), or on all heads' entries of a row together; `value_norm`: every value head divided
+  by its root mean square, without a weight.  `norm_eps` for all of them.
+* `values_from_keys`: there is no Wv, the values are the keys as projected (with their bias, before their norm).
+* `temperature`: a stored number a head (`<prefix>.temp`) multiplies the scaled score; `softcap`: score <- softcap
+  tanh(score / softcap) (0: not).
+* `log_bias`: r1_h ln(1 + r2_h n) is taken off the score of a key n positions back (`<prefix>.r1`, `.r2`, a number a
+  head); `table_bias` (`rows`, `most`): a learned number for the distance's row of a table and the head is added
+  (`<prefix>.rel` [rows, heads], rows by `distance_rows`).
+* `entry_gate`: every entry of the heads' result times the sigmoid of one more projection of h (`<prefix>.g`, a row an
+  entry).
+Biases, norms and the store into the cache are one kernel (`qkv_norm_store`) on the product's 32-bit result; what
+shapes a score and the gate are inside the attention kernel.
+
 All projections of h are one matrix product ([q | k | v | gate]).
 """
 from __future__ import annotations
 
+import math
 from typing import Dict, List, Mapping, Optional
 
 import torch
@@ -46,6 +63,22 @@ def split_scratch(ctx: StepContext, dtype, heads: int, kv_heads: int, key_dim: i
     return dict(max_len=ctx.max_len, workspace=ctx.ws.alloc((need,), torch.float32)) if need else {}
 
 
+def distance_rows(rows: int, most: float, window: int = 0) -> List[int]:
+    """The row of a `rows`-row table for the distances 0, 1, ...: a distance below half = rows // 2 has a row of its own,
+    a farther one shares half + floor(ln(n / half) / ln(most / half) (rows - half)), at most the last row.  The list
+    ends where every farther distance has the last row, or with the farthest distance that a window shows."""
+    half = rows // 2
+    if rows < 2 or not most > half:
+        raise ValueError(f"a table of {rows} rows cannot end at a distance of {most}")
+    out: List[int] = []
+    while (not window or len(out) < window) and (not out or out[-1] < rows - 1):
+        n = len(out)
+        # (an exact step, which rounding may leave just below its whole number, counts as reached)
+        out.append(n if n < half else
+                   min(rows - 1, half + math.floor(math.log(n / half) / math.log(most / half) * (rows - half) + 1e-9)))
+    return out
+
+
 @MIXERS.register("sink_window_attention")
 class SinkWindowAttention(Mixer):
     takes_out = True
@@ -54,7 +87,10 @@ class SinkWindowAttention(Mixer):
                  prefix: str, window: int = 0, keep_first: int = 0, sink=True, head_gate: bool = False,
                  position: Optional[PartSpec] = None, rotary: Optional[Mapping] = None,
                  qk_norm_eps: Optional[float] = None, names: Optional[Mapping[str, str]] = None,
-                 probabilities: str = "float32") -> None:
+                 probabilities: str = "float32", qkv_bias: bool = False, out_bias: bool = False,
+                 qk_norm: Optional[str] = None, value_norm: bool = False, norm_eps: float = 0.0,
+                 values_from_keys: bool = False, temperature: bool = False, softcap: float = 0.0, log_bias: bool = False,
+                 table_bias: Optional[Mapping] = None, entry_gate: bool = False) -> None:
         if heads % kv_heads != 0:
             raise ValueError(f"{heads} heads cannot share {kv_heads} kv heads evenly")
         self.rot_dims, self.rot_interleaved, self.rot_magnitude, self.freq_table = 0, False, 1.0, []
@@ -75,6 +111,21 @@ class SinkWindowAttention(Mixer):
         self.prepared = rotary is not None or qk_norm_eps is not None  # q, k and v pass the kernel named above
         if self.prepared and head_gate:
             raise ValueError("a gate per head and a rotation or norm of q and k are not combined")
+        if qk_norm not in (None, "head", "row"):
+            raise ValueError(f"q and k are normed by 'head' or by 'row' (or not: None), found {qk_norm!r}")
+        self.qkv_bias, self.has_out_bias, self.qk_norm, self.value_norm = bool(qkv_bias), bool(out_bias), qk_norm, bool(value_norm)
+        self.norm_eps, self.values_from_keys, self.temperature = float(norm_eps), bool(values_from_keys), bool(temperature)
+        self.softcap, self.log_bias, self.entry_gate = float(softcap), bool(log_bias), bool(entry_gate)
+        self.table_bias = None if table_bias is None else (int(table_bias["rows"]), float(table_bias["most"]))
+        self.stored = bool(qkv_bias or qk_norm or value_norm or values_from_keys or entry_gate)  # by `qkv_norm_store`
+        self.shaped = bool(temperature or softcap or log_bias or table_bias is not None or entry_gate)
+        if self.stored and (self.prepared or position is not None or head_gate):
+            raise ValueError("biases, weighted norms, values from keys or a gate an entry are not combined with a rotation, "
+                             "a unit norm of q and k or a gate a head")
+        if self.values_from_keys and key_dim != value_dim:
+            raise ValueError(f"values that are the keys are as wide as they are ({key_dim}, {value_dim})")
+        if self.softcap < 0:
+            raise ValueError("the cap on the scores must not be negative")
         if window < 0 or keep_first < 0:
             raise ValueError("window and keep_first must not be negative")
         self.width, self.heads, self.kv_heads = int(width), int(heads), int(kv_heads)
@@ -87,7 +138,8 @@ class SinkWindowAttention(Mixer):
         if probabilities not in ("float32", "bfloat16"):
             raise ValueError(f"probabilities are 'float32' or 'bfloat16', found {probabilities!r}")
         self.probabilities = probabilities
-        n = {"q": "q", "k": "k", "v": "v", "gate": "g", "o": "o", "sink": "sink"}
+        n = {"q": "q", "k": "k", "v": "v", "gate": "g", "o": "o", "sink": "sink", "q_norm": "q.norm", "k_norm": "k.norm",
+             "temp": "temp", "r1": "r1", "r2": "r2", "rel": "rel"}
         n.update(names or {})
         self.names: Dict[str, str] = {key: f"{prefix}.{val}" for key, val in n.items()}
         self.position = build_part(POSITION_ENCODINGS, position) if position is not None else None
@@ -102,14 +154,29 @@ class SinkWindowAttention(Mixer):
     def graph_safe(self) -> bool:
         return self.position is None or self.position.graph_safe
 
+    def _projections(self):
+        """The projections of h, in the order of their one product: (key of the name, rows)."""
+        return [("q", self.q_width), ("k", self.k_width)] + \
+            ([] if self.values_from_keys else [("v", self.v_width)]) + \
+            ([("gate", self.heads)] if self.head_gate else [("gate", self.o_width)] if self.entry_gate else [])
+
     def tensor_specs(self) -> List[TensorSpec]:
-        specs = [
-            TensorSpec(self.names["q"], (self.q_width, self.width)),
-            TensorSpec(self.names["k"], (self.k_width, self.width)),
-            TensorSpec(self.names["v"], (self.v_width, self.width)),
-        ]
-        if self.head_gate:
-            specs.append(TensorSpec(self.names["gate"], (self.heads, self.width)))
+        nm = self.names
+        specs = []
+        for key, width in self._projections():
+            specs.append(TensorSpec(nm[key], (width, self.width)))
+            if self.qkv_bias and key != "gate":
+                specs.append(TensorSpec(nm[key] + ".b", (width,), kind=VECTOR32))
+        if self.qk_norm:
+            whole = self.qk_norm == "row"
+            specs += [TensorSpec(nm["q_norm"], (self.q_width if whole else self.key_dim,), kind=VECTOR32, init="around_one"),
+                      TensorSpec(nm["k_norm"], (self.k_width if whole else self.key_dim,), kind=VECTOR32, init="around_one")]
+        for key in (["temp"] if self.temperature else []) + (["r1", "r2"] if self.log_bias else []):
+            specs.append(TensorSpec(nm[key], (self.heads,), kind=VECTOR32, init="around_one"))
+        if self.table_bias is not None:
+            specs.append(TensorSpec(nm["rel"], (self.table_bias[0], self.heads), kind=VECTOR32))
+        if self.has_out_bias:
+            specs.append(TensorSpec(nm["o"] + ".b", (self.width,), kind=VECTOR32))
         if self.learned_sink:
             specs.append(TensorSpec(self.names["sink"], (self.heads,), kind=VECTOR32))
         specs.append(TensorSpec(self.names["o"], (self.width, self.o_width)))
@@ -117,13 +184,29 @@ class SinkWindowAttention(Mixer):
 
     def bind(self, tensors: Mapping[str, torch.Tensor], env: BuildEnv) -> None:
         super().bind(tensors, env)
-        mats = [tensors[self.names[key]] for key in ("q", "k", "v") + (("gate",) if self.head_gate else ())]
+        nm = self.names
+        mats = [tensors[nm[key]] for key, _ in self._projections()]
         if len({m.dtype for m in mats}) != 1:
             raise ValueError(f"{self.names['q']}: the projections of one input are stored in different dtypes")
         self.w_in = product_weight(env, torch.cat(mats, dim=0))
         self.w_o = product_weight(env, tensors[self.names["o"]])
         if self.learned_sink:
             self.sink_w = tensors[self.names["sink"]].contiguous()
+        get = lambda key, there: tensors[nm[key]].contiguous() if there else None
+        self.q_norm_w, self.k_norm_w = get("q_norm", self.qk_norm), get("k_norm", self.qk_norm)
+        self.in_bias = torch.cat([tensors[nm[key] + ".b"] for key, _ in self._projections() if key != "gate"]).contiguous() \
+            if self.qkv_bias else None
+        self.out_bias = tensors[nm["o"] + ".b"].contiguous() if self.has_out_bias else None
+        self.shape_kw: Dict[str, object] = {}  # how `sink_attention` shapes the scores
+        if self.softcap:
+            self.shape_kw["softcap"] = self.softcap
+        if self.temperature:
+            self.shape_kw["temp"] = get("temp", True)
+        if self.log_bias:
+            self.shape_kw["log_bias"] = (get("r1", True), get("r2", True))
+        if self.table_bias is not None:  # looked up by distance: one number a head and distance
+            rows = torch.tensor(distance_rows(*self.table_bias, self.window), device=tensors[nm["rel"]].device)
+            self.shape_kw["distance_bias"] = tensors[nm["rel"]].index_select(0, rows).t().contiguous()
         if self.position is not None:
             self.position.bind(tensors, env)
         self.freqs = torch.tensor(self.freq_table, dtype=torch.float64, device=env.device) if self.rot_dims else None
@@ -134,7 +217,7 @@ class SinkWindowAttention(Mixer):
 
     def lengths_uneven(self, kernels, lengths) -> bool:
         ask = getattr(kernels, "decode_lengths_uneven", None)
-        plain = not (self.sink or self.head_gate or self.keep_first or self.window) and self.key_dim == self.value_dim \
+        plain = not (self.sink or self.head_gate or self.keep_first or self.window or self.shaped) and self.key_dim == self.value_dim \
             and self.probabilities == "bfloat16"
         return bool(ask(lengths)) if ask is not None and plain else False
 
@@ -142,21 +225,34 @@ class SinkWindowAttention(Mixer):
         """Whether this step's attention is the causal kernel's (`attention`): the design lets the probabilities be
         rounded to bfloat16 for their product with the values (that kernel's way; the general kernel keeps them
         32-bit), the mask and softmax are plain, and the kernel object runs the shape on its matrix cores."""
-        if self.probabilities != "bfloat16" or self.sink or self.head_gate or self.keep_first \
+        if self.probabilities != "bfloat16" or self.sink or self.head_gate or self.keep_first or self.shaped \
                 or self.key_dim != self.value_dim:
             return False
         ask = getattr(kn, "attention_on_matrix_cores", None)
         return ask is not None and bool(ask(ctx.dtype, self.heads, self.kv_heads, self.key_dim, cache.block_size))
 
     def forward(self, h: torch.Tensor, ctx: StepContext, cache: Optional[LayerCache],
-                out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                out: Optional[torch.Tensor] = None, leave_bias: bool = False) -> torch.Tensor:
         if cache is None or cache.k is None:
             raise RuntimeError("attention needs a key/value cache")
         kn = ctx.kernels
         rows = h.shape[0]
-        total = self.q_width + self.k_width + self.v_width + (self.heads if self.head_gate else 0)
+        total = sum(n for _, n in self._projections())
         total_padded = (total + 3) // 4 * 4  # rows of the product start on 16 bytes
-        if self.prepared:
+        wide_gate = None
+        if self.stored:
+            # biases and norms are taken on the product's 32-bit result; keys and values go straight into the cache
+            proj = ctx.ws.alloc((rows, total_padded), torch.float32)[:, :total]
+            project(kn, ctx, h, self.w_in, proj)
+            q, k, v, gate = ctx.ws.alloc((rows, self.q_width), ctx.dtype), None, None, None
+            n_qkv = total - (self.o_width if self.entry_gate else 0)
+            place = dict(row_pos=ctx.row_pos, row_seq=ctx.row_seq, seq_slot=ctx.seq_slot, block_table=cache.block_table,
+                         kcache=cache.k, vcache=cache.v, block_size=cache.block_size) if cache.write else {}
+            kn.qkv_norm_store(proj[:, :n_qkv], q, self.heads, self.kv_heads, self.key_dim, self.value_dim, self.norm_eps,
+                              bias=self.in_bias, q_weight=self.q_norm_w, k_weight=self.k_norm_w, norm_qk=self.qk_norm,
+                              norm_v=self.value_norm, v_from_k=self.values_from_keys, **place)
+            wide_gate = proj[:, n_qkv:] if self.entry_gate else None
+        elif self.prepared:
             # the product's 32-bit result is rotated and normed in 32-bit, then rounded to what the cache holds
             proj = ctx.ws.alloc((rows, total_padded), torch.float32)[:, :total]
             project(kn, ctx, h, self.w_in, proj)
@@ -176,7 +272,7 @@ class SinkWindowAttention(Mixer):
             gate = proj[:, self.q_width + self.k_width + self.v_width :] if self.head_gate else None
             if self.position is not None:
                 self.position.apply(q, k, ctx)
-        if cache.write:
+        if cache.write and k is not None:
             kn.kv_store(k, v, self.kv_heads, self.key_dim, self.value_dim, ctx.row_pos, ctx.row_seq, ctx.seq_slot,
                         cache.block_table, cache.k, cache.v, cache.block_size)
         att = ctx.ws.alloc((rows, self.o_width), ctx.dtype)
@@ -188,18 +284,21 @@ class SinkWindowAttention(Mixer):
                          ctx.cu_rows, cache.block_table, cache.k, cache.v, cache.block_size, self.scale, self.window,
                          decode=ctx.decode, max_len=ctx.max_len,
                          workspace=ctx.ws.alloc((need,), torch.float32) if need else None, uneven=ctx.uneven)
-            if out is None:
-                out = ctx.ws.alloc((rows, self.width), torch.float32)
-            project(kn, ctx, att, self.w_o, out)
-            return out
+            return self._project_out(ctx, att, out, leave_bias)
         kn.sink_attention(q, att, self.heads, self.kv_heads, self.key_dim, self.value_dim, ctx.row_pos, ctx.row_seq,
                           ctx.seq_slot, cache.block_table, cache.k, cache.v, cache.block_size, self.scale,
                           window=self.window, keep_first=self.keep_first, sink=self.sink, gate=gate,
-                          decode=ctx.decode, **({"sink_values": self.sink_w} if self.learned_sink else {}),
+                          decode=ctx.decode, **self.shape_kw, **({"wide_gate": wide_gate} if wide_gate is not None else {}),
+                          **({"sink_values": self.sink_w} if self.learned_sink else {}),
                           **split_scratch(ctx, q.dtype, self.heads, self.kv_heads, self.key_dim,
                                                              self.value_dim, cache.block_size, self.window,
                                                              self.keep_first))
+        return self._project_out(ctx, att, out, leave_bias)
+
+    def _project_out(self, ctx: StepContext, att: torch.Tensor, out: Optional[torch.Tensor], leave_bias: bool) -> torch.Tensor:
         if out is None:
-            out = ctx.ws.alloc((rows, self.width), torch.float32)
-        project(kn, ctx, att, self.w_o, out)
+            out = ctx.ws.alloc((att.shape[0], self.width), torch.float32)
+        project(ctx.kernels, ctx, att, self.w_o, out)
+        if self.out_bias is not None and not leave_bias:
+            ctx.kernels.add_bias(out, self.out_bias)
         return out

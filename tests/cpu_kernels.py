@@ -25,10 +25,14 @@ class CpuKernels:
     def use_stream(self, stream) -> None:
         pass
 
-    def embed(self, table, tokens, out, scale=1.0):
+    def embed(self, table, tokens, out, scale=1.0, row_pos=None, freqs=None):
         t = tokens[: out.shape[0]].long()
         known = (t >= 0) & (t < table.shape[0])  # no row of the table: zeros, as the library does
         out.copy_(table[t.clamp(0, table.shape[0] - 1)].float() * known[:, None] * scale)
+        if freqs is not None:
+            ang = row_pos[: out.shape[0]].double()[:, None] * freqs[None, :]
+            out[:, 0::2] += torch.sin(ang).float()
+            out[:, 1::2] += torch.cos(ang[:, : out.shape[1] // 2]).float()
 
     @staticmethod
     def _whole(delta, like):
@@ -179,7 +183,8 @@ class CpuKernels:
 
     def sink_attention(self, q, out, heads, kv_heads, key_dim, value_dim, row_pos, row_seq, seq_slot, block_table,
                        kcache, vcache, block_size, scale, window=0, keep_first=0, sink=True, gate=None, decode=False,
-                       sink_values=None, maps=1):
+                       sink_values=None, maps=1, softcap=0.0, temp=None, log_bias=None, distance_bias=None,
+                       wide_gate=None):
         if maps > 1:  # a cached key row holds the keys of `maps` key heads side by side; they share the value head
             nb, g_heads, bs, wide = kcache.shape
             kcache = kcache.reshape(nb, g_heads, bs, maps, key_dim).permute(0, 1, 3, 2, 4).reshape(nb, kv_heads, bs, key_dim)
@@ -194,6 +199,15 @@ class CpuKernels:
             for h in range(heads):
                 g = h // (heads // kv_heads)
                 s = (kk[:, g] @ q[r, h * key_dim : (h + 1) * key_dim].float()) * scale
+                back = p - torch.tensor(ts)
+                if temp is not None:
+                    s = s * temp[h]
+                if softcap:
+                    s = softcap * torch.tanh(s / softcap)
+                if log_bias is not None:
+                    s = s - log_bias[0][h] * torch.log1p(log_bias[1][h] * back.float())
+                if distance_bias is not None:
+                    s = s + distance_bias[h][back.clamp(max=distance_bias.shape[1] - 1)]
                 at = float(sink_values[h]) if sink_values is not None else 0.0
                 m = torch.clamp(s.max(), min=at) if sink else s.max()
                 e = torch.exp(s - m)
@@ -201,6 +215,8 @@ class CpuKernels:
                 o = (e[:, None] * vv[:, g]).sum(0) / denom
                 if gate is not None:
                     o = o * torch.sigmoid(gate[r, h].float())
+                if wide_gate is not None:
+                    o = o * torch.sigmoid(wide_gate[r, h * value_dim : (h + 1) * value_dim])
                 out[r, h * value_dim : (h + 1) * value_dim] = o.to(out.dtype)
 
     def causal_conv(self, x, weight, bias, state, out, row_pos, row_seq, seq_slot, seq_start, seq_len, cu_rows, batch,
@@ -222,7 +238,18 @@ class CpuKernels:
                 state[slot][: taps - 1] = hist[hist.shape[0] - (taps - 1) :]
 
     def ssd_scan(self, x, b_in, c_in, dt, dt_bias, a_log, d_skip, state, y, heads, head_dim, n_state, groups, seq_slot,
-                 cu_rows, batch):
+                 cu_rows, batch, decay=None, ones=False):
+        if decay is not None:  # given decays and steps, perhaps a last column whose input is one
+            for b in range(batch):
+                s = state[int(seq_slot[b])]
+                for r in range(int(cu_rows[b]), int(cu_rows[b + 1])):
+                    xr = x[r].float().reshape(heads, -1)
+                    xr = torch.cat([xr, torch.ones(heads, 1)], 1) if ones else xr
+                    br = b_in[r].float().reshape(groups, n_state).repeat_interleave(heads // groups, 0)
+                    cr = c_in[r].float().reshape(groups, n_state).repeat_interleave(heads // groups, 0)
+                    s.mul_(decay[r][:, None, None]).add_(dt[r][:, None, None] * xr[:, :, None] * br[:, None, :])
+                    y[r] = (s * cr[:, None, :]).sum(-1).reshape(-1)
+            return
         for b in range(batch):
             r0, r1 = int(cu_rows[b]), int(cu_rows[b + 1])
             s = state[int(seq_slot[b])]  # [heads, head_dim, n_state]
@@ -267,9 +294,10 @@ class CpuKernels:
         v = v * (weight if weight.numel() == n else weight.repeat(n // weight.numel()))
         out.copy_((v if gate_first else v * gate).to(out.dtype))
 
-    def rmsnorm_mean(self, stack, weights, eps, out):
+    def rmsnorm_mean(self, stack, weights, eps, out, biases=None):
         acc = torch.zeros_like(out)
-        for t, w in zip(stack, weights):
+        for t, w, b in zip(stack, weights, biases or [None] * len(weights)):
+            t = t if b is None else t + b
             acc += t / torch.sqrt((t * t).mean(-1, keepdim=True) + eps) * w
         out.copy_(acc / len(weights))
 
@@ -305,6 +333,69 @@ class CpuKernels:
         x += yf / torch.sqrt((yf * yf).mean(-1, keepdim=True) + eps) * weight
         if rounded is not None:
             rounded.copy_(x.to(rounded.dtype))
+
+    @query
+    def mean_residual_takes(self, width):
+        return width % 4 == 0
+
+    def mean_residual(self, x, stack, weights, biases, branch_eps, weight, eps, rounded=None):
+        y = torch.empty_like(x)
+        self.rmsnorm_mean(stack, weights, branch_eps, y, biases)
+        self.rmsnorm_residual(x, y, weight, eps, rounded)
+
+    def add_bias(self, x, bias):
+        x += bias
+
+    def qkv_norm_store(self, src, q_out, heads, kv_heads, key_dim, value_dim, eps, bias=None, q_weight=None, k_weight=None,
+                       norm_qk=None, norm_v=False, v_from_k=False, row_pos=None, row_seq=None, seq_slot=None,
+                       block_table=None, kcache=None, vcache=None, block_size=0):
+        rows, qw, kw = src.shape[0], heads * key_dim, kv_heads * key_dim
+        t = src.float() if bias is None else src.float() + bias
+
+        def unit(v, weight, per):
+            v = v.reshape(rows, -1, per)
+            v = v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps)
+            return (v if weight is None else v * weight).reshape(rows, -1)
+
+        q, k = t[:, :qw], t[:, qw : qw + kw]
+        v = k if v_from_k else t[:, qw + kw :]
+        if norm_qk:
+            q = unit(q, q_weight, qw if norm_qk == "row" else key_dim)
+            k = unit(k, k_weight, kw if norm_qk == "row" else key_dim)
+        if norm_v:
+            v = unit(v, None, value_dim)
+        q_out.copy_(q.to(q_out.dtype))
+        if kcache is not None:
+            self.kv_store(k.to(kcache.dtype), v.to(vcache.dtype), kv_heads, key_dim, value_dim, row_pos, row_seq, seq_slot,
+                          block_table, kcache, vcache, block_size)
+
+    def selective_scan(self, x, dt, b_in, c_in, z, dt_bias, a_log, d_skip, state, out, seq_slot, cu_rows, batch):
+        a = -torch.exp(a_log)
+        for b in range(batch):
+            s = state[int(seq_slot[b])]  # [channels, n_state]
+            for r in range(int(cu_rows[b]), int(cu_rows[b + 1])):
+                step = torch.nn.functional.softplus(dt[r] + dt_bias, threshold=1e9)
+                xr, zr = x[r].float(), z[r].float()
+                s.mul_(torch.exp(step[:, None] * a)).add_((step * xr)[:, None] * b_in[r].float()[None, :])
+                y = s @ c_in[r].float() + d_skip * xr
+                out[r] = (y * zr / (1 + torch.exp(-zr))).to(out.dtype)
+
+    def memory_gates(self, i_in, f_in, i_bias, f_bias, cap, m_state, decay, take, floor, seq_slot, cu_rows, batch):
+        for b in range(batch):
+            m = m_state[int(seq_slot[b])]
+            for r in range(int(cu_rows[b]), int(cu_rows[b + 1])):
+                i = cap * torch.tanh((i_in[r] + i_bias) / cap)
+                f = torch.nn.functional.logsigmoid(cap * torch.tanh((f_in[r] + f_bias) / cap))
+                top = torch.maximum(f + m, i)
+                decay[r], take[r], floor[r] = torch.exp(f + m - top), torch.exp(i - top), torch.exp(-top)
+                m.copy_(top)
+
+    def memory_out(self, y, floor, z, weight, scale, den_eps, eps, out):
+        rows, heads = floor.shape
+        t = y.reshape(rows, heads, -1) * scale
+        o = t[:, :, :-1] / (torch.maximum(t[:, :, -1:].abs(), floor[:, :, None]) + den_eps)
+        o = (o / torch.sqrt((o * o).mean(-1, keepdim=True) + eps)).reshape(rows, -1)
+        out.copy_((o * weight * torch.sigmoid(z.float())).to(out.dtype))
 
     def rmsnorm_cols(self, src, weight, eps, out):
         v = src.float()
