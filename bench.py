@@ -38,6 +38,9 @@ design of the same sizes, whose gated delta rule (one decay a head) and attentio
 `--design sofinex`: the same for the design of differential attention under a sliding window, in turn with layers of
 windowed attention with a learned sink beside the gated delta rule; beside the Llama shape and beside the Mifidra
 design of the same sizes (the closest: the same attention kernel and delta rule, experts chosen within groups).
+`--design puzonex`: the same for the design of the selective scan, windowed attention with capped and biased scores, and
+attention whose values are its keys beside a matrix memory (per four layers two, one and one); beside the Llama shape
+and beside the Vafodra design of the same sizes (the closest: windowed attention with a sink beside a state-space scan).
 """
 from __future__ import annotations
 
@@ -182,6 +185,26 @@ def sofinex_config(width: int, layers: int, vocab: int) -> dict:
             "vocab": vocab, "width": width}
 
 
+def puzonex_config(width: int, layers: int, vocab: int) -> dict:
+    """Layer sizes of a real model for the design.  Per four layers: two selective scans (twice the width of channels, a
+    state of 16, four taps, step sizes through a sixteenth of the width); one layer of windowed attention whose values are
+    its keys (heads of 128, a fourth as many key heads, a window of 1 024, a table of 32 biases) beside a matrix memory
+    (heads of 256 x 512, half as wide in q and k as the model and as wide in v); one layer of windowed attention with
+    a sink and a logarithmic bias (the same heads and window).  Gated units of 3.5 times the width."""
+    heads = width // 128
+    shaped = {"dim": 128, "vdim": 128, "heads": heads, "kv_heads": max(1, heads // 4), "scale": 128 ** -0.5, "softcap": 30.0,
+              "mask": {"size": 1024}}
+    memory = {"heads": max(1, width // 512), "dim": 256, "vdim": 512, "gate_cap": 15.0}
+    mlp = {"kind": "dense", "ff": width * 7 // 2}
+    selective = {"type": "mamba1", "mlp": mlp,
+                 "mixer": {"inner": 2 * width, "state": 16, "dt_rank": width // 16, "conv": 4}}
+    parallel = {"type": "parallel", "mlp": mlp,
+                "mixer": {"left": {**shaped, "bias_max": 512, "bias_rows": 32}, "right": memory}}
+    attention = {"type": "attention", "mlp": mlp, "mixer": shaped}
+    made = [(selective, parallel, attention, selective)[i % 4] for i in range(layers)]
+    return {"architecture": "Puzonex", "layers": made, "norm": {"eps": 1e-5}, "vocab": vocab, "width": width}
+
+
 def design_run(args) -> int:
     import torch
 
@@ -199,8 +222,9 @@ def design_run(args) -> int:
         made = {"vafodra": lambda: lq.VafodraConfig.from_dict(vafodra_config(width, layers, vocab)),
                 "vupelorn": lambda: lq.VupelornConfig.from_dict(vupelorn_config(width, layers, vocab)),
                 "mifidra": lambda: lq.MifidraConfig.from_dict(mifidra_config(width, layers, vocab)),
-                "sofinex": lambda: lq.SofinexConfig.from_dict(sofinex_config(width, layers, vocab))}
-        closest = {"mifidra": "vafodra", "sofinex": "mifidra"}.get(args.design)
+                "sofinex": lambda: lq.SofinexConfig.from_dict(sofinex_config(width, layers, vocab)),
+                "puzonex": lambda: lq.PuzonexConfig.from_dict(puzonex_config(width, layers, vocab))}
+        closest = {"mifidra": "vafodra", "sofinex": "mifidra", "puzonex": "vafodra"}.get(args.design)
         beside = [(closest, made[closest]())] if closest else []
         for name, config in [(args.design, made[args.design]())] + beside + [("llama", lq.LlamaConfig.from_dict(llama))]:
             engine = lq.random_engine(config, seed=0, dtype=args.dtype, max_tokens=batch * 4096 + n_prefill + 64,
@@ -291,7 +315,7 @@ def main() -> int:
                     help="float32: the true 32-bit path (use --layers with the larger shapes)")
     ap.add_argument("--context", type=int, default=0,
                     help="tokens a sequence may hold (default: the shape's 8192); for decoding over longer prompts")
-    ap.add_argument("--design", choices=["vafodra", "vupelorn", "mifidra", "sofinex"], default=None,
+    ap.add_argument("--design", choices=["vafodra", "vupelorn", "mifidra", "sofinex", "puzonex"], default=None,
                     help="measure this design beside the Llama shape of equal size instead of the default workload")
     ap.add_argument("--design-widths", default="2048,4096", help="model widths of --design, with commas between them")
     args = ap.parse_args()
