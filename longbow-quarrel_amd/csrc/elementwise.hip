@@ -1194,6 +1194,30 @@ extern "C" int lq_bigram_add(float* x, const void* table, int table_dtype, const
   return 0;
 }
 
+template <typename T>
+__global__ __launch_bounds__(256) void sum_pieces_kernel(const float* __restrict__ src, int pieces, T* __restrict__ out, int ldo,
+                                                         int rows, int n) {
+  const long long total = (long long)rows * n, i = (long long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= total) return;
+  float v = src[i];
+  for (int p = 1; p < pieces; ++p) v += src[i + p * total];
+  const long long r = i / n;
+  out[r * ldo + i - r * n] = from_f32<T>(v);
+}
+
+// src [pieces, rows, n] dense: out [rows, n] (stride ldo) = their sum in ascending order
+extern "C" int lq_sum_pieces(const float* src, int pieces, void* out, int out_dtype, int ldo, int rows, int n,
+                             hipStream_t stream) {
+  LQ_REQUIRE(src && out && pieces > 0 && rows > 0 && n > 0 && ldo >= n, "sum_pieces: %d pieces of %d x %d, stride %d", pieces, rows, n, ldo);
+  const long long blocks = ((long long)rows * n + 255) / 256;
+  LQ_REQUIRE(blocks < (1ll << 31), "sum_pieces: too large");
+  if (out_dtype == LQ_F32) sum_pieces_kernel<float><<<(unsigned)blocks, 256, 0, stream>>>(src, pieces, (float*)out, ldo, rows, n);
+  else if (out_dtype == LQ_BF16) sum_pieces_kernel<bf16_t><<<(unsigned)blocks, 256, 0, stream>>>(src, pieces, (bf16_t*)out, ldo, rows, n);
+  else LQ_REQUIRE(false, "sum_pieces: unknown dtype %d", out_dtype);
+  LQ_CHECK_LAUNCH("sum_pieces");
+  return 0;
+}
+
 __global__ __launch_bounds__(256) void add_bias_kernel(float* __restrict__ x, const float* __restrict__ b, int width) {
   float* row = x + (long long)blockIdx.x * width;
   for (int i = threadIdx.x; i < width; i += 256) row[i] += b[i];

@@ -48,16 +48,18 @@ extern "C" int lq_linear_swiglu_supported(int in_dtype, int N, int K) {
 }
 
 // out[M, N/2] = silu(gate) * up where [gate | up] = x . W^T and W's N rows hold gate and up rows
-// interleaved in groups of 8 (rows 16j..16j+7 gate 8j..8j+7, rows 16j+8..16j+15 up 8j..8j+7).
+// interleaved in groups of 8 (rows 16j..16j+7 gate 8j..8j+7, rows 16j+8..16j+15 up 8j..8j+7).  `gelu`: the tanh form of
+// gelu in silu's place (bfloat16 out).
 extern "C" int lq_linear_swiglu(const void* x, const void* w, void* out, int in_dtype, int out_dtype, int M,
-                                int N, int K, int lda, int ldw, int ldc, int w_packed, hipStream_t stream) {
+                                int N, int K, int lda, int ldw, int ldc, int w_packed, int gelu, hipStream_t stream) {
+  LQ_REQUIRE(!gelu || out_dtype == LQ_BF16, "linear+swiglu: the gelu form leaves bfloat16");
   LQ_REQUIRE(M > 0 && N > 0 && K > 0, "linear+swiglu: sizes M=%d N=%d K=%d must be positive", M, N, K);
   LQ_REQUIRE(lda >= K && ldw >= K && ldc >= N / 2, "linear+swiglu: a row stride is smaller than its row");
   LQ_REQUIRE(x && w && out, "linear+swiglu: null pointer");
   LQ_REQUIRE(lq_linear_swiglu_supported(in_dtype, N, K) && lq_gemm_mfma_accepts(x, w, in_dtype, K, lda, ldw),
              "linear+swiglu: needs bfloat16, 16-byte aligned rows, K %% 8 == 0 and N %% 16 == 0");
   LQ_REQUIRE(!w_packed || (ldw == K && lq_weight_packable(in_dtype, N, K)), "linear+swiglu: this weight cannot be packed");
-  return lq_gemm_mfma(x, w, out, out_dtype, M, N, K, lda, ldw, ldc, 1, 1, 0, w_packed, stream);
+  return lq_gemm_mfma(x, w, out, out_dtype, M, N, K, lda, ldw, ldc, gelu ? 3 : 1, 1, 0, w_packed, stream);
 }
 
 // ------------------------------------------------------------------ the products around a norm (decoding)

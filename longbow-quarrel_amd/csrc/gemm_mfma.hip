@@ -63,14 +63,25 @@ __device__ inline void store_out<bf16_t>(bf16_t* p, float v) {
 // Epilogues.  EPI_SWIGLU expects the weight rows interleaved in groups of 8: rows 16j..16j+7 are
 // gate rows 8j..8j+7 and rows 16j+8..16j+15 the matching up rows, so that the lane holding gate
 // column c (c % 16 < 8) finds its up value 8 lanes further; it writes silu(gate) * up to
-// out[m][8j + c % 8], an [M, N / 2] matrix.
+// out[m][8j + c % 8], an [M, N / 2] matrix.  EPI_GEGLU is the same with the tanh form of gelu in silu's place.
 // EPI_RESIDUAL adds the product into C (the float32 residual stream, updated in place) and leaves, per
 // row, the sum of squares of the block's updated columns in a table, for the norm that follows.
-enum { EPI_NONE = 0, EPI_SWIGLU = 1, EPI_RESIDUAL = 2 };
+enum { EPI_NONE = 0, EPI_SWIGLU = 1, EPI_RESIDUAL = 2, EPI_GEGLU = 3 };
+constexpr bool is_glu(int epi) { return epi == EPI_SWIGLU || epi == EPI_GEGLU; }
 
 // silu(g) u = g u / (1 + e^-g), for 16-bit outputs: the hardware's exponential and reciprocal (an ulp or so
 // each, far below the rounding of the result) instead of a division and a library call per element
 __device__ inline float silu_mul(float g, float u) { return g * __builtin_amdgcn_rcpf(1.0f + __expf(-g)) * u; }
+
+// gelu(g) u with the tanh form: 0.5 (1 + tanh y) = 1 / (1 + e^(-2 y)), y = sqrt(2 / pi) (g + 0.044715 g^3), so it is silu
+// with another exponent
+template <int EPI>
+__device__ inline float glu_mul(float g, float u) {
+  if constexpr (EPI == EPI_GEGLU)
+    return g * __builtin_amdgcn_rcpf(1.0f + __expf(-1.5957691216057308f * fmaf(0.044715f * g * g, g, g))) * u;
+  else
+    return silu_mul(g, u);
+}
 
 // the value of the lane 8 places away within its row of 16 lanes (lane ^ 8), by a DPP rotation
 __device__ inline float from_lane_xor8(float v) {
@@ -89,11 +100,11 @@ __device__ inline void tile_epilogue(f32x16 (&acc)[WM][WN], TO* __restrict__ C, 
 #pragma unroll
       for (int e = 0; e < 16; ++e) {
         const int row = row0 + i * 32 + (e >> 2) * 8 + (lane >> 5) * 4 + (e & 3);
-        if (EPI == EPI_SWIGLU) {
+        if (is_glu(EPI)) {
           // gate column c (c % 16 < 8) and its up column c + 8 sit 8 lanes apart
           const float up = __shfl(acc[i][j][e], lane + 8, 64);
           if ((col & 15) < 8 && row < M && col + 8 < N)
-            store_out<TO>(C + (long long)row * ldc + ((col >> 4) << 3) + (col & 7), silu_mul(acc[i][j][e], up));
+            store_out<TO>(C + (long long)row * ldc + ((col >> 4) << 3) + (col & 7), glu_mul<EPI>(acc[i][j][e], up));
         } else {
           if (row < M && col < N) store_out<TO>(C + (long long)row * ldc + col, acc[i][j][e]);
         }
@@ -108,13 +119,13 @@ __device__ inline void tile_epilogue(f32x16 (&acc)[WM][WN], TO* __restrict__ C, 
 template <int WM, int WN, int BM, int BN, int EPI, int THREADS>
 __device__ inline void block_epilogue_16(f32x16 (&acc)[WM][WN], bf16_t* __restrict__ C, int ldc, int M, int N, int m0,
                                          int n0, int wrow, int wcol, int lane, int tid, bf16_t* tile) {
-  constexpr int OUT_W = EPI == EPI_SWIGLU ? BN / 2 : BN;
+  constexpr int OUT_W = is_glu(EPI) ? BN / 2 : BN;
 #pragma unroll
   for (int i = 0; i < WM; ++i)
 #pragma unroll
     for (int j = 0; j < WN; ++j) {
       const int col = wcol + j * 32 + (lane & 31);  // within the block tile
-      if constexpr (EPI == EPI_SWIGLU) {
+      if constexpr (is_glu(EPI)) {
         // Gate column c (c % 16 < 8) and its up column c + 8 sit 8 lanes apart.  Two rows at a time: the
         // gate lane takes the up value of the first row from its partner and gives it the gate value of the
         // second, so that every lane works out one product of the pair and no lane stands idle.
@@ -124,7 +135,7 @@ __device__ inline void block_epilogue_16(f32x16 (&acc)[WM][WN], bf16_t* __restri
         for (int e = 0; e < 16; e += 2) {
           const int row = wrow + i * 32 + (e >> 2) * 8 + (lane >> 5) * 4 + (e & 3) + (gate_lane ? 0 : 1);
           const float got = from_lane_xor8(gate_lane ? acc[i][j][e + 1] : acc[i][j][e]);
-          const float v = gate_lane ? silu_mul(acc[i][j][e], got) : silu_mul(got, acc[i][j][e + 1]);
+          const float v = gate_lane ? glu_mul<EPI>(acc[i][j][e], got) : glu_mul<EPI>(got, acc[i][j][e + 1]);
           tile[row * OUT_W + out_col] = f32_to_bf16(v);
         }
       } else {
@@ -136,7 +147,7 @@ __device__ inline void block_epilogue_16(f32x16 (&acc)[WM][WN], bf16_t* __restri
       }
     }
   __syncthreads();
-  const int n_out = EPI == EPI_SWIGLU ? N / 2 : N, c0 = EPI == EPI_SWIGLU ? n0 / 2 : n0;
+  const int n_out = is_glu(EPI) ? N / 2 : N, c0 = is_glu(EPI) ? n0 / 2 : n0;
   const bool vec = ldc % 8 == 0 && ((uintptr_t)C % 16) == 0;
   constexpr int CPR = OUT_W / 8;  // 16-byte chunks a row
   for (int c = tid; c < BM * CPR; c += THREADS) {
@@ -556,7 +567,7 @@ __global__ __launch_bounds__(GM * GN * 64, 2) void gemm_bf16_pipelined_kernel(
     if (group == 0) asm volatile("s_barrier" ::: "memory");
   }
   if constexpr (sizeof(TO) == 2) {
-    constexpr int OUT_BYTES = S::BM * (EPI == EPI_SWIGLU ? S::BN / 2 : S::BN) * 2;
+    constexpr int OUT_BYTES = S::BM * (is_glu(EPI) ? S::BN / 2 : S::BN) * 2;
     static_assert(OUT_BYTES <= S::LDS_BYTES, "the output tile must fit the stages");
     __syncthreads();  // every wave is past its last fragment read
     block_epilogue_16<WM, WN, S::BM, S::BN, EPI, S::NW * 64>(acc, C, ldc, M, N, m0, n0, wm * WM * 32, wn * WN * 32, lane,
@@ -663,9 +674,9 @@ __global__ __launch_bounds__(KW * 64) void gemm_bf16_skinny_kernel(const bf16_t*
 #pragma unroll
         for (int w = 0; w < KW; ++w) s += red[w][t * 256 + e * 64 + lane];
         const int row = t * 16 + g * 4 + e;
-        if (EPI == EPI_SWIGLU) {
+        if (is_glu(EPI)) {
           const float up = __shfl(s, lane + 8, 64);
-          if (c16 < 8 && row < M && col + 8 < N) store_out<TO>(C + (long long)row * ldc + (n0 >> 1) + c16, silu_mul(s, up));
+          if (c16 < 8 && row < M && col + 8 < N) store_out<TO>(C + (long long)row * ldc + (n0 >> 1) + c16, glu_mul<EPI>(s, up));
         } else {
           if (row < M && col < N) store_out<TO>(C + (long long)row * ldc + col, s);
         }
@@ -813,10 +824,10 @@ __global__ __launch_bounds__(KW * 64) void gemm_bf16_skinny_v3_kernel(const bf16
     const int col = col_begin + t * 16 + c16;
     const int row = (v >> 2) * 16 + g * 4 + (v & 3);
     if (SCALED) s *= rstd_sh[min(row, M - 1)];
-    if (EPI == EPI_SWIGLU) {
+    if (is_glu(EPI)) {
       const float up = __shfl(s, lane + 8, 64);
       if (c16 < 8 && row < M && col + 8 < col_end)
-        store_out<TO>(C + (long long)row * ldc + ((col_begin + t * 16) >> 1) + c16, silu_mul(s, up));
+        store_out<TO>(C + (long long)row * ldc + ((col_begin + t * 16) >> 1) + c16, glu_mul<EPI>(s, up));
     } else if constexpr (EPI == EPI_RESIDUAL) {
       static_assert(EPI != EPI_RESIDUAL || sizeof(TO) == 4, "the residual stream is float32");
       float fresh = 0.f;
@@ -933,7 +944,7 @@ int launch_skinny_v3(const void* X, const void* W, void* C, int M, int N, int K,
   constexpr int KW = v3_kw(MT);
   LQ_REQUIRE(!packed || (K % 64 == 0 && N % 8 == 0), "linear: a packed weight has K in 64s and rows in eights");
   int cols, grid;
-  v3_runs(N, lq_compute_units() / splits, EPI == EPI_SWIGLU ? 16 : 8, cols, grid);
+  v3_runs(N, lq_compute_units() / splits, is_glu(EPI) ? 16 : 8, cols, grid);
   const int ksteps = lq_ceil_div(K, 32);
   // an even number of 32-k steps a wave: its slice starts at a multiple of 64, where a packed weight's slabs do
   const int ks_per_wave = (lq_ceil_div(ksteps, KW * splits) + 1) / 2 * 2;
@@ -1128,7 +1139,7 @@ int dispatch(const void* x, const void* w, void* out, int M, int N, int K, int l
       const int tn = lq_ceil_div(N, 256), rest = (tm * tn) % cus;
       if (N % 256 == 0 && tm * tn > cus && 4 * rest >= cus && rest % tm == 0 && 2 * rest <= cus + cus / 8) {
         const int n1 = (tn - rest / tm) * 256, n2 = N - n1;
-        const int col2 = EPI == EPI_SWIGLU ? n1 / 2 : n1;  // where the second launch's columns start in out
+        const int col2 = is_glu(EPI) ? n1 / 2 : n1;  // where the second launch's columns start in out
         int rc = launch_pipelined<4, 2, 2, 4, 64, 2, EPI, TO, true>(x, w, out, M, n1, K, lda, ldw, ldc, 1, 0, stream, packed);
         if (rc != 0) return rc;
         return launch_pipelined<4, 2, 2, 2, 64, 2, EPI, TO, true>(x, (const bf16_t*)w + (long long)n1 * ldw,
@@ -1213,13 +1224,17 @@ int lq_gemm_mfma(const void* x, const void* w, void* out, int out_dtype, int M, 
       return dispatch<EPI_NONE, float>(x, w, out, M, N, K, lda, ldw, ldc, splits, split_stride, stream, packed);
     if (out_dtype == LQ_BF16)
       return dispatch<EPI_NONE, bf16_t>(x, w, out, M, N, K, lda, ldw, ldc, splits, split_stride, stream, packed);
-  } else if (epilogue == EPI_SWIGLU) {
+  } else if (epilogue == EPI_SWIGLU || epilogue == EPI_GEGLU) {
     if (N % 16 != 0) {
       lq_set_error("linear+swiglu: %d interleaved rows are not a multiple of 16", N);
       return -1;
     }
-    if (out_dtype == LQ_F32) return dispatch<EPI_SWIGLU, float>(x, w, out, M, N, K, lda, ldw, ldc, 1, 0, stream, packed);
-    if (out_dtype == LQ_BF16) return dispatch<EPI_SWIGLU, bf16_t>(x, w, out, M, N, K, lda, ldw, ldc, 1, 0, stream, packed);
+    if (epilogue == EPI_GEGLU) {
+      if (out_dtype == LQ_BF16) return dispatch<EPI_GEGLU, bf16_t>(x, w, out, M, N, K, lda, ldw, ldc, 1, 0, stream, packed);
+    } else {
+      if (out_dtype == LQ_F32) return dispatch<EPI_SWIGLU, float>(x, w, out, M, N, K, lda, ldw, ldc, 1, 0, stream, packed);
+      if (out_dtype == LQ_BF16) return dispatch<EPI_SWIGLU, bf16_t>(x, w, out, M, N, K, lda, ldw, ldc, 1, 0, stream, packed);
+    }
   }
   lq_set_error("linear: unknown out dtype %d or epilogue %d", out_dtype, epilogue);
   return -1;

@@ -112,6 +112,87 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
   store_as<T>(out + (long long)r * ldo + c, activate(acc, act));
 }
 
+// The same for rows whose channels come in fours on 16 (or 8) bytes: a thread owns four channels of ROWS neighbouring rows
+// of the step and keeps their last TAPS - 1 inputs in registers, so an input is read once and not once a tap.  The sums
+// are the kernel's above, in its order.  `single`: every sequence brings one row, and the thread that has read a
+// sequence's old inputs also moves them on.
+template <typename T>
+__device__ inline float4 load4(const T* p);
+template <>
+__device__ inline float4 load4<float>(const float* p) { return *(const float4*)p; }
+template <>
+__device__ inline float4 load4<bf16_t>(const bf16_t* p) {
+  const uint2 v = *(const uint2*)p;
+  return make_float4(__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16),
+                     __uint_as_float(v.y & 0xffff0000u));
+}
+template <typename T>
+__device__ inline void store4(T* p, float4 v);
+template <>
+__device__ inline void store4<float>(float* p, float4 v) { *(float4*)p = v; }
+template <>
+__device__ inline void store4<bf16_t>(bf16_t* p, float4 v) {
+  uint2 packed;
+  packed.x = (uint32_t)f32_to_bf16(v.x).bits | ((uint32_t)f32_to_bf16(v.y).bits << 16);
+  packed.y = (uint32_t)f32_to_bf16(v.z).bits | ((uint32_t)f32_to_bf16(v.w).bits << 16);
+  *(uint2*)p = packed;
+}
+
+template <typename T, int TAPS, int ROWS>
+__global__ __launch_bounds__(256) void causal_conv4_kernel(const T* __restrict__ x, int ldx, const float* __restrict__ w,
+                                                           const float* __restrict__ bias, float* __restrict__ state,
+                                                           T* __restrict__ out, int ldo, int rows, int C,
+                                                           const int* __restrict__ row_seq, const int* __restrict__ row_pos,
+                                                           const int* __restrict__ seq_slot,
+                                                           const int* __restrict__ seq_start, int act, int single) {
+  const int c = (blockIdx.x * 64 + threadIdx.x) * 4;
+  const int first = (blockIdx.y * 4 + threadIdx.y) * ROWS;
+  if (c >= C || first >= rows) return;
+  float wt[4][TAPS];
+#pragma unroll
+  for (int e = 0; e < 4; ++e)
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) wt[e][j] = w[(long long)(c + e) * TAPS + j];
+  float4 bv = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (bias != nullptr) bv = *(const float4*)(bias + c);
+  float4 hist[TAPS];  // hist[j]: the input TAPS - 1 - j tokens before the row; the last is the row's own
+  int before = -1;    // the sequence that hist belongs to
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) {
+    const int r = first + i;
+    if (r >= rows) break;
+    const int b = row_seq[r];
+    const long long slot = (long long)seq_slot[b] * (TAPS - 1);
+    if (b != before) {  // a tile's first row, or another sequence's
+      const int since = row_pos[r] - seq_start[b];  // rows of this step before this one, in its sequence
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) {
+        const int back = TAPS - 1 - j;
+        hist[j] = back <= since ? load4<T>(x + (long long)(r - back) * ldx + c)
+                                : *(const float4*)(state + (slot + TAPS - 1 - (back - since)) * C + c);
+      }
+      before = b;
+    } else {
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) hist[j] = hist[j + 1];
+    }
+    hist[TAPS - 1] = load4<T>(x + (long long)r * ldx + c);
+    float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) {
+      acc.x = fmaf(wt[0][j], hist[j].x, acc.x), acc.y = fmaf(wt[1][j], hist[j].y, acc.y);
+      acc.z = fmaf(wt[2][j], hist[j].z, acc.z), acc.w = fmaf(wt[3][j], hist[j].w, acc.w);
+    }
+    if (bias != nullptr) acc.x += bv.x, acc.y += bv.y, acc.z += bv.z, acc.w += bv.w;
+    store4<T>(out + (long long)r * ldo + c,
+              make_float4(activate(acc.x, act), activate(acc.y, act), activate(acc.z, act), activate(acc.w, act)));
+    if (single) {
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) *(float4*)(state + (slot + j) * C + c) = hist[j + 1];
+    }
+  }
+}
+
 // The state after the step: the last taps - 1 inputs of each sequence (old ones move up where the step brought fewer).
 template <typename T>
 __global__ __launch_bounds__(256) void conv_state_kernel(const T* __restrict__ x, int ldx, float* __restrict__ state,
@@ -1031,7 +1112,30 @@ template <typename T>
 static int launch_causal_conv(const T* x, int ldx, const float* w, const float* bias, float* state, T* out, int ldo, int rows,
                               int C, int taps, const int* row_seq, const int* row_pos, const int* seq_slot,
                               const int* seq_start, const int* cu_rows, int batch, int act, hipStream_t stream) {
-  for (int r0 = 0; r0 < rows; r0 += 65535) {
+  const bool fours = C % 4 == 0 && ldx % 4 == 0 && ldo % 4 == 0 && taps >= 2 && taps <= 4 && rows <= 65535 * 4 &&
+                     (uintptr_t)x % (4 * sizeof(T)) == 0 && (uintptr_t)out % (4 * sizeof(T)) == 0 &&
+                     (uintptr_t)state % 16 == 0 && (uintptr_t)bias % 16 == 0;
+  if (fours) {
+    const bool single = rows == batch;  // (every sequence of a step brings at least one row)
+    const int per = rows >= 512 ? 8 : 1;
+    const dim3 grid(lq_ceil_div(C, 256), lq_ceil_div(rows, 4 * per)), block(64, 4);
+#define LQ_CONV4(TAPS, ROWS)                                                                                              \
+  causal_conv4_kernel<T, TAPS, ROWS><<<grid, block, 0, stream>>>(x, ldx, w, bias, state, out, ldo, rows, C, row_seq,      \
+                                                                 row_pos, seq_slot, seq_start, act, single ? 1 : 0)
+#define LQ_CONV4_TAPS(TAPS)           \
+  do {                                \
+    if (per == 8) LQ_CONV4(TAPS, 8);  \
+    else LQ_CONV4(TAPS, 1);           \
+  } while (0)
+    if (taps == 2) LQ_CONV4_TAPS(2);
+    else if (taps == 3) LQ_CONV4_TAPS(3);
+    else LQ_CONV4_TAPS(4);
+#undef LQ_CONV4_TAPS
+#undef LQ_CONV4
+    LQ_CHECK_LAUNCH("causal_conv(fours)");
+    if (single) return 0;
+  }
+  for (int r0 = 0; !fours && r0 < rows; r0 += 65535) {
     const int nr = rows - r0 < 65535 ? rows - r0 : 65535;
     causal_conv_kernel<T><<<dim3(lq_ceil_div(C, 256), nr), 256, 0, stream>>>(
         x, ldx, w, bias, state, out + (long long)r0 * ldo, ldo, C, taps, row_seq + r0, row_pos + r0, seq_slot, seq_start,

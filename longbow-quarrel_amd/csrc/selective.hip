@@ -222,28 +222,34 @@ void dispatch_selective(const void* x, const float* dt, const void* Bm, const vo
 // Per head, with i = cap tanh((raw_i + b_i) / cap) and f = log sigmoid(cap tanh((raw_f + b_f) / cap)) the logarithms of
 // the gates and a running maximum m (zero before the first token):
 //   m_t = max(f_t + m_(t-1), i_t);   decay = exp(f_t + m_(t-1) - m_t);   take = exp(i_t - m_t);   floor = exp(-m_t).
-// One wavefront a (sequence, head), 64 tokens at a time: a token is the map m -> max(F + m, I) with (F, I) = (f, i), maps
-// compose to maps of the same form, so the running maxima of 64 tokens are a scan over the lanes.
+// A workgroup of WAVES wavefronts a (sequence, head), 64 tokens a wavefront at a time: a token is the map m -> max(F + m, I)
+// with (F, I) = (f, i), maps compose to maps of the same form, so the running maxima of 64 tokens are a scan over the
+// lanes, and a wavefront's start is the wavefronts' maps before it applied to the chunk's.
 __device__ inline float soft_cap_f(float v, float cap) { return cap * tanhf(v / cap); }
 
-__global__ __launch_bounds__(64) void memory_gates_kernel(const float* __restrict__ zi, int ldi, const float* __restrict__ zf,
-                                                          int ldf, const float* __restrict__ bi, const float* __restrict__ bf,
-                                                          float cap, float* __restrict__ m_state, float* __restrict__ decay,
-                                                          float* __restrict__ take, float* __restrict__ floor_out, int heads,
-                                                          const int* __restrict__ seq_slot, const int* __restrict__ cu_rows) {
-  const int b = blockIdx.x / heads, h = blockIdx.x % heads, lane = threadIdx.x;
+template <int WAVES>
+__global__ __launch_bounds__(64 * WAVES) void memory_gates_kernel(const float* __restrict__ zi, int ldi,
+                                                                  const float* __restrict__ zf, int ldf,
+                                                                  const float* __restrict__ bi, const float* __restrict__ bf,
+                                                                  float cap, float* __restrict__ m_state,
+                                                                  float* __restrict__ decay, float* __restrict__ take,
+                                                                  float* __restrict__ floor_out, int heads,
+                                                                  const int* __restrict__ seq_slot,
+                                                                  const int* __restrict__ cu_rows) {
+  __shared__ float whole_f[WAVES], whole_i[WAVES];
+  const int b = blockIdx.x / heads, h = blockIdx.x % heads, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   float* mp = m_state + (long long)seq_slot[b] * heads + h;
-  float m = *mp;
+  float m = *mp;  // the maximum before the chunk (every thread holds it)
   const long long r0 = cu_rows[b], r1 = cu_rows[b + 1];
-  for (long long c0 = r0; c0 < r1; c0 += 64) {
-    const long long r = c0 + lane;
+  for (long long c0 = r0; c0 < r1; c0 += 64 * WAVES) {
+    const long long r = c0 + threadIdx.x;
     const bool live = r < r1;
     float i = -INFINITY, f = 0.f;  // (a lane past the end maps m to itself)
     if (live) {
       i = soft_cap_f(zi[r * ldi + h] + bi[h], cap);
       f = -softplus_f(-soft_cap_f(zf[r * ldf + h] + bf[h], cap));
     }
-    float F = f, I = i;  // the composition of this lane's token with all before it in the chunk
+    float F = f, I = i;  // the composition of this lane's token with all before it in the wavefront
 #pragma unroll
     for (int off = 1; off < 64; off <<= 1) {
       const float Fb = __shfl_up(F, off, 64), Ib = __shfl_up(I, off, 64);
@@ -252,17 +258,27 @@ __global__ __launch_bounds__(64) void memory_gates_kernel(const float* __restric
         F += Fb;
       }
     }
-    const float top = fmaxf(F + m, I);
+    float start = m;
+    if constexpr (WAVES > 1) {
+      if (lane == 63) whole_f[wave] = F, whole_i[wave] = I;
+      __syncthreads();
+      for (int w = 0; w < WAVES; ++w) {
+        if (w == wave) start = m;
+        m = fmaxf(whole_f[w] + m, whole_i[w]);
+      }
+      __syncthreads();  // (the next chunk writes the maps anew)
+    }
+    const float top = fmaxf(F + start, I);
     float before = __shfl_up(top, 1, 64);
-    if (lane == 0) before = m;
+    if (lane == 0) before = start;
     if (live) {
       decay[r * heads + h] = expf(f + before - top);
       take[r * heads + h] = expf(i - top);
       floor_out[r * heads + h] = expf(-top);
     }
-    m = __shfl(top, 63, 64);
+    if constexpr (WAVES == 1) m = __shfl(top, 63, 64);
   }
-  if (lane == 0) *mp = m;
+  if (threadIdx.x == 0) *mp = m;
 }
 
 // The memory's answer from the scan's results.  y [rows, heads * (P + 1)]: a head's S^T q and, in its last column, n . q,
@@ -348,14 +364,19 @@ extern "C" int lq_selective_scan(const void* x, int ldx, const float* dt, int ld
   return 0;
 }
 
-// zi and zf [rows, heads] (raw logits), bi and bf [heads], m_state [slots, heads]; decay, take and floor [rows, heads] dense
+// zi and zf [rows, heads] (raw logits), bi and bf [heads], m_state [slots, heads]; decay, take and floor [rows, heads] dense;
+// `rows` all sequences' rows together (for the launch's shape alone)
 extern "C" int lq_memory_gates(const float* zi, int ldi, const float* zf, int ldf, const float* bi, const float* bf, float cap,
                                float* m_state, float* decay, float* take, float* floor_out, int heads, const int* seq_slot,
-                               const int* cu_rows, int batch, hipStream_t stream) {
-  LQ_REQUIRE(heads > 0 && batch > 0 && cap > 0.f && ldi >= heads && ldf >= heads, "memory_gates: %d heads, cap %g", heads, (double)cap);
+                               const int* cu_rows, int batch, int rows, hipStream_t stream) {
+  LQ_REQUIRE(rows >= 0 && heads > 0 && batch > 0 && cap > 0.f && ldi >= heads && ldf >= heads, "memory_gates: %d heads, cap %g", heads, (double)cap);
   LQ_REQUIRE(zi && zf && bi && bf && m_state && decay && take && floor_out && seq_slot && cu_rows, "memory_gates: null pointer");
-  memory_gates_kernel<<<(unsigned)(batch * heads), 64, 0, stream>>>(zi, ldi, zf, ldf, bi, bf, cap, m_state, decay, take, floor_out,
-                                                                    heads, seq_slot, cu_rows);
+#define LQ_GATES(WAVES)                                                                                                     \
+  memory_gates_kernel<WAVES><<<(unsigned)(batch * heads), 64 * WAVES, 0, stream>>>(zi, ldi, zf, ldf, bi, bf, cap, m_state, decay, \
+                                                                                   take, floor_out, heads, seq_slot, cu_rows)
+  if (rows > 64ll * batch) LQ_GATES(16);  // (some sequence brings more than a wavefront's tokens)
+  else LQ_GATES(1);
+#undef LQ_GATES
   LQ_CHECK_LAUNCH("memory_gates");
   return 0;
 }

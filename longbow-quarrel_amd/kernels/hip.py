@@ -56,7 +56,7 @@ def load_library() -> ctypes.CDLL:
     # launch itself is 3).
     vp, ci, cl, cf = c_void_p, c_int, c_longlong, c_float
     lib.lq_linear.argtypes = [vp, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci, ci, cl, ci, ci, vp]
-    lib.lq_linear_swiglu.argtypes = [vp, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci, ci, vp]
+    lib.lq_linear_swiglu.argtypes = [vp, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci, ci, ci, vp]
     lib.lq_rmsnorm.argtypes = [vp, vp, ci, ci, cl, vp, cf, vp, ci, ci, ci, vp]
     lib.lq_attention.argtypes = [vp, ci, vp, ci, ci, ci, ci, ci, ci, ci, vp, vp, vp, vp, vp, ci, vp, vp, ci, cf, ci, ci, ci,
                                  vp, cl, vp, cl, vp, vp, ci, ci, vp, ci, ci, cl, ci, vp]
@@ -293,6 +293,16 @@ class HipKernels:
         self._check(self.lib.lq_cast(_ptr(src), c_int(_code(src)), _ptr(out), c_int(_code(out)),
                                      c_longlong(src.numel()), self.stream))
 
+    def sum_pieces(self, pieces: torch.Tensor, out: torch.Tensor) -> None:
+        """out [rows, n] (any dtype, any row stride) = the sum over the first axis of pieces [p, rows, n] (float32, dense), in
+        ascending order: a product that shared K over blocks, added up."""
+        self._dev(pieces, out)
+        ro, no, ldo = self._mat(out, "sum_pieces: out")
+        if pieces.dtype != torch.float32 or pieces.dim() != 3 or not pieces.is_contiguous() or tuple(pieces.shape[1:]) != (ro, no):
+            raise KernelLibraryError("sum_pieces: pieces float32 [p, rows, n], out [rows, n]")
+        self._check(self.lib.lq_sum_pieces(_ptr(pieces), c_int(pieces.shape[0]), _ptr(out), c_int(_code(out)), c_int(ldo),
+                                           c_int(ro), c_int(no), self.stream))
+
     @query
     def linear_pieces(self, dtype: torch.dtype, m: int, n: int, k: int) -> int:
         """In how many pieces `linear` would like to leave this product (1: whole).  A caller whose
@@ -388,8 +398,9 @@ class HipKernels:
             return False
         return bool(self.lib.lq_linear_swiglu_supported(c_int(_DTYPE_CODE[dtype]), c_int(rows_out), c_int(k)))
 
-    def linear_swiglu(self, x: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> None:
-        """out[M, I] = silu(gate) * up with [gate | up] = x . w^T, in one kernel.  w [2 I, K] holds the
+    def linear_swiglu(self, x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, activation: str = "silu") -> None:
+        """out[M, I] = silu(gate) * up with [gate | up] = x . w^T, in one kernel; `activation` "gelu_tanh": the tanh form
+        of gelu in silu's place (bfloat16 out).  w [2 I, K] holds the
         gate and up rows interleaved in groups of 8: rows 16j..16j+7 gate 8j..8j+7, rows 16j+8..16j+15
         up 8j..8j+7 (see `interleave_gate_up`)."""
         m, k, ldx = self._mat(x, "linear_swiglu: x")
@@ -398,8 +409,10 @@ class HipKernels:
         if kw != k or mo != m or no != n // 2 or n % 16 != 0 or x.dtype != w.dtype:
             raise KernelLibraryError(
                 f"linear_swiglu: x {tuple(x.shape)}, w {tuple(w.shape)}, out {tuple(out.shape)} do not fit")
+        if activation not in ("silu", "gelu_tanh"):
+            raise KernelLibraryError(f"linear_swiglu: activation {activation!r}")
         rc = self.lib.lq_linear_swiglu(x.data_ptr(), w.data_ptr(), out.data_ptr(), _code(x), _code(out), m, n, k,
-                                       ldx, ldw, ldc, _packed(w), self.stream)
+                                       ldx, ldw, ldc, _packed(w), 1 if activation == "gelu_tanh" else 0, self.stream)
         if rc:
             self._check(rc)
 
@@ -1026,7 +1039,7 @@ class HipKernels:
         self._check(self.lib.lq_memory_gates(
             _ptr(i_in), c_int(self._rows2d(i_in, "i")), _ptr(f_in), c_int(self._rows2d(f_in, "f")), _ptr(i_bias), _ptr(f_bias),
             c_float(cap), _ptr(m_state), _ptr(decay), _ptr(take), _ptr(floor), c_int(heads), _ptr(seq_slot), _ptr(cu_rows),
-            c_int(batch), self.stream))
+            c_int(batch), c_int(rows), self.stream))
 
     def memory_out(self, y: torch.Tensor, floor: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, scale: float,
                    den_eps: float, eps: float, out: torch.Tensor) -> None:

@@ -551,6 +551,20 @@ def project_delta(kn, ctx: StepContext, x: torch.Tensor, w: torch.Tensor) -> tor
     return out
 
 
+def project_narrow(kn, ctx: StepContext, x: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> None:
+    """out = x . w^T for a weight of few rows, whose tiles alone would leave most of the chip idle: where the kernels would
+    share K over blocks, they do, and the pieces are added up into `out` (in its own dtype)."""
+    rows, n = x.shape[0], w.shape[0]
+    add = getattr(kn, "sum_pieces", None)
+    pieces = kn.linear_pieces(x.dtype, rows, n, x.shape[1]) if add is not None and w.dtype == x.dtype else 1
+    if pieces <= 1:
+        project(kn, ctx, x, w, out)
+        return
+    parts = ctx.ws.alloc((pieces, rows, n), torch.float32)
+    kn.linear(x, w, parts)
+    add(parts, out)
+
+
 def product_weight(env: BuildEnv, w: torch.Tensor):
     """A weight [N, K] as the kernels' products like to hold it, asked once when weights are bound: what
     `kernels.pack_weight` makes of it (something that `linear` and its siblings take in a tensor's place and that

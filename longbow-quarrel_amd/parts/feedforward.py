@@ -72,7 +72,8 @@ class SwiGLU(FeedForward):
 @FEED_FORWARDS.register("glu")
 class GatedLinearUnit(FeedForward):
     """down(act(gate(h)) * up(h)) with a choice of `activation` ("relu", "silu", "gelu_tanh").  gate and up are one
-    matrix product whose 32-bit result the activation kernel reads.  With `bias` every projection has one
+    matrix product whose 32-bit result the activation kernel reads; with "gelu_tanh" and no bias, in a bfloat16 run, the
+    product's epilogue applies it (gate and up rows interleaved when weights are bound).  With `bias` every projection has one
     (`<name>.b`): the activation kernel adds gate's and up's; down's is one more column of its weight, which meets a
     column of ones that the activation kernel leaves behind its result."""
 
@@ -91,6 +92,7 @@ class GatedLinearUnit(FeedForward):
         self.w_gate_up: Optional[torch.Tensor] = None
         self.w_down: Optional[torch.Tensor] = None
         self.b_gate_up: Optional[torch.Tensor] = None
+        self.fused = False
 
     def tensor_specs(self) -> List[TensorSpec]:
         specs = [
@@ -109,7 +111,13 @@ class GatedLinearUnit(FeedForward):
         gate, up = tensors[self.names["gate"]], tensors[self.names["up"]]
         if gate.dtype != up.dtype:
             raise ValueError(f"{self.names['gate']}: gate and up projections are stored in different dtypes")
-        self.w_gate_up = product_weight(env, torch.cat([gate, up], dim=0))
+        kn = env.kernels
+        self.fused = self.activation == "gelu_tanh" and not self.bias and gate.dtype == env.dtype == torch.bfloat16 and \
+            self.inner % 8 == 0 and getattr(kn, "linear_swiglu_supported", lambda *a: False)(gate.dtype, 2 * self.inner, self.width)
+        if self.fused:
+            self.w_gate_up = product_weight(env, kn.interleave_gate_up(gate, up))
+        else:
+            self.w_gate_up = product_weight(env, torch.cat([gate, up], dim=0))
         down = tensors[self.names["down"]]
         if self.bias:
             self.b_gate_up = torch.cat([tensors[self.names["gate"] + ".b"], tensors[self.names["up"] + ".b"]]).contiguous()
@@ -122,6 +130,13 @@ class GatedLinearUnit(FeedForward):
     def forward(self, h, ctx: StepContext, out: Optional[torch.Tensor] = None) -> torch.Tensor:
         kn = ctx.kernels
         rows = h.shape[0]
+        if self.fused:
+            act = ctx.ws.alloc((rows, self.inner), ctx.dtype)
+            kn.linear_swiglu(h, self.w_gate_up, act, activation=self.activation)
+            if out is None:
+                out = ctx.ws.alloc((rows, self.width), torch.float32)
+            project(kn, ctx, act, self.w_down, out)
+            return out
         gu = ctx.ws.alloc((rows, 2 * self.inner), torch.float32)
         project(kn, ctx, h, self.w_gate_up, gu)
         if self.bias:

@@ -13,7 +13,7 @@ from typing import Dict, List, Mapping, Optional
 import torch
 
 from .base import (MIXERS, VECTOR32, BuildEnv, Mixer, MultiCache, MultiNeed, StateNeed, StepContext, TensorSpec,
-                   product_weight, project)
+                   product_weight, project, project_narrow)
 
 
 def _round4(n: int) -> int:
@@ -185,7 +185,7 @@ class Mamba1(_Recurrent):
         kn.causal_conv(u[:, :c], self.conv_w, self.conv_b, conv_state, x, ctx.row_pos, ctx.row_seq, ctx.seq_slot,
                        ctx.seq_start, ctx.seq_len, ctx.cu_rows, ctx.batch, activation="silu")
         low = ctx.ws.alloc((rows, _round8(r + 2 * n)), ctx.dtype)[:, : r + 2 * n]
-        project(kn, ctx, x, self.w_x, low)
+        project_narrow(kn, ctx, x, self.w_x, low)
         dt = ctx.ws.alloc((rows, _round4(c)), torch.float32)[:, :c]
         project(kn, ctx, low[:, :r], self.w_dt, dt)
         y = ctx.ws.alloc((rows, _round8(c)), ctx.dtype)[:, :c]

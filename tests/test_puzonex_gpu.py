@@ -433,6 +433,68 @@ def test_lookup_with_sinusoids(kn, width, dtype):
     assert float((want[3] - want[4]).abs().max()) > 0.1  # one token at two places
 
 
+@pytest.mark.parametrize("rows,k,inner", [(1, 512, 64), (5, 64, 40), (16, 1024, 2048), (40, 1024, 2048), (300, 512, 2048),
+                                          (130, 96, 24), (700, 2048, 2816), (2048, 1024, 4096)])
+def test_gated_unit_with_the_tanh_gelu_in_the_products_epilogue(kn, rows, k, inner):
+    """Every way the product can take (few rows, some rows, prompts, a remainder of columns in a launch of its own), dense
+    and packed weights; the other activation of that epilogue is another function."""
+    x, gate, up = rnd(rows, k, seed=1).to(torch.bfloat16), rnd(inner, k, seed=2, std=2 / k ** 0.5), rnd(inner, k, seed=3, std=k ** -0.5)
+    gate, up = gate.to(torch.bfloat16), up.to(torch.bfloat16)
+    g, u = x.float() @ gate.float().T, x.float() @ up.float().T
+    want = pp.gelu_tanh(g.double()) * u.double()
+    assert kn.linear_swiglu_supported(torch.bfloat16, 2 * inner, k)
+    w = kn.interleave_gate_up(dev(gate, torch.bfloat16), dev(up, torch.bfloat16))
+    for weight in (w, kn.pack_weight(w)):
+        out = torch.zeros((rows, inner), dtype=torch.bfloat16, device=DEV)
+        kn.linear_swiglu(dev(x, torch.bfloat16), weight, out, activation="gelu_tanh")
+        assert pc.err(out, want) < 6e-3
+    small = want.abs() < 0.1 * want.abs().max()  # (the far tail of the negative gates included)
+    assert float((out.cpu().double() - want)[small].abs().max() / want.abs().max()) < 2e-3
+    kn.linear_swiglu(dev(x, torch.bfloat16), w, out)
+    assert pc.err(out, want) > 2e-2
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_pieces_of_a_product_added_up(kn, dtype):
+    pieces = rnd(5, 37, 21, seed=1)
+    out = torch.full((37, 30), 9.0, dtype=dtype, device=DEV)
+    kn.sum_pieces(dev(pieces), out[:, :21])
+    assert pc.err(out[:, :21], pieces.double().sum(0)) < (1e-6 if dtype == torch.float32 else 5e-3)
+    assert bool((out[:, 21:] == 9.0).all())
+
+
+def test_short_convolution_of_many_rows(kn):
+    """Rows enough for several a thread: two long sequences and a short one, whose rows meet inside a thread's run, from
+    states that an earlier step left; the same bits as row by row."""
+    C, taps, lens = 136, 4, (301, 3, 290)
+    w, b = dev(rnd(C, taps, seed=1)), dev(rnd(C, seed=2))
+    for dtype in (torch.float32, torch.bfloat16):
+        x, n = dev(rnd(sum(lens), C, seed=3), dtype), sum(lens)
+        before = rnd(3, taps - 1, C, seed=4)
+        start = [7, 0, 2]
+        before[1] = 0  # (the second sequence is at its start)
+        cu = i32([0] + np.cumsum(lens).tolist())
+        pos = [s + i for s, l in zip(start, lens) for i in range(l)]
+        seq = [i for i, l in enumerate(lens) for _ in range(l)]
+        out, state = torch.zeros((n, C), dtype=dtype, device=DEV), dev(before)
+        kn.causal_conv(x, w, b, state, out, i32(pos), i32(seq), i32([0, 1, 2]), i32(start),
+                       i32([s + l for s, l in zip(start, lens)]), cu, 3)
+        at = 0
+        for i, l in enumerate(lens):
+            hist = torch.cat([before[i].double(), x[at : at + l].cpu().double()])
+            want = pp.short_conv(hist, w.cpu().double(), b.cpu().double())[taps - 1 :]
+            assert pc.err(out[at : at + l], want) < (2e-6 if dtype == torch.float32 else 1e-2)
+            assert pc.err(state[i], hist[-(taps - 1) :]) == 0
+            at += l
+        single = dev(before)
+        for t in range(3):  # single tokens of all three: the same bits
+            rows = [0 + t, 301 + t, 304 + t]
+            one = torch.zeros((3, C), dtype=dtype, device=DEV)
+            kn.causal_conv(x[rows].contiguous(), w, b, single, one, i32([7 + t, t, 2 + t]), i32(range(3)), i32([0, 1, 2]),
+                           i32([7 + t, t, 2 + t]), i32([8 + t, 1 + t, 3 + t]), i32(range(4)), 3)
+            assert torch.equal(one, out[rows])
+
+
 def test_shaped_sizes_that_do_not_fit_are_refused(kn):
     from longbow_quarrel_amd.kernels.hip import KernelLibraryError
     cache = Paged(4, 1, 16, 16, torch.float32)
@@ -590,6 +652,18 @@ def test_a_slow_decay_keeps_old_tokens_in_the_state(cases, name):
     assert pc.err(case.run_cut(t, [700]), want) < TOL_F32
     assert pc.err(case.run_cut(t[:260], [3, 64, 1, 2, 130]), want[:260]) < TOL_F32
     assert pc.err(case.run_cut(t, [100, 560, 2]), want) < TOL_F32
+
+
+def test_a_narrow_product_that_shares_its_channels_over_blocks(cases):
+    """Channels enough that the product of step sizes, B and C leaves pieces (and is added up) in a long prompt and not in a
+    short one."""
+    cfg = copy.deepcopy(pc.CFG_SCAN)
+    cfg["layers"][0]["mixer"].update(inner=2048, state=16, dt_rank=8)
+    case = cases("scan-wide", "bfloat16", cfg=cfg)
+    assert case.eng.kernels.linear_pieces(torch.bfloat16, 300, 40, 2048) > 1
+    t = pc.tokens(300, case.vocab, 3)
+    pc.assert_close_bf16(case.run_cut(t, [300]), case.want(t), case.noise(t))
+    pc.assert_close_bf16(case.run_cut(t, [9, 270, 2]), case.want(t), case.noise(t))
 
 
 def test_the_first_tokens_see_zeros_ahead_of_the_sequence(cases):
