@@ -8,6 +8,7 @@ int lq_gemm_mfma(const void* x, const void* w, void* out, int out_dtype, int M, 
                  int ldw, int ldc, int epilogue, int splits, long long split_stride, int packed, hipStream_t stream);
 bool lq_gemm_packable(int N, int K);
 int lq_gemm_mfma_splits(int M, int N, int K);
+int lq_gemm_narrow_splits(int M, int N, int K);
 int lq_gemm_fused_parts(int M, int N, int K);
 int lq_gemm_residual(const void* act, const void* w, float* x, float* sq_out, const float* gain, void* scaled,
                      int ld_scaled, int M, int N, int K, int lda, int ldw, int ldx, int packed, hipStream_t stream);
@@ -21,6 +22,14 @@ int lq_gemm_scaled(const void* h, int ldh, const float* sq_parts, int n_parts, i
 extern "C" int lq_linear_splits(int in_dtype, int M, int N, int K, int force_generic) {
   if (force_generic || in_dtype != LQ_BF16 || K % 8 != 0) return 1;
   return lq_gemm_mfma_splits(M, N, K);
+}
+
+// The same for a caller that adds the pieces up right away, by a kernel of its own: a few rows of a weight with few rows
+// and a long K are then shared out as well.
+extern "C" int lq_linear_narrow_splits(int in_dtype, int M, int N, int K, int force_generic) {
+  const int usual = lq_linear_splits(in_dtype, M, N, K, force_generic);
+  if (usual > 1 || force_generic || in_dtype != LQ_BF16 || K % 8 != 0) return usual;
+  return lq_gemm_narrow_splits(M, N, K);
 }
 
 // Whether a bfloat16 weight [N, K] may be handed to the products packed (lq_pack_weight): only where every

@@ -617,7 +617,11 @@ template <int KW, int MT, int EPI, typename TO>
 __global__ __launch_bounds__(KW * 64) void gemm_bf16_skinny_kernel(const bf16_t* __restrict__ X, int ldx,
                                                                    const bf16_t* __restrict__ W, int ldw,
                                                                    TO* __restrict__ C, int ldc, int M,
-                                                                   int N, int K) {
+                                                                   int N, int K, long long split_stride) {
+  // gridDim.y shares of K (multiples of 64), a piece of the result each
+  const int share = K / (int)gridDim.y;
+  X += (long long)blockIdx.y * share, W += (long long)blockIdx.y * share, C += (long long)blockIdx.y * split_stride;
+  K = share;
   constexpr int SK_UNROLL = sk_unroll(MT);
   __shared__ float red[KW][MT * 256];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -686,9 +690,9 @@ __global__ __launch_bounds__(KW * 64) void gemm_bf16_skinny_kernel(const bf16_t*
 
 template <int KW, int MT, int EPI, typename TO>
 int launch_skinny(const void* X, const void* W, void* C, int M, int N, int K, int ldx, int ldw, int ldc,
-                  hipStream_t stream) {
-  gemm_bf16_skinny_kernel<KW, MT, EPI, TO><<<lq_ceil_div(N, 16), KW * 64, 0, stream>>>(
-      (const bf16_t*)X, ldx, (const bf16_t*)W, ldw, (TO*)C, ldc, M, N, K);
+                  hipStream_t stream, int splits = 1, long long split_stride = 0) {
+  gemm_bf16_skinny_kernel<KW, MT, EPI, TO><<<dim3(lq_ceil_div(N, 16), splits), KW * 64, 0, stream>>>(
+      (const bf16_t*)X, ldx, (const bf16_t*)W, ldw, (TO*)C, ldc, M, N, K, split_stride);
   LQ_CHECK_LAUNCH("linear(mfma skinny)");
   return 0;
 }
@@ -1081,6 +1085,17 @@ int launch_mid(const void* x, const void* w, void* out, int M, int N, int K, int
   return launch_pipelined<4, 2, 2, 2, 64, 3, EPI, TO>(x, w, out, M, N, K, lda, ldw, ldc, splits, split_stride, stream, packed);
 }
 
+// Shares of K for up to 16 rows of a weight with so few columns that its tiles of 16 leave most of the chip idle and
+// one of them walks a long K: asked for by callers that add the pieces up right away (`lq_linear_narrow_splits`).
+int narrow_splits(int M, int N, int K) {
+  if (M > 16 || N >= 8 * lq_compute_units() || K % 64 != 0) return 1;
+  int splits = 1;
+  while (splits < 16 && lq_ceil_div(N, 16) * splits * 2 <= 2 * lq_compute_units() && K % (128 * splits) == 0 &&
+         K / (splits * 2) >= 1024)
+    splits *= 2;
+  return splits;
+}
+
 int mfma_splits(int M, int N, int K) {
   if (mid_rows(M, N, K)) return mid_splits(M, N, K);
   return M <= 64 ? v3_splits(M, N, K) : tiled_splits(M, N, K);
@@ -1092,6 +1107,10 @@ int dispatch(const void* x, const void* w, void* out, int M, int N, int K, int l
   // a packed weight is wide and has K in 64s (gemm_packable): every way below that it can take ends in the
   // pipelined kernel with slabs of 64 k or in the balanced one
   LQ_REQUIRE(!packed || gemm_packable(N, K), "linear: a %d x %d weight cannot be packed", N, K);
+  if constexpr (EPI == EPI_NONE && sizeof(TO) == 4) {
+    if (splits > 1 && splits == narrow_splits(M, N, K) && !packed)
+      return launch_skinny<8, 1, EPI, TO>(x, w, out, M, N, K, lda, ldw, ldc, stream, splits, split_stride);
+  }
   if (splits > 1) {
     if (EPI != EPI_NONE || splits != mfma_splits(M, N, K)) {
       lq_set_error("linear: %d shares of K are not what this product takes (%d)", splits, mfma_splits(M, N, K));
@@ -1163,6 +1182,8 @@ int dispatch(const void* x, const void* w, void* out, int M, int N, int K, int l
 }  // namespace
 
 int lq_gemm_mfma_splits(int M, int N, int K) { return mfma_splits(M, N, K); }
+
+int lq_gemm_narrow_splits(int M, int N, int K) { return narrow_splits(M, N, K); }
 
 // The decode pair around a norm.  `residual`: x[M, N] (float32) += act[M, K] . w[N, K]^T; sq_out[M][parts]
 // takes each row's sum of squares over a block's columns, and, with a gain, scaled[M, N] takes

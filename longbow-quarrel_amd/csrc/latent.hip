@@ -187,6 +187,83 @@ __global__ __launch_bounds__(256) void qkv_norm_store_kernel(const float* __rest
   }
 }
 
+// The same with a unit's entries in registers (a unit is read once), for units, head sizes and rows in fours: PER runs of
+// four entries a thread.
+template <typename T, bool WIDE, int PER>
+__global__ __launch_bounds__(256) void qkv_norm_store4_kernel(const float* __restrict__ src, T* __restrict__ q_out,
+                                                              T* __restrict__ kcache, T* __restrict__ vcache, QkvUnits a) {
+  __shared__ float red[16];
+  const int r = blockIdx.x;
+  const int i0 = WIDE ? threadIdx.x : threadIdx.x & 63;
+  constexpr int STEP = WIDE ? 256 : 64;
+  const int u = WIDE ? (int)blockIdx.y : (int)blockIdx.y * 4 + (int)(threadIdx.x >> 6);
+  const int QW = a.H * a.D, KW = a.G * a.D, VW = a.G * a.V, unit_v = a.norm_v ? a.V : VW;
+  const int nq = QW / a.unit_q, nk = kcache != nullptr ? KW / a.unit_k : 0, nv = kcache != nullptr ? VW / unit_v : 0;
+  if (u >= nq + nk + nv) return;  // (WIDE: the whole workgroup)
+  const int which = u < nq ? 0 : u < nq + nk ? 1 : 2;
+  int n, at, col;
+  const float* w = nullptr;
+  bool norm = a.norm_qk != 0;
+  if (which == 0) n = a.unit_q, at = u * n, col = at, w = a.wq;
+  else if (which == 1) n = a.unit_k, at = (u - nq) * n, col = QW + at, w = a.wk;
+  else n = unit_v, at = (u - nq - nk) * n, col = (a.v_from_k ? QW : QW + KW) + at, norm = a.norm_v != 0;
+  const float4* s = (const float4*)(src + (long long)r * a.lds + col);
+  const float4* b = a.bias != nullptr ? (const float4*)(a.bias + col) : nullptr;
+  const int quads = n / 4;
+  float4 v[PER];
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int i = i0 + j * STEP;
+    v[j] = i < quads ? s[i] : make_float4(0.f, 0.f, 0.f, 0.f);
+    if (b != nullptr && i < quads) {
+      const float4 add = b[i];
+      v[j].x += add.x, v[j].y += add.y, v[j].z += add.z, v[j].w += add.w;
+    }
+  }
+  long long blk = 0;
+  int off = 0;
+  if (which != 0) {
+    const int p = a.row_pos[r];
+    blk = a.block_table[(long long)a.seq_slot[a.row_seq[r]] * a.bt_stride + p / a.BS];
+    off = p % a.BS;
+  }
+  float inv = 1.f;
+  if (norm) {
+#pragma unroll
+    for (int j = 0; j < PER; ++j)
+      ss = fmaf(v[j].x, v[j].x, fmaf(v[j].y, v[j].y, fmaf(v[j].z, v[j].z, fmaf(v[j].w, v[j].w, ss))));
+    inv = 1.f / sqrtf((WIDE ? block_sum(ss, red) : wave_sum(ss)) / (float)n + a.eps);
+  }
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int i = i0 + j * STEP;
+    if (i >= quads) continue;
+    float x0 = v[j].x * inv, x1 = v[j].y * inv, x2 = v[j].z * inv, x3 = v[j].w * inv;
+    if (w != nullptr) {
+      const float4 wv = ((const float4*)w)[i];
+      x0 *= wv.x, x1 *= wv.y, x2 *= wv.z, x3 *= wv.w;
+    }
+    const int e = at + 4 * i;
+    if (which == 2) {
+      const int g = e / a.V;
+      T* o = vcache + ((blk * a.G + g) * (long long)a.V + e - g * a.V) * a.BS + off;
+      o[0] = from_f32<T>(x0), o[a.BS] = from_f32<T>(x1), o[2 * a.BS] = from_f32<T>(x2), o[3 * a.BS] = from_f32<T>(x3);
+      continue;
+    }
+    const int g = e / a.D;
+    T* o = which == 0 ? q_out + (long long)r * a.ldq + e : kcache + ((blk * a.G + g) * a.BS + off) * (long long)a.D + e - g * a.D;
+    if constexpr (sizeof(T) == 4) {
+      *(float4*)o = make_float4(x0, x1, x2, x3);
+    } else {
+      uint2 packed;
+      packed.x = (uint32_t)f32_to_bf16(x0).bits | ((uint32_t)f32_to_bf16(x1).bits << 16);
+      packed.y = (uint32_t)f32_to_bf16(x2).bits | ((uint32_t)f32_to_bf16(x3).bits << 16);
+      *(uint2*)o = packed;
+    }
+  }
+}
+
 // A product a head: out[r, h ohs + n] = sum_k x[r, h K + k] w[h, n, k], bfloat16 operands on
 // v_mfma_f32_16x16x16_bf16 (exact products, 32-bit sums).  A workgroup of four wavefronts takes 64 rows by 64
 // columns of one head; a wavefront 16 rows by the 64 columns, its operands straight from memory (a head's weight
@@ -318,8 +395,23 @@ extern "C" int lq_qkv_norm_store(const float* src, int lds_, const float* bias, 
   const int gy = wide ? units : lq_ceil_div(units, 4);
   LQ_REQUIRE(gy <= 65535, "qkv_norm_store: too many heads");
   const dim3 grid(rows, gy);
+  // what fits the kernel that keeps a unit in registers: everything in fours on whole vectors (the choice follows from
+  // the model's sizes and the buffers' alignment, which are the same in every step)
+  const int el = dtype == LQ_F32 ? 4 : 2, unit_v = norm_v ? value_dim : VW;
+  int most = unit_q > unit_k ? unit_q : unit_k;
+  if (kcache != nullptr && unit_v > most) most = unit_v;
+  const bool fours = key_dim % 4 == 0 && value_dim % 4 == 0 && lds_ % 4 == 0 && ldq % 4 == 0 && (uintptr_t)src % 16 == 0 &&
+                     (uintptr_t)bias % 16 == 0 && (uintptr_t)wq % 16 == 0 && (uintptr_t)wk % 16 == 0 &&
+                     (uintptr_t)q_out % (4 * el) == 0 && (uintptr_t)kcache % (4 * el) == 0 && most <= 16384;
+#define LQ_QKV4(T, WIDE, PER)                                                                                        \
+  qkv_norm_store4_kernel<T, WIDE, PER><<<grid, 256, 0, stream>>>(src, (T*)q_out, (T*)kcache, (T*)vcache, a)
 #define LQ_QKV(T)                                                                                                    \
   do {                                                                                                               \
+    if (fours && !wide && most <= 256) LQ_QKV4(T, false, 1);                                                         \
+    else if (fours && !wide) LQ_QKV4(T, false, 2);                                                                   \
+    else if (fours && most <= 4096) LQ_QKV4(T, true, 4);                                                             \
+    else if (fours) LQ_QKV4(T, true, 16);                                                                            \
+    else                                                                                                             \
     if (wide) qkv_norm_store_kernel<T, true><<<grid, 256, 0, stream>>>(src, (T*)q_out, (T*)kcache, (T*)vcache, a);   \
     else qkv_norm_store_kernel<T, false><<<grid, 256, 0, stream>>>(src, (T*)q_out, (T*)kcache, (T*)vcache, a);       \
   } while (0)
@@ -327,6 +419,7 @@ extern "C" int lq_qkv_norm_store(const float* src, int lds_, const float* bias, 
   else if (dtype == LQ_BF16) LQ_QKV(bf16_t);
   else LQ_REQUIRE(false, "qkv_norm_store: unknown dtype %d", dtype);
 #undef LQ_QKV
+#undef LQ_QKV4
   LQ_CHECK_LAUNCH("qkv_norm_store");
   return 0;
 }

@@ -164,6 +164,70 @@ __global__ __launch_bounds__(SEL_TH) void selective_scan_kernel(const T* __restr
   if (live && nseg > 1 && a.pass == 1 && l == 0) a.seg_steps[((long long)b * a.nseg + seg) * a.channels + mine] = steps;
 }
 
+// A step of single tokens: the same operations on one token a sequence, straight from memory (nothing is shared by
+// enough threads to be worth a stop in LDS).
+template <int LN, bool WHOLE, typename T>
+__global__ __launch_bounds__(SEL_TH) void selective_step_kernel(const T* __restrict__ x, const float* __restrict__ dt,
+                                                                const T* __restrict__ Bm, const T* __restrict__ Cm,
+                                                                const T* __restrict__ z, T* __restrict__ out, SelArgs a) {
+  constexpr int COLS = SEL_TH / LN;
+  const int l = threadIdx.x % LN, b = blockIdx.y, ch = blockIdx.x * COLS + (int)threadIdx.x / LN, N = a.N;
+  const bool live = ch < a.channels;
+  const int c = live ? ch : 0;
+  const long long r = a.cu_rows[b];
+  float* sp = a.state + ((long long)a.seq_slot[b] * a.channels + c) * N;
+  float S[SEL_SLAB], A2[SEL_SLAB], bv[SEL_SLAB], cv[SEL_SLAB];
+  if (WHOLE) {  // (every lane has its eight entries: they go as 16-byte loads)
+    const float* ap = a.a_log + (long long)c * N + l * SEL_SLAB;
+    const float4 a0 = *(const float4*)ap, a1 = *(const float4*)(ap + 4);
+    const float4 s0 = *(const float4*)(sp + l * SEL_SLAB), s1 = *(const float4*)(sp + l * SEL_SLAB + 4);
+#pragma unroll
+    for (int i = 0; i < SEL_SLAB; ++i) {
+      bv[i] = to_f32(Bm[r * a.ldb + l * SEL_SLAB + i]);
+      cv[i] = to_f32(Cm[r * a.ldc + l * SEL_SLAB + i]);
+    }
+    A2[0] = a0.x, A2[1] = a0.y, A2[2] = a0.z, A2[3] = a0.w, A2[4] = a1.x, A2[5] = a1.y, A2[6] = a1.z, A2[7] = a1.w;
+    S[0] = s0.x, S[1] = s0.y, S[2] = s0.z, S[3] = s0.w, S[4] = s1.x, S[5] = s1.y, S[6] = s1.z, S[7] = s1.w;
+  } else {
+#pragma unroll
+    for (int i = 0; i < SEL_SLAB; ++i) {
+      const int n = l * SEL_SLAB + i;
+      const bool has = n < N;
+      A2[i] = has ? a.a_log[(long long)c * N + n] : 0.f;
+      bv[i] = has ? to_f32(Bm[r * a.ldb + n]) : 0.f;
+      cv[i] = has ? to_f32(Cm[r * a.ldc + n]) : 0.f;
+      S[i] = has ? sp[n] : 0.f;
+    }
+  }
+  const float raw = dt[r * a.lddt + c], bias = a.dt_bias[c], xv = to_f32(x[r * a.ldx + c]), zv = to_f32(z[r * a.ldz + c]);
+  const float D = a.d_skip[c];
+  const float step = softplus_f(raw + bias), dx = step * xv;
+  float acc = 0.f, acc1 = 0.f;
+#pragma unroll
+  for (int i = 0; i < SEL_SLAB; ++i) {
+    A2[i] = WHOLE || l * SEL_SLAB + i < N ? -expf(A2[i]) * LOG2E : 0.f;
+    S[i] = fmaf(S[i], __builtin_amdgcn_exp2f(step * A2[i]), dx * bv[i]);
+  }
+#pragma unroll
+  for (int i = 0; i < SEL_SLAB; i += 2) {
+    acc = fmaf(S[i], cv[i], acc);
+    acc1 = fmaf(S[i + 1], cv[i + 1], acc1);
+  }
+  acc = group_sum<LN>(acc + acc1);
+  if (!live) return;
+  if (WHOLE) {
+    *(float4*)(sp + l * SEL_SLAB) = make_float4(S[0], S[1], S[2], S[3]);
+    *(float4*)(sp + l * SEL_SLAB + 4) = make_float4(S[4], S[5], S[6], S[7]);
+  } else {
+#pragma unroll
+    for (int i = 0; i < SEL_SLAB; ++i) {
+      const int n = l * SEL_SLAB + i;
+      if (n < N) sp[n] = S[i];
+    }
+  }
+  if (l == 0) out[r * a.ldo + c] = from_f32<T>(fmaf(D, xv, acc) * silu_f(zv));
+}
+
 // Between the two passes: segment 0 left the state at its true end, every other segment the state it reaches from zero
 // and the sum of its steps.  In order, every segment's true start takes the place of what it left, and the last
 // segment's true end goes into the cache.
@@ -199,22 +263,28 @@ long long selective_floats(int batch, int channels, int N, int max_rows) {
 
 template <int LN, typename T>
 void launch_selective(const void* x, const float* dt, const void* Bm, const void* Cm, const void* z, void* out, const SelArgs& a,
-                      int batch, hipStream_t stream) {
+                      int batch, bool single, hipStream_t stream) {
   dim3 grid(lq_ceil_div(a.channels, SEL_TH / LN), batch, a.nseg);
-  selective_scan_kernel<LN, T><<<grid, SEL_TH, 0, stream>>>((const T*)x, dt, (const T*)Bm, (const T*)Cm, (const T*)z, (T*)out, a);
+  const bool whole = a.N == LN * SEL_SLAB && (uintptr_t)a.state % 16 == 0 && (uintptr_t)a.a_log % 16 == 0;
+  if (single && whole)
+    selective_step_kernel<LN, true, T><<<grid, SEL_TH, 0, stream>>>((const T*)x, dt, (const T*)Bm, (const T*)Cm, (const T*)z, (T*)out, a);
+  else if (single)
+    selective_step_kernel<LN, false, T><<<grid, SEL_TH, 0, stream>>>((const T*)x, dt, (const T*)Bm, (const T*)Cm, (const T*)z, (T*)out, a);
+  else
+    selective_scan_kernel<LN, T><<<grid, SEL_TH, 0, stream>>>((const T*)x, dt, (const T*)Bm, (const T*)Cm, (const T*)z, (T*)out, a);
 }
 
 template <typename T>
 void dispatch_selective(const void* x, const float* dt, const void* Bm, const void* Cm, const void* z, void* out,
-                        const SelArgs& a, int batch, hipStream_t stream) {
+                        const SelArgs& a, int batch, bool single, hipStream_t stream) {
   switch (sel_lanes(a.N)) {
-    case 1: return launch_selective<1, T>(x, dt, Bm, Cm, z, out, a, batch, stream);
-    case 2: return launch_selective<2, T>(x, dt, Bm, Cm, z, out, a, batch, stream);
-    case 4: return launch_selective<4, T>(x, dt, Bm, Cm, z, out, a, batch, stream);
-    case 8: return launch_selective<8, T>(x, dt, Bm, Cm, z, out, a, batch, stream);
-    case 16: return launch_selective<16, T>(x, dt, Bm, Cm, z, out, a, batch, stream);
-    case 32: return launch_selective<32, T>(x, dt, Bm, Cm, z, out, a, batch, stream);
-    default: return launch_selective<64, T>(x, dt, Bm, Cm, z, out, a, batch, stream);
+    case 1: return launch_selective<1, T>(x, dt, Bm, Cm, z, out, a, batch, single, stream);
+    case 2: return launch_selective<2, T>(x, dt, Bm, Cm, z, out, a, batch, single, stream);
+    case 4: return launch_selective<4, T>(x, dt, Bm, Cm, z, out, a, batch, single, stream);
+    case 8: return launch_selective<8, T>(x, dt, Bm, Cm, z, out, a, batch, single, stream);
+    case 16: return launch_selective<16, T>(x, dt, Bm, Cm, z, out, a, batch, single, stream);
+    case 32: return launch_selective<32, T>(x, dt, Bm, Cm, z, out, a, batch, single, stream);
+    default: return launch_selective<64, T>(x, dt, Bm, Cm, z, out, a, batch, single, stream);
   }
 }
 
@@ -326,13 +396,16 @@ extern "C" long long lq_selective_scan_workspace(int batch, int channels, int N,
 
 // x, z and out [rows, channels], B and C [rows, N] in one dtype, dt [rows, channels] 32-bit (before its softplus),
 // dt_bias and d_skip [channels], a_log [channels, N], state [slots, channels, N]; rows lie sequence by sequence
-// (cu_rows).  `max_rows`: the most rows a sequence brings (0: unknown); `scratch`: lq_selective_scan_workspace(...)
+// (cu_rows), every one of the `batch` sequences with at least one of the `rows`.  `max_rows`: the most rows a sequence
+// brings (0: unknown); `scratch`: lq_selective_scan_workspace(...)
 // floats, or null (then no segments).
 extern "C" int lq_selective_scan(const void* x, int ldx, const float* dt, int lddt, const void* Bm, int ldb, const void* Cm,
                                  int ldc, const void* z, int ldz, const float* dt_bias, const float* a_log,
                                  const float* d_skip, float* state, void* out, int ldo, int dtype, int channels, int N,
-                                 const int* seq_slot, const int* cu_rows, int batch, int max_rows, float* scratch,
+                                 const int* seq_slot, const int* cu_rows, int batch, int rows, int max_rows, float* scratch,
                                  long long scratch_floats, hipStream_t stream) {
+  LQ_REQUIRE(rows >= batch, "selective_scan: %d rows of %d sequences", rows, batch);
+  const bool single = rows == batch;  // every sequence brings one token
   LQ_REQUIRE(channels > 0 && N > 0 && batch > 0 && batch <= 65535, "selective_scan: %d channels, state %d, %d sequences", channels, N, batch);
   LQ_REQUIRE(N <= 64 * SEL_SLAB, "selective_scan: state size %d is larger than %d", N, 64 * SEL_SLAB);
   LQ_REQUIRE(ldx >= channels && lddt >= channels && ldz >= channels && ldo >= channels && ldb >= N && ldc >= N,
@@ -349,8 +422,8 @@ extern "C" int lq_selective_scan(const void* x, int ldx, const float* dt, int ld
     a.seg_steps = scratch + (long long)batch * SEL_SEGMENTS * channels * N;
   }
   auto run = [&]() {
-    if (dtype == LQ_F32) dispatch_selective<float>(x, dt, Bm, Cm, z, out, a, batch, stream);
-    else dispatch_selective<bf16_t>(x, dt, Bm, Cm, z, out, a, batch, stream);
+    if (dtype == LQ_F32) dispatch_selective<float>(x, dt, Bm, Cm, z, out, a, batch, single, stream);
+    else dispatch_selective<bf16_t>(x, dt, Bm, Cm, z, out, a, batch, single, stream);
   };
   run();
   LQ_CHECK_LAUNCH("selective_scan");

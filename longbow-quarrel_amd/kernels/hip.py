@@ -313,6 +313,15 @@ class HipKernels:
         return int(self.lib.lq_linear_splits(c_int(_DTYPE_CODE[dtype]), c_int(m), c_int(n), c_int(k),
                                              c_int(1 if self.force_generic else 0)))
 
+    @query
+    def linear_narrow_pieces(self, dtype: torch.dtype, m: int, n: int, k: int) -> int:
+        """The same for a caller that adds the pieces up right away (`sum_pieces`): also a few rows of a weight with few
+        rows of its own and a long K."""
+        if dtype not in _DTYPE_CODE:
+            return 1
+        return int(self.lib.lq_linear_narrow_splits(c_int(_DTYPE_CODE[dtype]), c_int(m), c_int(n), c_int(k),
+                                                    c_int(1 if self.force_generic else 0)))
+
     def linear(self, x: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> None:
         """out[M, N] = x[M, K] . w[N, K]^T with 32-bit accumulation; or out[pieces, M, N] with
         `linear_pieces` pieces that sum to it."""
@@ -321,7 +330,8 @@ class HipKernels:
         pieces, stride = 1, 0
         if out.dim() == 3:
             pieces, stride = out.shape[0], m * n
-            if not out.is_cuda or not out.is_contiguous() or pieces != self.linear_pieces(x.dtype, m, n, k):
+            if not out.is_cuda or not out.is_contiguous() or pieces not in (self.linear_pieces(x.dtype, m, n, k),
+                                                                            self.linear_narrow_pieces(x.dtype, m, n, k)):
                 raise KernelLibraryError(f"linear: {pieces} pieces asked (dense, on the GPU), linear_pieces says "
                                          f"{self.linear_pieces(x.dtype, m, n, k)}")
             mo, no, ldc = out.shape[1], out.shape[2], n
@@ -1012,7 +1022,7 @@ class HipKernels:
         self._check(self.lib.lq_selective_scan(
             _ptr(x), c_int(ld(x, "x")), _ptr(dt), c_int(ld(dt, "dt")), _ptr(b_in), c_int(ld(b_in, "B")), _ptr(c_in),
             c_int(ld(c_in, "C")), _ptr(z), c_int(ld(z, "z")), _ptr(dt_bias), _ptr(a_log), _ptr(d_skip), _ptr(state), _ptr(out),
-            c_int(ld(out, "out")), c_int(_code(x)), c_int(ch), c_int(n), _ptr(seq_slot), _ptr(cu_rows), c_int(batch),
+            c_int(ld(out, "out")), c_int(_code(x)), c_int(ch), c_int(n), _ptr(seq_slot), _ptr(cu_rows), c_int(batch), c_int(rows),
             c_int(max_rows if workspace is not None else 0), _ptr(workspace),
             c_longlong(0 if workspace is None else workspace.numel()), self.stream))
 

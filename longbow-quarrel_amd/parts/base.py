@@ -556,7 +556,7 @@ def project_narrow(kn, ctx: StepContext, x: torch.Tensor, w: torch.Tensor, out: 
     share K over blocks, they do, and the pieces are added up into `out` (in its own dtype)."""
     rows, n = x.shape[0], w.shape[0]
     add = getattr(kn, "sum_pieces", None)
-    pieces = kn.linear_pieces(x.dtype, rows, n, x.shape[1]) if add is not None and w.dtype == x.dtype else 1
+    pieces = kn.linear_narrow_pieces(x.dtype, rows, n, x.shape[1]) if add is not None and w.dtype == x.dtype else 1
     if pieces <= 1:
         project(kn, ctx, x, w, out)
         return

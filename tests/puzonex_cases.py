@@ -182,6 +182,8 @@ def make_weights(cfg: dict, seed: int, sharp: float = 1.0, memory: float = 0.0) 
             t = normal(1.0, -1.0 - memory)
         elif n.endswith(".f.b"):
             t = normal(1.0, 1.0 + memory)
+        elif n.endswith(".i.b"):  # (low enough that the bound on a memory's denominator binds at many tokens)
+            t = normal(0.5, -1.0)
         elif leaf == "b":
             t = normal(0.5)
         elif leaf in ("i", "f"):  # (several tokens share a memory: one alone would leave its answer to a single product)

@@ -203,7 +203,8 @@ def test_shaped_single_tokens_whose_keys_are_shared_out_over_workgroups(kn, size
     # heads, kv heads, key size, value size, norm of q and k, norm of v, values are keys, biases
     (4, 2, 16, 40, "head", True, False, True), (6, 2, 24, 24, "row", False, True, True), (3, 1, 7, 7, "row", False, True, True),
     (5, 5, 10, 6, "head", True, False, False), (8, 2, 128, 128, "row", False, True, True), (8, 2, 128, 64, "head", True, False, True),
-    (2, 1, 16, 16, None, False, False, True), (32, 8, 64, 64, "row", True, False, True), (1, 1, 600, 600, "head", True, False, True),
+    (2, 1, 16, 16, None, False, False, True), (32, 8, 64, 64, "row", True, False, True), (1, 1, 600, 600, "head", True, False, True), (4, 1, 384, 384, "head", True, False, True),
+    (40, 2, 128, 96, "row", False, False, True),
 ])
 def test_biases_norms_and_the_store_of_q_k_and_v(kn, sizes, dtype):
     H, G, D, P, norm, norm_v, tied, biased = sizes
@@ -226,7 +227,7 @@ def test_biases_norms_and_the_store_of_q_k_and_v(kn, sizes, dtype):
     args = dict(bias=None if bias is None else dev(bias), q_weight=None if wq is None else dev(wq),
                 k_weight=None if wk is None else dev(wk), norm_qk=norm, norm_v=norm_v, v_from_k=tied)
     tol = 3e-6 if dtype == torch.float32 else 1e-2
-    # the rows in two launches, the second without a cache first (q alone)
+    # the rows in two launches, each without a cache first (q alone)
     for lo, hi in ((0, 70), (70, T)):
         place = dict(row_pos=i32(range(lo, hi)), row_seq=i32([0] * (hi - lo)), seq_slot=i32([0]), block_table=cache.table,
                      kcache=cache.k, vcache=cache.v, block_size=64)
@@ -274,6 +275,27 @@ def test_selective_scan(kn, sizes, dtype):
     for i in (0, 1):
         assert pc.err(torch.cat(got[i]), full[i][5][: at[i]]) < (2e-5 if dtype == torch.float32 else 1e-2), i
     assert bool((state[1] == 0).all()) and bool((state[3] == 0).all())  # nobody's slots
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("sizes", [(300, 16), (40, 8), (13, 5), (70, 64), (33, 20)])
+def test_selective_scan_of_single_tokens(kn, sizes, dtype):
+    """A step of single tokens gives the bits that the same tokens give in a longer step."""
+    C, N = sizes
+    A_log, D, bias = dev(rnd(C, N, seed=1)), dev(rnd(C, seed=2)), dev(rnd(C, seed=3, mean=-1.0))
+    x, z, B, Cm = (dev(rnd(12, w, seed=4 + i), dtype) for i, w in enumerate((C, C, N, N)))
+    dt = dev(rnd(12, C, seed=9))
+    start = rnd(4, C, N, seed=10)
+    whole, state = torch.zeros((12, C), dtype=dtype, device=DEV), dev(start)
+    kn.selective_scan(x, dt, B, Cm, z, bias, A_log, D, state, whole, i32([3, 1]), i32([0, 6, 12]), 2)
+    single = dev(start)
+    for t in range(6):
+        rows = [t, 6 + t]
+        one = torch.zeros((2, C), dtype=dtype, device=DEV)
+        kn.selective_scan(*(v[rows].contiguous() for v in (x, dt, B, Cm, z)), bias, A_log, D, single, one, i32([3, 1]),
+                          i32([0, 1, 2]), 2)
+        assert torch.equal(one, whole[rows]), t
+    assert torch.equal(single, state)
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
@@ -452,6 +474,20 @@ def test_gated_unit_with_the_tanh_gelu_in_the_products_epilogue(kn, rows, k, inn
     assert float((out.cpu().double() - want)[small].abs().max() / want.abs().max()) < 2e-3
     kn.linear_swiglu(dev(x, torch.bfloat16), w, out)
     assert pc.err(out, want) > 2e-2
+
+
+@pytest.mark.parametrize("rows,n,k", [(1, 40, 2048), (8, 288, 8192), (16, 17, 4096), (3, 160, 2112), (5, 1000, 6144)])
+def test_few_rows_of_a_narrow_weight_share_a_long_k_over_blocks(kn, rows, n, k):
+    x, w = rnd(rows, k, seed=1).to(torch.bfloat16), rnd(n, k, seed=2, std=k ** -0.5).to(torch.bfloat16)
+    pieces = kn.linear_narrow_pieces(torch.bfloat16, rows, n, k)
+    assert pieces > 1 or k == 2112
+    if pieces == 1:
+        return
+    parts, out = torch.zeros((pieces, rows, n), device=DEV), torch.zeros((rows, n), device=DEV)
+    kn.linear(dev(x, torch.bfloat16), dev(w, torch.bfloat16), parts)
+    kn.sum_pieces(parts, out)
+    assert pc.err(out, x.double() @ w.double().T) < 2e-6
+    assert all(float(p.abs().max()) > 0 for p in parts)
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
