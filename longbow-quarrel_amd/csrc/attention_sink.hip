@@ -2,7 +2,8 @@
 // softmax's denominator, keys and values of different sizes, and an optional gate per head; over the paged cache.
 //
 // Row r of the step has position p = row_pos[r] in the sequence row_seq[r] and sees key t when t <= p and
-// (p - t < window or t < keep_first); window = 0: every t <= p.  Query head h reads kv head h / (nh / nkv).
+// (p - t < window or t < keep_first); window = 0: every t <= p.  chunk > 0: only keys of the row's own run of so many
+// positions (counted from 0), p / chunk == t / chunk.  Query head h reads kv head h / (nh / nkv).
 // score = q . k * scale; the softmax runs with a maximum that starts at 0 and a sum that starts at 1 when
 // there is a sink (a key of score 0 without a value; with `sinks`, a learned score a query head that is not scaled:
 // the maximum starts there), at -inf and 0 otherwise.  out = sum p_t v_t, times
@@ -65,7 +66,14 @@ struct SinkArgs {
   ScoreShape shape;
   const float* wide_gate;
   int ldwg;
+  int chunk;  // 0: no chunks
 };
+
+// the first key of the window (or of the chunk) of a row at position p
+__device__ inline int first_key(const SinkArgs& a, int p) {
+  const int lo = (a.window > 0 && p >= a.window) ? p - a.window + 1 : 0;
+  return a.chunk > 0 ? max(lo, p / a.chunk * a.chunk) : lo;
+}
 
 // What a lane needs of its query head to shape a score.
 struct HeadShape {
@@ -152,7 +160,7 @@ __global__ __launch_bounds__(64 * SPLIT) void sink_tiles_kernel(const T* __restr
   const int HS = a.KD / 16, BS = a.BS;
   const int my_row = r0 + min(c / GH, n_rows - 1), h = hbase + c % GH;
   const int my_pos = a.row_pos[my_row], my_seq = a.row_seq[my_row];
-  const int my_lo = (a.window > 0 && my_pos >= a.window) ? my_pos - a.window + 1 : 0;
+  const int my_lo = first_key(a, my_pos);
   HeadShape hs;
   if constexpr (SHAPED) hs = head_shape(a, h);
   float* myq = smem + (g * 16 + c) * QROW;
@@ -401,7 +409,7 @@ __global__ __launch_bounds__(64) void sink_rows_kernel(const T* __restrict__ q, 
   const int kvh = h / (a.nh / a.nkv), BS = a.BS, KD = a.KD, VD = a.VD;
   const int nvh = a.nkv / a.maps, g = kvh / a.maps, kmap = kvh % a.maps;  // g: the value head
   const int p = a.row_pos[r];
-  const int lo = (a.window > 0 && p >= a.window) ? p - a.window + 1 : 0;
+  const int lo = first_key(a, p);
   const int* table = a.block_table + (long long)a.seq_slot[a.row_seq[r]] * a.bt_stride;
   for (int d = lane; d < KD; d += 64) qs[d] = to_f32(q[(long long)r * a.ldq + h * KD + d]);
   HeadShape hs;
@@ -496,7 +504,7 @@ struct TileShape {
 };
 
 TileShape tile_shape(int el, int rows, int batch, int nh, int nkv, int KD, int VD, int BS, int window, int keep_first,
-                     int max_len) {
+                     int chunk, int max_len) {
   TileShape t = {false, 1, 1, 0, 0, 1, 0};
   if (KD % 16 != 0 || VD % 16 != 0 || KD > MAX_KD || VD > 256 || BS % 16 != 0) return t;
   const int hsv = VD / 16;
@@ -508,7 +516,8 @@ TileShape tile_shape(int el, int rows, int batch, int nh, int nkv, int KD, int V
   t.rows_per_tile = rows == batch ? 1 : 16 / t.heads_per_tile;  // single tokens: a tile a row of the step
   t.grid_x = lq_ceil_div(rows, t.rows_per_tile), t.grid_y = nh / t.heads_per_tile;
   if (el == 2 && rows == batch && max_len > 0) {
-    const int keys = window > 0 ? (max_len < window + keep_first + 128 ? max_len : window + keep_first + 128) : max_len;
+    int keys = window > 0 ? (max_len < window + keep_first + 128 ? max_len : window + keep_first + 128) : max_len;
+    if (chunk > 0 && chunk + 64 < keys) keys = chunk + 64;  // (a chunk's first key need not lie on a multiple of 64)
     const int rounds = lq_ceil_div(lq_ceil_div(keys, 64), SPLIT);
     const long long tiles = (long long)t.grid_x * t.grid_y;
     long long k = 2ll * lq_compute_units() / (tiles > 0 ? tiles : 1);
@@ -533,7 +542,7 @@ bool launch_tiles(const void* q, void* out, const void* gate, const void* kcache
   if (a.ldq % 4 != 0 || ((uintptr_t)q % (4 * el)) != 0 || ((uintptr_t)kcache % (4 * el)) != 0 ||
       ((uintptr_t)vcache % (4 * el)) != 0)
     return false;
-  const TileShape t = tile_shape(el, a.rows, batch, a.nh, a.nkv, a.KD, a.VD, a.BS, a.window, a.keep_first,
+  const TileShape t = tile_shape(el, a.rows, batch, a.nh, a.nkv, a.KD, a.VD, a.BS, a.window, a.keep_first, a.chunk,
                                  part != nullptr ? max_len : 0);
   if (!t.tiles) return false;
   SinkArgs b = a;
@@ -584,9 +593,11 @@ extern "C" int lq_kv_store(const void* k, int ldk, const void* v, int ldv, int d
 // Float32 entries of scratch with which a launch of single tokens shares its keys out over several workgroups a tile
 // (0: it does not).  `max_len`: an upper bound of the sequences' lengths.
 extern "C" long long lq_sink_attention_workspace(int dtype, int rows, int batch, int nh, int nkv, int KD, int VD,
-                                                 int block_size, int window, int keep_first, int max_len) {
+                                                 int block_size, int window, int keep_first, int chunk,
+                                                 int max_len) {
   if (rows <= 0 || batch <= 0 || nh <= 0 || nkv <= 0 || nh % nkv != 0 || block_size <= 0) return 0;
-  return tile_shape(dtype == LQ_BF16 ? 2 : 4, rows, batch, nh, nkv, KD, VD, block_size, window, keep_first, max_len).part_floats;
+  return tile_shape(dtype == LQ_BF16 ? 2 : 4, rows, batch, nh, nkv, KD, VD, block_size, window, keep_first, chunk,
+                    max_len).part_floats;
 }
 
 // `gate`: null, or [rows, nh] logits (stride ldg) in the dtype of q.  `rows == batch` means single tokens.  `part`:
@@ -598,7 +609,9 @@ extern "C" int lq_sink_attention(const void* q, int ldq, void* out, int ldo, con
                                  const void* vcache, int block_size, float scale, int window, int keep_first, int sink,
                                  int force_rows, int max_len, float* part, long long part_floats, const float* sinks,
                                  int maps, int out_f32, float cap, const float* temp, const float* r1, const float* r2,
-                                 const float* dist, int dist_n, const float* wide_gate, int ldwg, hipStream_t stream) {
+                                 const float* dist, int dist_n, const float* wide_gate, int ldwg, int chunk,
+                                 hipStream_t stream) {
+  LQ_REQUIRE(chunk >= 0 && (chunk == 0 || keep_first == 0), "sink_attention: chunks of %d with %d kept first tokens", chunk, keep_first);
   LQ_REQUIRE(cap >= 0.f && (r1 == nullptr) == (r2 == nullptr) && (dist == nullptr || dist_n > 0),
              "sink_attention: a cap of %g, a table by distance of %d entries", (double)cap, dist_n);
   LQ_REQUIRE(wide_gate == nullptr || ldwg >= nh * VD, "sink_attention: the wide gate's stride is smaller than its row");
@@ -618,7 +631,7 @@ extern "C" int lq_sink_attention(const void* q, int ldq, void* out, int ldo, con
   a.ksplit = 1, a.part = nullptr;
   a.maps = maps, a.out_f32 = out_f32 || dtype == LQ_F32, a.sinks = sinks;
   a.shape = {cap, temp, r1, r2, dist, dist_n};
-  a.wide_gate = wide_gate, a.ldwg = ldwg;
+  a.wide_gate = wide_gate, a.ldwg = ldwg, a.chunk = chunk;
   if (!force_rows) {
     const bool done = dtype == LQ_F32
                           ? launch_tiles<float>(q, out, gate, kcache, vcache, a, batch, max_len, part, part_floats, stream)

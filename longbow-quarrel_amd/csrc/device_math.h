@@ -15,7 +15,7 @@ __device__ inline float gelu_tanh_f(float z) {
 
 __device__ inline float gelu_erf_f(float z) { return 0.5f * z * (1.f + erff(z * 0.70710678118654752f)); }
 
-enum { ACT_NONE = 0, ACT_SILU = 1, ACT_RELU = 2, ACT_GELU_TANH = 3, ACT_GELU_ERF = 4 };
+enum { ACT_NONE = 0, ACT_SILU = 1, ACT_RELU = 2, ACT_GELU_TANH = 3, ACT_GELU_ERF = 4, ACT_RELU2 = 5 };
 
 __device__ inline float activate(float z, int act) {
   switch (act) {
@@ -23,6 +23,7 @@ __device__ inline float activate(float z, int act) {
     case ACT_RELU: return fmaxf(z, 0.f);
     case ACT_GELU_TANH: return gelu_tanh_f(z);
     case ACT_GELU_ERF: return gelu_erf_f(z);
+    case ACT_RELU2: { const float r = fmaxf(z, 0.f); return r * r; }
     default: return z;
   }
 }

@@ -118,12 +118,13 @@ __global__ __launch_bounds__(256) void rotary_qkv_kernel(const float* __restrict
   for (int e = blockIdx.y * blockDim.x + threadIdx.x; e < VW; e += blockDim.x * gridDim.y) vo[e] = from_f32<T>(vs[e]);
 }
 
-// Queries, keys and values of a step's rows without a rotation, from the 32-bit result of their one product to what the
-// attention kernel reads and straight into the paged cache.  src [rows, H D + G D (+ G V)]; `bias` (a number a column, or
-// null) is added first.  q and k are normed in units of `unit_q` and `unit_k` entries (a head each, or the whole row of
+// Queries, keys and values of a step's rows, from the 32-bit result of their one product to what the attention kernel
+// reads and straight into the paged cache.  src [rows, H D + G D (+ G V)]; `bias` (a number a column, or null) is added
+// first.  With `cs` (cos and sin of the row's angles, [rows][dims / 2][2]) the first `dims` entries of every query and key
+// head are then rotated, pairs and magnitude as in `rotary_kernel` (units of a head only).  q and k are normed in units of `unit_q` and `unit_k` entries (a head each, or the whole row of
 // all heads; units divided by their root mean square, eps inside the root, times a weight of the unit's size), values in
 // units of a head without a weight (`norm_v`) or not at all; `v_from_k`: there are no value columns, the values are the
-// keys as they are before their norm.  k and v go to the row's position in the cache (K [block][G][BS][D],
+// keys as they are before rotation and norm.  k and v go to the row's position in the cache (K [block][G][BS][D],
 // V [block][G][V][BS]); kcache null: q alone is wanted.  A wavefront takes a unit (WIDE: a workgroup), so a unit's sum of
 // squares is one fixed tree whatever else is in the launch.
 struct QkvUnits {
@@ -132,7 +133,23 @@ struct QkvUnits {
   const float *bias, *wq, *wk;
   const int *row_pos, *row_seq, *seq_slot, *block_table;
   int bt_stride, BS;
+  int unit_v;  // value entries a unit
+  const float* cs;
+  int dims, interleaved;
+  float mag;
 };
+
+// Entry i of a head (v its value, `mate` what the entry of its pair holds) after the rotation.
+__device__ inline float turned_entry(const QkvUnits& a, const float* cs, int i, float v, float mate) {
+  const int half = a.dims >> 1, j = a.interleaved ? i >> 1 : i < half ? i : i - half;
+  const bool first = a.interleaved ? !(i & 1) : i < half;
+  const float c = cs[2 * j] * a.mag, s = cs[2 * j + 1] * a.mag;
+  return first ? v * c - mate * s : v * c + mate * s;
+}
+
+__device__ inline int pair_mate(const QkvUnits& a, int i) {
+  return a.interleaved ? i ^ 1 : i < (a.dims >> 1) ? i + (a.dims >> 1) : i - (a.dims >> 1);
+}
 
 template <typename T, bool WIDE>
 __global__ __launch_bounds__(256) void qkv_norm_store_kernel(const float* __restrict__ src, T* __restrict__ q_out,
@@ -142,7 +159,7 @@ __global__ __launch_bounds__(256) void qkv_norm_store_kernel(const float* __rest
   const int i0 = WIDE ? threadIdx.x : threadIdx.x & 63;
   constexpr int STEP = WIDE ? 256 : 64;
   int u = WIDE ? (int)blockIdx.y : (int)blockIdx.y * 4 + (int)(threadIdx.x >> 6);
-  const int QW = a.H * a.D, KW = a.G * a.D, VW = a.G * a.V, unit_v = a.norm_v ? a.V : VW;
+  const int QW = a.H * a.D, KW = a.G * a.D, VW = a.G * a.V, unit_v = a.unit_v;
   const int nq = QW / a.unit_q, nk = kcache != nullptr ? KW / a.unit_k : 0, nv = kcache != nullptr ? VW / unit_v : 0;
   if (u >= nq + nk + nv) return;  // (WIDE: the whole workgroup)
   const int which = u < nq ? 0 : u < nq + nk ? 1 : 2;
@@ -154,11 +171,18 @@ __global__ __launch_bounds__(256) void qkv_norm_store_kernel(const float* __rest
   else n = unit_v, at = (u - nq - nk) * n, col = (a.v_from_k ? QW : QW + KW) + at, norm = a.norm_v != 0;
   const float* s = src + (long long)r * a.lds + col;
   const float* b = a.bias != nullptr ? a.bias + col : nullptr;
+  const float* cs = a.cs != nullptr && which != 2 ? a.cs + (long long)r * a.dims : nullptr;
+  auto entry = [&](int i) -> float {
+    const float v = b != nullptr ? s[i] + b[i] : s[i];
+    if (cs == nullptr || i >= a.dims) return v;
+    const int m = pair_mate(a, i);
+    return turned_entry(a, cs, i, v, b != nullptr ? s[m] + b[m] : s[m]);
+  };
   float inv = 1.f;
   if (norm) {
     float ss = 0.f;
     for (int i = i0; i < n; i += STEP) {
-      const float v = b != nullptr ? s[i] + b[i] : s[i];
+      const float v = entry(i);
       ss = fmaf(v, v, ss);
     }
     inv = 1.f / sqrtf((WIDE ? block_sum(ss, red) : wave_sum(ss)) / (float)n + a.eps);
@@ -171,7 +195,7 @@ __global__ __launch_bounds__(256) void qkv_norm_store_kernel(const float* __rest
     off = p % a.BS;
   }
   for (int i = i0; i < n; i += STEP) {
-    float v = b != nullptr ? s[i] + b[i] : s[i];
+    float v = entry(i);
     if (norm) v *= inv;
     if (w != nullptr) v *= w[i];
     const int e = at + i;
@@ -197,7 +221,7 @@ __global__ __launch_bounds__(256) void qkv_norm_store4_kernel(const float* __res
   const int i0 = WIDE ? threadIdx.x : threadIdx.x & 63;
   constexpr int STEP = WIDE ? 256 : 64;
   const int u = WIDE ? (int)blockIdx.y : (int)blockIdx.y * 4 + (int)(threadIdx.x >> 6);
-  const int QW = a.H * a.D, KW = a.G * a.D, VW = a.G * a.V, unit_v = a.norm_v ? a.V : VW;
+  const int QW = a.H * a.D, KW = a.G * a.D, VW = a.G * a.V, unit_v = a.unit_v;
   const int nq = QW / a.unit_q, nk = kcache != nullptr ? KW / a.unit_k : 0, nv = kcache != nullptr ? VW / unit_v : 0;
   if (u >= nq + nk + nv) return;  // (WIDE: the whole workgroup)
   const int which = u < nq ? 0 : u < nq + nk ? 1 : 2;
@@ -219,6 +243,29 @@ __global__ __launch_bounds__(256) void qkv_norm_store4_kernel(const float* __res
     if (b != nullptr && i < quads) {
       const float4 add = b[i];
       v[j].x += add.x, v[j].y += add.y, v[j].z += add.z, v[j].w += add.w;
+    }
+  }
+  if (a.cs != nullptr && which != 2) {
+    const float* cs = a.cs + (long long)r * a.dims;
+    const float* sf = (const float*)s;
+    const float* bf = (const float*)b;
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int e = 4 * (i0 + j * STEP);
+      if (e >= n || e >= a.dims) continue;
+      float* x = &v[j].x;
+      float mate[4];
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        if (a.interleaved) mate[k] = x[k ^ 1];
+        else {
+          const int m = e + k < a.dims ? pair_mate(a, e + k) : e;
+          mate[k] = bf != nullptr ? sf[m] + bf[m] : sf[m];
+        }
+      }
+#pragma unroll
+      for (int k = 0; k < 4; ++k)
+        if (e + k < a.dims) x[k] = turned_entry(a, cs, e + k, x[k], mate[k]);
     }
   }
   long long blk = 0;
@@ -377,7 +424,10 @@ extern "C" int lq_qkv_norm_store(const float* src, int lds_, const float* bias, 
                                  int unit_k, int norm_qk, int norm_v, int v_from_k, float eps, void* q_out, int ldq, int dtype,
                                  int rows, int heads, int kv_heads, int key_dim, int value_dim, const int* row_pos,
                                  const int* row_seq, const int* seq_slot, const int* block_table, int bt_stride, void* kcache,
-                                 void* vcache, int block_size, hipStream_t stream) {
+                                 void* vcache, int block_size, const float* cos_sin, int dims, int interleaved,
+                                 float magnitude, hipStream_t stream) {
+  LQ_REQUIRE(cos_sin == nullptr || (dims >= 2 && dims % 2 == 0 && dims <= key_dim && unit_q == key_dim && unit_k == key_dim),
+             "qkv_norm_store: %d rotated entries in units of %d and %d for heads of %d", dims, unit_q, unit_k, key_dim);
   LQ_REQUIRE(rows > 0 && rows <= 0x7fffffff && heads > 0 && kv_heads > 0 && key_dim > 0 && value_dim > 0,
              "qkv_norm_store: rows %d, heads %d and %d, sizes %d and %d", rows, heads, kv_heads, key_dim, value_dim);
   LQ_REQUIRE(!v_from_k || key_dim == value_dim, "qkv_norm_store: values that are the keys have their size (%d, %d)", key_dim, value_dim);
@@ -388,16 +438,19 @@ extern "C" int lq_qkv_norm_store(const float* src, int lds_, const float* bias, 
   LQ_REQUIRE(kcache == nullptr || (row_pos && row_seq && seq_slot && block_table && block_size > 0 && bt_stride > 0),
              "qkv_norm_store: the cache needs the rows' places");
   LQ_REQUIRE(norm_qk || (wq == nullptr && wk == nullptr), "qkv_norm_store: weights without a norm");
+  // (values go head by head where queries and keys do; they are only copied there)
+  const int unit_v = norm_v || (unit_q == key_dim && unit_k == key_dim) ? value_dim : VW;
   QkvUnits a = {lds_, ldq, heads, kv_heads, key_dim, value_dim, unit_q, unit_k, norm_qk, norm_v, v_from_k,
-                eps, bias, wq, wk, row_pos, row_seq, seq_slot, block_table, bt_stride, block_size};
-  const int units = QW / unit_q + (kcache ? KW / unit_k + (norm_v ? kv_heads : 1) : 0);
-  const bool wide = unit_q > 512 || unit_k > 512 || (kcache && !norm_v && VW > 512);
+                eps, bias, wq, wk, row_pos, row_seq, seq_slot, block_table, bt_stride, block_size,
+                unit_v, cos_sin, cos_sin != nullptr ? dims : 0, interleaved, magnitude};
+  const int units = QW / unit_q + (kcache ? KW / unit_k + VW / unit_v : 0);
+  const bool wide = unit_q > 512 || unit_k > 512 || (kcache && unit_v > 512);
   const int gy = wide ? units : lq_ceil_div(units, 4);
   LQ_REQUIRE(gy <= 65535, "qkv_norm_store: too many heads");
   const dim3 grid(rows, gy);
   // what fits the kernel that keeps a unit in registers: everything in fours on whole vectors (the choice follows from
   // the model's sizes and the buffers' alignment, which are the same in every step)
-  const int el = dtype == LQ_F32 ? 4 : 2, unit_v = norm_v ? value_dim : VW;
+  const int el = dtype == LQ_F32 ? 4 : 2;
   int most = unit_q > unit_k ? unit_q : unit_k;
   if (kcache != nullptr && unit_v > most) most = unit_v;
   const bool fours = key_dim % 4 == 0 && value_dim % 4 == 0 && lds_ % 4 == 0 && ldq % 4 == 0 && (uintptr_t)src % 16 == 0 &&

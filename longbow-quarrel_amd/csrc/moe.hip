@@ -1,6 +1,6 @@
 // Kernels of a mixture of experts whose experts' matrices lie side by side: the router's choice and the experts'
 // activation.  Router scores and weights are 32-bit.
-#include "common.h"
+#include "device_math.h"
 
 namespace {
 
@@ -10,7 +10,8 @@ namespace {
 // the experts form that many equal groups of neighbours; a group's mark is the sum of its two largest choice scores
 // (of its one, in groups of one), and only experts of the `keep` groups with the largest marks (the lower index on a
 // tie) can be chosen.  `softmax`: s = softmax(z) over all E outputs in the sigmoid's place.  `mark_max`: a group's mark
-// is its largest choice score alone.  `renorm_eps` is added to the chosen scores' sum before the division.  The last
+// is its largest choice score alone.  `softmax` 2: the `top` largest logits win and the weights are the softmax over these
+// alone (no correction, groups or identity experts).  `renorm_eps` is added to the chosen scores' sum before the division.  The last
 // `n_ident` of the E outputs are experts without tensors: their weights go to `ident` [rows, n_ident] (-1: not
 // chosen) and `route` has the E - n_ident others.
 __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ z, int ldz, float* __restrict__ route,
@@ -26,6 +27,23 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
   float* out_ident = n_ident > 0 ? ident + (long long)r * n_ident : nullptr;
   auto out = [&](int e) -> float& { return e < R ? out_real[e] : out_ident[e - R]; };
   for (int e = 0; e < E; ++e) out(e) = -1.f;
+  if (softmax == 2) {
+    float first = 0.f, sum = 0.f;
+    for (int k = 0; k < top; ++k) {
+      int best = -1;
+      float bz = 0.f;
+      for (int e = 0; e < E; ++e)
+        if (out(e) < 0.f && (best < 0 || zr[e] > bz)) best = e, bz = zr[e];
+      if (best < 0) break;
+      if (k == 0) first = bz;
+      const float w = expf(bz - first);
+      out(best) = w == w ? w : 0.f;
+      sum += out(best);
+    }
+    for (int e = 0; e < E; ++e)
+      if (out(e) >= 0.f) out(e) /= sum;
+    return;
+  }
   float zmax = -INFINITY, inv_sum = 1.f;
   if (softmax) {
     for (int e = 0; e < E; ++e) zmax = fmaxf(zmax, zr[e]);
@@ -124,6 +142,42 @@ __global__ __launch_bounds__(256) void moe_glu_kernel(const float* __restrict__ 
   out[r * ldo + i] = from_f32<T>(y);
 }
 
+// The same for experts without a gate: u [rows, E ff + shared], out likewise: out = act(u) w for a chosen expert's entries,
+// 0 for the others'; the last `shared` columns (an expert that every row uses) pass with weight one.  VEC entries a thread,
+// all of one expert.
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void moe_act_kernel(const float* __restrict__ u, long long ldu, const float* __restrict__ route,
+                                                      T* __restrict__ out, long long ldo, int E, int ff, int shared, int act) {
+  const int r = blockIdx.y;
+  const int i = (blockIdx.x * 256 + threadIdx.x) * VEC;
+  if (i >= E * ff + shared) return;
+  const float w = i < E * ff ? route[(long long)r * E + i / ff] : 1.f;
+  float v[VEC];
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) v[j] = 0.f;
+  if (w >= 0.f) {
+    if constexpr (VEC == 4) {
+      const float4 q = *(const float4*)(u + r * ldu + i);
+      v[0] = q.x, v[1] = q.y, v[2] = q.z, v[3] = q.w;
+    } else {
+      v[0] = u[r * ldu + i];
+    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) v[j] = activate(v[j], act) * w;
+  }
+  T* o = out + r * ldo + i;
+  if constexpr (VEC == 4 && sizeof(T) == 2) {
+    uint2 packed;
+    packed.x = (uint32_t)f32_to_bf16(v[0]).bits | ((uint32_t)f32_to_bf16(v[1]).bits << 16);
+    packed.y = (uint32_t)f32_to_bf16(v[2]).bits | ((uint32_t)f32_to_bf16(v[3]).bits << 16);
+    *(uint2*)o = packed;
+  } else if constexpr (VEC == 4) {
+    *(float4*)o = make_float4(v[0], v[1], v[2], v[3]);
+  } else {
+    *o = from_f32<T>(v[0]);
+  }
+}
+
 // ---- a step's rows sorted by expert ----------------------------------------------------------------------------------
 // counts[e] = rows that chose expert e; one workgroup an expert.
 __global__ __launch_bounds__(256) void moe_count_kernel(const float* __restrict__ route, int rows, int E,
@@ -205,6 +259,8 @@ extern "C" int lq_moe_route(const float* z, int ldz, float* route, int rows, int
              "moe_route: %d experts in %d groups of which %d are kept", experts, groups, keep);
   LQ_REQUIRE(rows > 0 && experts > 0 && top >= 1 && top <= experts && ldz >= experts, "moe_route: rows %d, %d of %d experts",
              rows, top, experts);
+  LQ_REQUIRE(softmax >= 0 && softmax <= 2 && (softmax != 2 || (correction == nullptr && groups <= 1 && n_ident == 0)),
+             "moe_route: a softmax over the chosen logits takes no correction, groups or identity experts");
   LQ_REQUIRE(n_ident >= 0 && n_ident < experts && (n_ident == 0 || ident != nullptr) && renorm_eps >= 0.f,
              "moe_route: %d identity experts of %d", n_ident, experts);
   LQ_REQUIRE(z && route, "moe_route: null pointer");
@@ -246,6 +302,35 @@ extern "C" int lq_moe_glu(const float* gu, long long ldg, const float* route, vo
     else LQ_REQUIRE(false, "moe_glu: unknown dtype %d", out_dtype);
   }
   LQ_CHECK_LAUNCH("moe_glu");
+  return 0;
+}
+
+// u and out [rows, experts * ff + shared]; route [rows, experts]; act: an activation's number (device_math.h)
+extern "C" int lq_moe_act(const float* u, long long ldu, const float* route, void* out, int out_dtype, long long ldo, int rows,
+                          int experts, int ff, int shared, int act, hipStream_t stream) {
+  const long long n = (long long)experts * ff + shared;
+  LQ_REQUIRE(rows > 0 && experts > 0 && ff > 0 && shared >= 0 && n <= 0x7fffff00, "moe_act: rows %d, experts %d, inner %d, shared %d",
+             rows, experts, ff, shared);
+  LQ_REQUIRE(ldu >= n && ldo >= n, "moe_act: a row stride is smaller than its row");
+  LQ_REQUIRE(u && route && out, "moe_act: null pointer");
+  LQ_REQUIRE(act >= ACT_SILU && act <= ACT_RELU2, "moe_act: unknown activation %d", act);
+  LQ_REQUIRE(out_dtype == LQ_F32 || out_dtype == LQ_BF16, "moe_act: unknown dtype %d", out_dtype);
+  const int el = out_dtype == LQ_F32 ? 4 : 2;
+  const bool fours = ff % 4 == 0 && shared % 4 == 0 && ldu % 4 == 0 && ldo % 4 == 0 && (uintptr_t)u % 16 == 0 &&
+                     (uintptr_t)out % (4 * el) == 0;
+  for (int r0 = 0; r0 < rows; r0 += 65535) {
+    const int nr = rows - r0 < 65535 ? rows - r0 : 65535;
+    const dim3 grid((unsigned)lq_ceil_div64(n, fours ? 1024 : 256), nr);
+#define LQ_MOE_ACT(T, VEC)                                                                                              \
+  moe_act_kernel<T, VEC><<<grid, 256, 0, stream>>>(u + r0 * ldu, ldu, route + (long long)r0 * experts, (T*)out + r0 * ldo, \
+                                                   ldo, experts, ff, shared, act)
+    if (out_dtype == LQ_F32 && fours) LQ_MOE_ACT(float, 4);
+    else if (out_dtype == LQ_F32) LQ_MOE_ACT(float, 1);
+    else if (fours) LQ_MOE_ACT(bf16_t, 4);
+    else LQ_MOE_ACT(bf16_t, 1);
+#undef LQ_MOE_ACT
+  }
+  LQ_CHECK_LAUNCH("moe_act");
   return 0;
 }
 

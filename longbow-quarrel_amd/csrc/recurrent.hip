@@ -953,7 +953,7 @@ __global__ __launch_bounds__(TH) void delta_channel_scan_kernel(const float* __r
 
 // ---------------------------------------------------------------- norms after the scans
 // One workgroup a (row, group of `group` columns).  gate_first: v = y silu(z), out = v / rms(v) w;
-// else: out = y / rms(y) w silu(z).  `sigmoid_gate`: sigmoid(z) in the place of silu(z).  w has `wlen` entries and repeats (one weight for all groups, or one a column).
+// else: out = y / rms(y) w silu(z).  `sigmoid_gate`: sigmoid(z) in the place of silu(z).  w has `wlen` entries and repeats (one weight for all groups, or one a column); null: no weight.
 template <typename T>
 __global__ void gated_rmsnorm_kernel(const float* __restrict__ y, int ldy, const float* __restrict__ z, int ldz,
                                      const float* __restrict__ w, int wlen, float eps, int group, T* __restrict__ out,
@@ -970,7 +970,8 @@ __global__ void gated_rmsnorm_kernel(const float* __restrict__ y, int ldy, const
   const float inv = 1.f / sqrtf(block_sum(ss, red) / group + eps);
   for (int c = threadIdx.x; c < group; c += blockDim.x) {
     const float gate = sigmoid_gate ? sigmoid_f(zr[c]) : silu_f(zr[c]);
-    const float v = gate_first ? yr[c] * gate * inv * w[(c0 + c) % wlen] : yr[c] * inv * w[(c0 + c) % wlen] * gate;
+    const float wv = w != nullptr ? w[(c0 + c) % wlen] : 1.f;
+    const float v = gate_first ? yr[c] * gate * inv * wv : yr[c] * inv * wv * gate;
     store_as<T>(out + (long long)r * ldo + c0 + c, v);
   }
 }
@@ -1068,7 +1069,7 @@ extern "C" int lq_add_scaled(float* x, const float* delta, int pieces, long long
 extern "C" int lq_glu(const void* gu, int in_dtype, int ld, void* out, int out_dtype, int ldo, int rows, int I, int act,
                       const float* bias, int tail, const float* row_gate, int ldrg, int gated, hipStream_t stream) {
   LQ_REQUIRE(rows > 0 && I > 0 && ld >= (gated ? 2 : 1) * I && tail >= 0 && ldo >= I + tail, "glu: rows %d, inner %d, strides %d and %d", rows, I, ld, ldo);
-  LQ_REQUIRE(act >= ACT_SILU && act <= ACT_GELU_ERF, "glu: unknown activation %d", act);
+  LQ_REQUIRE(act >= ACT_SILU && act <= ACT_RELU2, "glu: unknown activation %d", act);
   LQ_REQUIRE(gated || (bias == nullptr && tail == 0), "glu: a plain activation takes no bias and leaves no tail");
   LQ_REQUIRE(row_gate == nullptr || ldrg >= 1, "glu: the rows' gate needs a stride");
   LQ_REQUIRE(rows <= 65535 * 64, "glu: too many rows");
@@ -1299,9 +1300,9 @@ extern "C" int lq_gated_rmsnorm(const float* y, int ldy, const float* z, int ldz
                                 int group, void* out, int out_dtype, int ldo, int rows, int n, int gate_first,
                                 int sigmoid_gate, hipStream_t stream) {
   LQ_REQUIRE(rows > 0 && n > 0 && group > 0 && n % group == 0, "gated_rmsnorm: %d columns in groups of %d", n, group);
-  LQ_REQUIRE(wlen > 0 && (wlen == n || group % wlen == 0), "gated_rmsnorm: a weight of %d entries for groups of %d", wlen, group);
+  LQ_REQUIRE(w == nullptr || (wlen > 0 && (wlen == n || group % wlen == 0)), "gated_rmsnorm: a weight of %d entries for groups of %d", wlen, group);
   LQ_REQUIRE(ldy >= n && ldz >= n && ldo >= n, "gated_rmsnorm: a row stride is smaller than its row");
-  LQ_REQUIRE(y && z && w && out, "gated_rmsnorm: null pointer");
+  LQ_REQUIRE(y && z && out, "gated_rmsnorm: null pointer");
   const int threads = group >= 1024 ? 256 : group > 64 ? 128 : 64;
   for (int r0 = 0; r0 < rows; r0 += 65535) {
     const int nr = rows - r0 < 65535 ? rows - r0 : 65535;

@@ -20,7 +20,7 @@ from .. import build as _build
 from .dry import query
 
 F32, BF16 = 0, 1
-ABI_VERSION = 11  # lq_abi_version() of the library these wrappers were written for
+ABI_VERSION = 12  # lq_abi_version() of the library these wrappers were written for
 _DTYPE_CODE = {torch.float32: F32, torch.bfloat16: BF16}
 
 
@@ -739,7 +739,8 @@ class HipKernels:
 
     @query
     def sink_attention_workspace(self, dtype: torch.dtype, rows: int, batch: int, heads: int, kv_heads: int, key_dim: int,
-                                 value_dim: int, block_size: int, window: int, keep_first: int, max_len: int) -> int:
+                                 value_dim: int, block_size: int, window: int, keep_first: int, max_len: int,
+                                 chunk: int = 0) -> int:
         """Float32 entries of scratch with which `sink_attention` shares the keys of a launch of single tokens out
         over several workgroups a tile (0: it does not); `max_len`: an upper bound of the lengths."""
         if dtype not in _DTYPE_CODE:
@@ -748,7 +749,7 @@ class HipKernels:
         return int(self.lib.lq_sink_attention_workspace(c_int(_DTYPE_CODE[dtype]), c_int(rows), c_int(batch), c_int(heads),
                                                         c_int(kv_heads), c_int(key_dim), c_int(value_dim),
                                                         c_int(block_size), c_int(window), c_int(keep_first),
-                                                        c_int(max_len)))
+                                                        c_int(chunk), c_int(max_len)))
 
     def sink_attention(self, q: torch.Tensor, out: torch.Tensor, heads: int, kv_heads: int, key_dim: int,
                        value_dim: int, row_pos: torch.Tensor, row_seq: torch.Tensor, seq_slot: torch.Tensor,
@@ -758,9 +759,10 @@ class HipKernels:
                        workspace: Optional[torch.Tensor] = None, sink_values: Optional[torch.Tensor] = None,
                        maps: int = 1, softcap: float = 0.0, temp: Optional[torch.Tensor] = None,
                        log_bias: Optional[tuple] = None, distance_bias: Optional[torch.Tensor] = None,
-                       wide_gate: Optional[torch.Tensor] = None) -> None:
+                       wide_gate: Optional[torch.Tensor] = None, chunk: int = 0) -> None:
         """Attention of the step's rows over their slots' cached keys: row at position p sees t <= p with
-        p - t < window (0: all) or t < keep_first; with `sink` the softmax's denominator has one more term e^0;
+        p - t < window (0: all) or t < keep_first, and with `chunk` > 0 only t of its own run of `chunk` positions
+        (p // chunk == t // chunk); with `sink` the softmax's denominator has one more term e^0;
         `gate` [rows, heads]: every head's result times the sigmoid of its entry.  Scores and probabilities
         are 32-bit.  out [rows, heads * value_dim] in the dtype of q and the cache.  `max_len` (an upper bound of the
         lengths) and `workspace` (`sink_attention_workspace(...)` floats) let a launch of single tokens share a tile's
@@ -819,7 +821,7 @@ class HipKernels:
             c_longlong(0 if workspace is None else workspace.numel()), _ptr(sink_values), c_int(maps),
             c_int(1 if out.dtype == torch.float32 else 0), c_float(softcap), _ptr(temp), _ptr(r1), _ptr(r2),
             _ptr(distance_bias), c_int(0 if distance_bias is None else int(distance_bias.shape[1])), _ptr(wide_gate),
-            c_int(0 if wide_gate is None else self._rows2d(wide_gate, "wide_gate")), self.stream))
+            c_int(0 if wide_gate is None else self._rows2d(wide_gate, "wide_gate")), c_int(chunk), self.stream))
 
     def diff_combine(self, both: torch.Tensor, out: torch.Tensor, heads: int, kv_heads: int, value_dim: int, lam: float,
                      eps: float, gain: float) -> None:
@@ -836,7 +838,7 @@ class HipKernels:
                                              c_float(gain), self.stream))
 
     # ------------------------------------------------------------------ recurrent mixers and what surrounds them
-    _ACTIVATIONS = {"none": 0, "silu": 1, "relu": 2, "gelu_tanh": 3, "gelu": 4}
+    _ACTIVATIONS = {"none": 0, "silu": 1, "relu": 2, "gelu_tanh": 3, "gelu": 4, "relu2": 5}
 
     @staticmethod
     def _f32(t: torch.Tensor, what: str, n: Optional[int] = None) -> None:
@@ -871,8 +873,8 @@ class HipKernels:
                                            c_longlong(x.numel()), self.stream))
 
     def activation(self, x: torch.Tensor, out: torch.Tensor, activation: str) -> None:
-        """out = act(x), element by element in 32-bit; act: silu, relu, gelu_tanh or gelu (the exact one, with the error
-        function)."""
+        """out = act(x), element by element in 32-bit; act: silu, relu, gelu_tanh, gelu (the exact one, with the
+        error function) or relu2 (the square of relu)."""
         rows, inner, ld = self._mat(x, "activation: x")
         ro, wide, ldo = self._mat(out, "activation: out")
         if (ro, wide) != (rows, inner) or activation not in self._ACTIVATIONS or activation == "none":
@@ -891,7 +893,7 @@ class HipKernels:
         ro, wide, ldo = self._mat(out, "glu: out")
         inner = wide - tail
         if ro != rows or tail < 0 or two != 2 * inner or activation not in self._ACTIVATIONS \
-                or activation in ("none", "gelu"):
+                or activation in ("none", "gelu", "relu2"):
             raise KernelLibraryError(f"glu: gate_up {tuple(gate_up.shape)}, out {tuple(out.shape)}, activation {activation!r}")
         if bias is not None:
             self._f32(bias, "glu: bias", 2 * inner)
@@ -1102,11 +1104,11 @@ class HipKernels:
                                            _ptr(cu_rows), c_int(batch), c_int(rows), c_int(1 if channel_decay else 0),
                                            self.stream))
 
-    def gated_rmsnorm(self, y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, eps: float, group: int,
+    def gated_rmsnorm(self, y: torch.Tensor, z: torch.Tensor, weight: Optional[torch.Tensor], eps: float, group: int,
                       out: torch.Tensor, gate_first: bool = True, gate: str = "silu") -> None:
         """RMS norm of y [rows, n] in parts of `group` columns, each by its own root mean square, with a gate
         silu(z): gate_first: (y silu(z)) normed, times weight; else y normed, times weight, times silu(z).  The
-        weight has n entries, or fewer that repeat (one weight for every part).  `gate` "sigmoid": sigmoid(z) in the
+        weight has n entries, or fewer that repeat (one weight for every part), or is None (no weight).  `gate` "sigmoid": sigmoid(z) in the
         place of silu(z)."""
         if gate not in ("silu", "sigmoid"):
             raise KernelLibraryError(f"gated_rmsnorm: the gate is 'silu' or 'sigmoid', found {gate!r}")
@@ -1115,11 +1117,12 @@ class HipKernels:
         ro, no, ldo = self._mat(out, "gated_rmsnorm: out")
         self._f32(y, "gated_rmsnorm: y")
         self._f32(z, "gated_rmsnorm: z")
-        self._f32(weight, "gated_rmsnorm: weight", weight.numel())
+        if weight is not None:
+            self._f32(weight, "gated_rmsnorm: weight", weight.numel())
         if (rz, nz) != (rows, n) or (ro, no) != (rows, n) or group <= 0 or n % group:
             raise KernelLibraryError("gated_rmsnorm: y, z and out must be [rows, n] with n a multiple of the group")
         self._check(self.lib.lq_gated_rmsnorm(_ptr(y), c_int(ldy), _ptr(z), c_int(ldz), _ptr(weight),
-                                              c_int(weight.numel()), c_float(eps), c_int(group), _ptr(out),
+                                              c_int(0 if weight is None else weight.numel()), c_float(eps), c_int(group), _ptr(out),
                                               c_int(_code(out)), c_int(ldo), c_int(rows), c_int(n),
                                               c_int(1 if gate_first else 0), c_int(1 if gate == "sigmoid" else 0),
                                               self.stream))
@@ -1278,12 +1281,15 @@ class HipKernels:
                        v_from_k: bool = False, row_pos: Optional[torch.Tensor] = None, row_seq: Optional[torch.Tensor] = None,
                        seq_slot: Optional[torch.Tensor] = None, block_table: Optional[torch.Tensor] = None,
                        kcache: Optional[torch.Tensor] = None, vcache: Optional[torch.Tensor] = None,
-                       block_size: int = 0) -> None:
+                       block_size: int = 0, cos_sin: Optional[torch.Tensor] = None, interleaved: bool = False,
+                       magnitude: float = 1.0) -> None:
         """src float32 [rows, queries | keys (| values)], `bias` (float32, a number a column) added first.  `norm_qk`:
         None, "head" (every query and key head divided by its root mean square) or "row" (all heads of a row's queries
         together, all of its keys together); q_weight and k_weight (of the normed run's size) multiply the result.
         `norm_v`: every value head divided by its root mean square, no weight.  `v_from_k`: src has no values, they are
-        the keys with their bias, before their norm.  Queries go to q_out in its dtype; keys and values straight into
+        the keys with their bias, before rotation and norm.  `cos_sin` (float32 [rows, pairs, 2], `rope_table`): the first
+        2 pairs entries of every query and key head are rotated after the bias and before the norm, in half-split or
+        interleaved pairs, cos and sin times `magnitude`.  Queries go to q_out in its dtype; keys and values straight into
         the paged cache (layout as `kv_store`) at the rows' positions, or nowhere when kcache is None."""
         rows, ns, lds = self._mat(src, "qkv_norm_store: src")
         rq, nq, ldq = self._mat(q_out, "qkv_norm_store: q")
@@ -1297,6 +1303,12 @@ class HipKernels:
         for t, what, n in ((q_weight, "q_weight", uq), (k_weight, "k_weight", uk)):
             if t is not None:
                 self._f32(t, "qkv_norm_store: " + what, n)
+        dims = 0
+        if cos_sin is not None:
+            dims = 2 * int(cos_sin.shape[1])
+            self._f32(cos_sin, "qkv_norm_store: cos_sin", rows * dims)
+            if norm_qk == "row" or dims > key_dim:
+                raise KernelLibraryError("qkv_norm_store: a rotation of at most a head's entries, not with a norm by row")
         if norm_qk is None and (q_weight is not None or k_weight is not None):
             raise KernelLibraryError("qkv_norm_store: weights without a norm")
         stride = 0
@@ -1313,7 +1325,7 @@ class HipKernels:
             c_int(0 if norm_qk is None else 1), c_int(1 if norm_v else 0), c_int(1 if v_from_k else 0), c_float(eps), _ptr(q_out),
             c_int(ldq), c_int(_code(q_out)), c_int(rows), c_int(heads), c_int(kv_heads), c_int(key_dim), c_int(value_dim),
             _ptr(row_pos), _ptr(row_seq), _ptr(seq_slot), _ptr(block_table), c_int(stride), _ptr(kcache), _ptr(vcache),
-            c_int(block_size), self.stream))
+            c_int(block_size), _ptr(cos_sin), c_int(dims), c_int(1 if interleaved else 0), c_float(magnitude), self.stream))
 
     def postnorm_residual(self, x: torch.Tensor, y: torch.Tensor, scales, weight: torch.Tensor, eps: float,
                           extra: Optional[torch.Tensor] = None, next_weight: Optional[torch.Tensor] = None,
@@ -1348,6 +1360,41 @@ class HipKernels:
         """x *= factor (dense float32)."""
         self._f32(x, "scale: x", x.numel())
         self._check(self.lib.lq_scale(_ptr(x), c_float(factor), c_longlong(x.numel()), self.stream))
+
+    def softcap(self, x: torch.Tensor, cap: float, factor: float = 1.0) -> None:
+        """x <- cap * tanh(factor * x / cap) (dense float32)."""
+        self._f32(x, "softcap: x", x.numel())
+        self._check(self.lib.lq_softcap(_ptr(x), c_float(cap), c_float(factor), c_longlong(x.numel()), self.stream))
+
+    def streams_step(self, src: torch.Tensor, streams: int, y: Optional[torch.Tensor] = None,
+                     mix: Optional[torch.Tensor] = None, out_weights: Optional[torch.Tensor] = None,
+                     out: Optional[torch.Tensor] = None, read: Optional[torch.Tensor] = None,
+                     norm_weight: Optional[torch.Tensor] = None, eps: float = 0.0, h: Optional[torch.Tensor] = None) -> None:
+        """Residual streams X = src [streams, rows, width] (or [rows, width]: all of them equal), float32.  With a
+        sublayer's result y [rows, width] (or pieces [n, rows, width] that sum to it), out[t] = sum_s mix[s, t] X[s] +
+        out_weights[t] y (mix [streams, streams]; out may be src).  With h: u = sum_t read[t] X'[t] of the new streams (of
+        X without y; read None: the plain sum), h = u / sqrt(mean(u^2) + eps) * norm_weight in the dtype of h."""
+        shared = src.dim() == 2
+        rows, width = src.shape[-2:]
+        self._f32(src, "streams_step: src", rows * width * (1 if shared else streams))
+        pieces, stride = 0, 0
+        if y is not None:
+            pieces, stride = self._pieces(y, src if shared else src[0], "streams_step")
+            self._f32(y, "streams_step: y", rows * width * pieces)
+            self._f32(mix, "streams_step: mix", streams * streams)
+            self._f32(out_weights, "streams_step: out_weights", streams)
+            self._f32(out, "streams_step: out", streams * rows * width)
+        if h is not None:
+            self._f32(norm_weight, "streams_step: norm_weight", width)
+            if read is not None:
+                self._f32(read, "streams_step: read", streams)
+            self._dev(h)
+            if tuple(h.shape) != (rows, width) or not h.is_contiguous():
+                raise KernelLibraryError("streams_step: h must be dense [rows, width]")
+        self._check(self.lib.lq_streams_step(_ptr(src), c_longlong(0 if shared else rows * width), c_int(streams), c_int(rows),
+                                             c_int(width), _ptr(y), c_int(pieces), c_longlong(stride), _ptr(mix),
+                                             _ptr(out_weights), _ptr(out), _ptr(read), _ptr(norm_weight), c_float(eps), _ptr(h),
+                                             c_int(_code(h) if h is not None else 0), self.stream))
 
     def linear_heads(self, x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, heads: int, out_head_stride: int) -> None:
         """A product a head: out[r, h out_head_stride .. + N) = x[r, h K .. + K) . w[h]^T with w [heads, N, K]: one
@@ -1413,6 +1460,54 @@ class HipKernels:
                                          c_int(max_rows if workspace is not None else 0), _ptr(workspace),
                                          c_longlong(0 if workspace is None else workspace.numel()), self.stream))
 
+    @query
+    def decay_scan_workspace(self, rows: int, batch: int, heads: int, key_dim: int, value_dim: int, max_rows: int) -> int:
+        """Float32 entries of scratch with which `decay_scan` cuts a step into chunks (0: it walks token by token);
+        `max_rows`: the most rows that a sequence brings."""
+        self.lib.lq_decay_scan_workspace.restype = c_longlong
+        return int(self.lib.lq_decay_scan_workspace(c_int(rows), c_int(batch), c_int(heads), c_int(key_dim), c_int(value_dim),
+                                                    c_int(max_rows)))
+
+    def decay_scan(self, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, powers: torch.Tensor, state: torch.Tensor,
+                   out: torch.Tensor, heads: int, key_dim: int, value_dim: int, k_scale: float, seq_slot: torch.Tensor,
+                   cu_rows: torch.Tensor, batch: int, activation: Optional[str] = None,
+                   cos_sin: Optional[torch.Tensor] = None, interleaved: bool = False, magnitude: float = 1.0,
+                   max_rows: int = 0, workspace: Optional[torch.Tensor] = None) -> None:
+        """Linear attention with a fixed decay a head over the rows of `batch` sequences (cu_rows): S <- decay S + k v^T,
+        out = S^T q.  q, k [rows, heads * key_dim], v and out [rows, heads * value_dim], float32, each perhaps a run of
+        columns of a wider row; powers [heads, 65]: the decays' powers 0 .. 64; state float32 [slots, heads, value_dim,
+        key_dim].  `activation` "silu": q, k and v pass silu first; `cos_sin` (float32 [rows, pairs, 2]): q and k are then
+        rotated (pairing and magnitude as `rotary`); k is multiplied by `k_scale`.  `max_rows` and `workspace`
+        (`decay_scan_workspace(...)` floats): a step of long portions is cut into chunks."""
+        rows, nq, ldq = self._mat(q, "decay_scan: q")
+        rk, nk, ldk = self._mat(k, "decay_scan: k")
+        rv, nv, ldv = self._mat(v, "decay_scan: v")
+        ro, no, ldo = self._mat(out, "decay_scan: out")
+        for t in (q, k, v, out):
+            self._f32(t, "decay_scan: q, k, v, out")
+        if (rk, nk) != (rows, nq) or nq != heads * key_dim or (rv, nv) != (rows, heads * value_dim) or (ro, no) != (rv, nv):
+            raise KernelLibraryError("decay_scan: q, k [rows, heads * key_dim], v, out [rows, heads * value_dim]")
+        self._f32(powers, "decay_scan: powers", heads * 65)
+        self._f32(state, "decay_scan: state")
+        if state.dim() != 4 or tuple(state.shape[1:]) != (heads, value_dim, key_dim) or not state.is_contiguous():
+            raise KernelLibraryError("decay_scan: state dense [slots, heads, value_dim, key_dim]")
+        if activation not in (None, "silu"):
+            raise KernelLibraryError(f"decay_scan: unknown activation {activation!r}")
+        self._i32(seq_slot, "seq_slot", batch)
+        self._i32(cu_rows, "cu_rows", batch + 1)
+        dims = 0
+        if cos_sin is not None:
+            dims = 2 * int(cos_sin.shape[1])
+            self._f32(cos_sin, "decay_scan: cos_sin", rows * dims)
+        if workspace is not None:
+            self._f32(workspace, "decay_scan: workspace", workspace.numel())
+        self._check(self.lib.lq_decay_scan(
+            _ptr(q), c_int(ldq), _ptr(k), c_int(ldk), _ptr(v), c_int(ldv), _ptr(powers), _ptr(state), _ptr(out), c_int(ldo),
+            c_int(rows), c_int(heads), c_int(key_dim), c_int(value_dim), c_float(k_scale),
+            c_int(self._ACTIVATIONS[activation or "none"]), _ptr(cos_sin), c_int(dims), c_int(1 if interleaved else 0),
+            c_float(magnitude), _ptr(seq_slot), _ptr(cu_rows), c_int(batch), c_int(max_rows if workspace is not None else 0),
+            _ptr(workspace), c_longlong(0 if workspace is None else workspace.numel()), self.stream))
+
     def moe_route(self, logits: torch.Tensor, route: torch.Tensor, top: int, renormalize: bool = False,
                   correction: Optional[torch.Tensor] = None, groups: int = 0, keep: int = 0, scoring: str = "sigmoid",
                   group_mark: str = "top2", renormalize_eps: float = 0.0,
@@ -1422,7 +1517,8 @@ class HipKernels:
         (float32 [experts]) the choice goes by score + correction, the weights stay the scores.  With `groups` > 1
         the experts form that many equal groups of neighbours and only experts of the `keep` groups whose two largest
         choice scores sum highest can be chosen (`group_mark` "max": whose largest choice score is highest).
-        `scoring` "softmax": the scores are softmax(logits) over all columns.  `renormalize_eps` is added to the chosen
+        `scoring` "softmax": the scores are softmax(logits) over all columns; "softmax_chosen": the `top` largest logits
+        win and the weights are the softmax over these alone (no correction, groups or identity).  `renormalize_eps` is added to the chosen
         scores' sum before the division.  `identity` (float32 [rows, n]): the last n columns of the logits are experts
         without tensors; their weights (-1: not chosen) go there and `route` is [rows, experts - n]."""
         rows, experts, ldz = self._mat(logits, "moe_route: logits")
@@ -1431,14 +1527,15 @@ class HipKernels:
         if identity is not None:
             n_ident = identity.shape[-1]
             self._f32(identity, "moe_route: identity", rows * n_ident)
-        if scoring not in ("sigmoid", "softmax") or group_mark not in ("top2", "max"):
+        how = {"sigmoid": 0, "softmax": 1, "softmax_chosen": 2}.get(scoring)
+        if how is None or group_mark not in ("top2", "max"):
             raise KernelLibraryError(f"moe_route: scoring {scoring!r}, group_mark {group_mark!r}")
         self._f32(route, "moe_route: route", rows * (experts - n_ident))
         if correction is not None:
             self._f32(correction, "moe_route: correction", experts)
         self._check(self.lib.lq_moe_route(_ptr(logits), c_int(ldz), _ptr(route), c_int(rows), c_int(experts), c_int(top),
                                           c_int(1 if renormalize else 0), _ptr(correction), c_int(groups), c_int(keep),
-                                          c_int(1 if scoring == "softmax" else 0), c_int(1 if group_mark == "max" else 0),
+                                          c_int(how), c_int(1 if group_mark == "max" else 0),
                                           c_float(renormalize_eps), _ptr(identity), c_int(n_ident), self.stream))
 
     def moe_identity(self, h: torch.Tensor, weights: torch.Tensor, out: torch.Tensor) -> None:
@@ -1471,6 +1568,21 @@ class HipKernels:
                                         c_longlong(ldo), c_int(rows), c_int(experts), c_int(ff), c_float(limit),
                                         c_int(1 if weight_input else 0), c_int(1 if activation == "silu" else 0),
                                         self.stream))
+
+    def moe_act(self, u: torch.Tensor, route: torch.Tensor, out: torch.Tensor, experts: int, ff: int, activation: str,
+                shared: int = 0) -> None:
+        """Experts without a gate: u float32 [rows, experts * ff + shared], route [rows, experts], out shaped like u:
+        act(u) times the expert's weight for a chosen expert's columns, 0 for the others'; the last `shared` columns (an
+        expert that every row uses) are act(u)."""
+        rows, nu, ldu = self._mat(u, "moe_act: u")
+        ro, no, ldo = self._mat(out, "moe_act: out")
+        self._f32(u, "moe_act: u")
+        self._f32(route, "moe_act: route", rows * experts)
+        if nu != experts * ff + shared or (ro, no) != (rows, nu) or self._ACTIVATIONS.get(activation, 0) == 0:
+            raise KernelLibraryError(f"moe_act: u and out [rows, experts * ff + shared], activation {activation!r}")
+        self._check(self.lib.lq_moe_act(_ptr(u), c_longlong(ldu), _ptr(route), _ptr(out), c_int(_code(out)), c_longlong(ldo),
+                                        c_int(rows), c_int(experts), c_int(ff), c_int(shared),
+                                        c_int(self._ACTIVATIONS[activation]), self.stream))
 
     def weight_rows(self, w, start: int, n: int):
         """Rows start .. start + n of a product weight as a weight of its own: a view of a dense one; of a packed
