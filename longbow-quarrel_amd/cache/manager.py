@@ -144,11 +144,12 @@ class KVGroup(CacheGroup):
         self._uploads_pending = False
 
     def trim(self, slot: int, length: int) -> None:
-        """A windowed group gives back the blocks no later query can reach."""
-        w = self.need.window
-        if w <= 0:
+        """A windowed or chunked group gives back the blocks no later query can reach."""
+        w, c = self.need.window, self.need.chunk
+        if w <= 0 and c <= 0:
             return
-        first_needed = max(0, length - w + 1) // BLOCK_SIZE
+        first = max(max(0, length - w + 1) if w > 0 else 0, length // c * c if c > 0 else 0)  # of the next query's keys
+        first_needed = first // BLOCK_SIZE
         owned = self.owned[slot]
         kept = blocks_for(self.need.keep_first)  # the blocks of the first positions stay for good
         for b in range(kept, min(first_needed, len(owned))):

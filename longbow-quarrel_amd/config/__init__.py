@@ -4,7 +4,8 @@ from .llama import LlamaConfig, RopeScaling
 from .mifidra import MifidraConfig
 from .puzonex import PuzonexConfig
 from .sofinex import SofinexConfig
+from .tukedra import TukedraConfig
 from .vafodra import VafodraConfig
 from .vupelorn import VupelornConfig
 
-__all__ = ["ConfigError", "ModelConfig", "read_config_json", "LlamaConfig", "MifidraConfig", "PuzonexConfig", "RopeScaling", "SofinexConfig", "VafodraConfig", "VupelornConfig"]
+__all__ = ["ConfigError", "ModelConfig", "read_config_json", "LlamaConfig", "MifidraConfig", "PuzonexConfig", "RopeScaling", "SofinexConfig", "TukedraConfig", "VafodraConfig", "VupelornConfig"]

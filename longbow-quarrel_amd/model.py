@@ -194,16 +194,22 @@ class DecoderModel:
                 more["next_extra"] = x_in  # a block that can adds it itself, with its last kernel
             pending = block.forward(x, pending, ctx, cache, **more)
             if ctx.observe is not None:
-                ctx.observe(f"run {i}", x, None if isinstance(pending, RowStats) or hasattr(pending, "settle")
-                            else pending)
+                seen, rest = x, pending
+                if hasattr(pending, "in_pieces"):  # the stream is not in x yet
+                    seen, rest = pending.in_pieces()
+                elif isinstance(pending, RowStats) or hasattr(pending, "settle"):
+                    rest = None
+                ctx.observe(f"run {i}", seen, rest)
         normed_ahead = None  # the last block has applied the final norm to every row already
         if getattr(pending, "norm", None) is self.final_norm and getattr(pending, "normed", None) is not None \
                 and ctx.want_all and n_want == ctx.rows:
             normed_ahead = pending.normed
-        if hasattr(pending, "settle"):  # a pending object of a block's own kind adds itself to the stream
-            pending = pending.settle(x, ctx)
         if n_want == 0:
             return None
+        if normed_ahead is None and hasattr(pending, "in_pieces"):  # only the wanted rows of the stream are added up
+            x, pending = pending.in_pieces()
+        elif normed_ahead is None and hasattr(pending, "settle"):  # a block's own kind adds itself to the stream
+            pending = pending.settle(x, ctx)
         ctx.ws.next_run()
         logits = ctx.logits_out
         if logits is None:

@@ -84,7 +84,7 @@ class TensorSpec:
     name: str  # the safetensors name
     shape: Tuple[int, ...]
     kind: str = MATRIX
-    init: str = "normal"  # random-weights rule: "normal" | "around_one" (a gain) | "zeros"
+    init: str = "normal"  # random-weights rule: "normal" | "around_one" (a gain) | "around_identity" | "zeros"
     optional: bool = False  # may be absent from the file (a tied head)
 
 
@@ -109,13 +109,15 @@ class KVNeed(CacheNeed):
     """Keys and values per position: `kv_heads` x `head_dim` each (values `value_dim` wide where that is
     set and differs); window = 0 keeps all positions, window = w keeps the last w (older blocks go back to
     the pool), except the blocks that hold the first `keep_first` positions, which every later query still
-    sees."""
+    sees.  chunk = c > 0: queries see their own run of c positions (counted from 0) only; the blocks of runs that are
+    over go back."""
 
     kv_heads: int
     head_dim: int
     window: int = 0
     value_dim: int = 0  # 0: as wide as the keys
     keep_first: int = 0
+    chunk: int = 0
 
     @property
     def v_dim(self) -> int:

@@ -10,7 +10,7 @@ from typing import List, Mapping, Optional
 
 import torch
 
-from .base import (BLOCKS, FEED_FORWARDS, MIXERS, NORMS, Block, BuildEnv, LayerCache, NormedRows, PartSpec,
+from .base import (BLOCKS, FEED_FORWARDS, MIXERS, NORMS, VECTOR32, Block, BuildEnv, LayerCache, NormedRows, PartSpec,
                    ResidualSink, RowStats, StepContext, TensorSpec, build_part)
 
 
@@ -372,3 +372,156 @@ class SandwichNormBlock(Block):
         if ahead is None and extra is None:
             return None
         return NormedAhead(h, ahead, added_extra=extra is not None)
+
+
+class StreamRead:
+    """What a sublayer of a `HyperConnectedBlock` reads: the streams' weighted sum, normed.  A block exposes the first of
+    its own as `first_norm`, so that the kernel that writes the streams ahead of it makes what it reads too."""
+
+    deferrable = False  # (no norm of one stream: other blocks do not apply it themselves)
+
+    def __init__(self, norm, block: "HyperConnectedBlock", sub: int) -> None:
+        self.norm, self.block, self.sub = norm, block, sub
+
+    @property
+    def weights(self) -> torch.Tensor:
+        return self.block.links[self.sub][0]
+
+    @property
+    def streams(self) -> int:
+        return self.block.streams
+
+
+class Streams:
+    """What a `HyperConnectedBlock` leaves pending: the streams [n, rows, width] in 32-bit; the residual stream proper is
+    their sum, which `x` does not hold yet (`settle`).  `normed` holds what `norm` (the `StreamRead` or the norm of the
+    sum that comes next) makes of them, where that was known."""
+
+    def __init__(self, stack: torch.Tensor, normed: Optional[torch.Tensor] = None, norm=None) -> None:
+        self.stack, self.normed, self.norm = stack, normed, norm
+
+    def settle(self, x: torch.Tensor, ctx: StepContext) -> None:
+        ctx.kernels.sum_pieces(self.stack, x)
+        return None
+
+    def in_pieces(self):
+        """The residual stream as (a dense part, what is to be added to it)."""
+        return self.stack[0], self.stack[1:] if self.stack.shape[0] > 1 else None
+
+
+@BLOCKS.register("hyper_connected")
+class HyperConnectedBlock(Block):
+    """Hyper-connections (Zhu, Huang, Huang, Zeng, Mao, Wu, Min, Zhou: "Hyper-Connections"), with constant weights: the
+    residual is `streams` copies X_1 .. X_n, all equal to the stream that the first such block finds.  For every sublayer,
+    with its learned numbers in [n], mix [n, n] (from, to) and out [n] (`<links>.in`, `.mix`, `.out`):
+
+        u = sum_s in_s X_s,      y = sublayer(norm(u)),      X_t <- sum_s mix_st X_s + out_t y   (from the old X).
+
+    The stream that other parts see (a norm behind the last such block, another kind of block) is the sum of the copies.
+    All 32-bit.  One kernel writes the copies with a sublayer's result and makes what the next sublayer reads: this block's
+    feed-forward, the next block's mixer (`next_norm` is its `first_norm`), or the model's norm of the sum.  The
+    feed-forward may be absent (its norm and links may then be in a file or not, and are not used)."""
+
+    takes_next_norm = True
+
+    def __init__(self, streams: int, mixer: PartSpec, mixer_norm: PartSpec, mixer_links: str,
+                 feed_forward: Optional[PartSpec] = None, ffn_norm: Optional[PartSpec] = None,
+                 ffn_links: Optional[str] = None) -> None:
+        self.streams = int(streams)
+        if self.streams < 1:
+            raise ValueError("hyper-connections need at least one stream")
+        self.mixer = build_part(MIXERS, mixer)
+        self.ffn = build_part(FEED_FORWARDS, feed_forward) if feed_forward is not None else None
+        if self.ffn is not None and (ffn_norm is None or ffn_links is None):
+            raise ValueError("a feed-forward needs the norm ahead of it and its links to the streams")
+        self.norms = [build_part(NORMS, n) for n in (mixer_norm, ffn_norm) if n is not None]
+        self.link_names = [n for n in (mixer_links, ffn_links) if n is not None]
+        if any(not getattr(n, "deferrable", False) for n in self.norms):
+            raise ValueError("the norms ahead of the sublayers must be RMS norms")
+        self.subs = 1 if self.ffn is None else 2  # sublayers; norms and links beyond them are idle
+        self.reads = [StreamRead(self.norms[i], self, i) for i in range(self.subs)]
+        self.links: List = []
+
+    @property
+    def graph_safe(self) -> bool:
+        return self.mixer.graph_safe and (self.ffn is None or self.ffn.graph_safe)
+
+    @property
+    def first_norm(self):
+        return self.reads[0]
+
+    def _link_specs(self, i: int) -> List[TensorSpec]:
+        n, name = self.streams, self.link_names[i]
+        return [TensorSpec(name + ".in", (n,), kind=VECTOR32, init="around_one"),
+                TensorSpec(name + ".mix", (n, n), kind=VECTOR32, init="around_identity"),
+                TensorSpec(name + ".out", (n,), kind=VECTOR32, init="around_one")]
+
+    def tensor_specs(self) -> List[TensorSpec]:
+        specs = self.mixer.tensor_specs() + (self.ffn.tensor_specs() if self.ffn is not None else [])
+        for i in range(self.subs):
+            specs += self.norms[i].tensor_specs() + self._link_specs(i)
+        idle = [s for n in self.norms[self.subs :] for s in n.tensor_specs()]
+        idle += [s for i in range(self.subs, len(self.link_names)) for s in self._link_specs(i)]
+        return specs + [dataclasses.replace(s, optional=True) for s in idle]
+
+    def bind(self, tensors: Mapping[str, torch.Tensor], env: BuildEnv) -> None:
+        super().bind(tensors, env)
+        for p in (self.mixer, self.ffn, *self.norms[: self.subs]):
+            if p is not None:
+                p.bind(tensors, env)
+        self.links = [tuple(tensors[f"{name}.{key}"].contiguous() for key in ("in", "mix", "out"))
+                      for name in self.link_names[: self.subs]]
+
+    @staticmethod
+    def _result(part, args, ctx: StepContext, width: int) -> torch.Tensor:
+        """A sublayer's result in 32-bit, [rows, width] or pieces [n, rows, width] that are still to be added."""
+        in_pieces = getattr(part, "forward_pieces", None)
+        if in_pieces is not None:
+            got, scales = in_pieces(*args)
+            for piece, scale in zip(got if got.dim() == 3 else got[None], scales):
+                if scale != 1.0:
+                    ctx.kernels.scale(piece, scale)
+            return got
+        got = part.forward(*args)
+        if got.dtype != torch.float32 or not got.is_contiguous():
+            out = ctx.ws.alloc((args[0].shape[0], width), torch.float32)
+            ParallelBlock._copy_into(ctx.kernels, got, out)
+            return out
+        return got
+
+    def forward(self, x: torch.Tensor, pending, ctx: StepContext, cache: Optional[LayerCache], next_norm=None):
+        kn, (rows, width) = ctx.kernels, x.shape
+        read = self.reads[0]
+        if isinstance(pending, Streams) and pending.stack.shape[0] == self.streams:
+            stack, fresh = pending.stack, False
+            h = pending.normed if pending.norm is read else None
+        else:
+            if hasattr(pending, "settle"):
+                pending = pending.settle(x, ctx)
+            if pending is not None and not isinstance(pending, RowStats):
+                kn.add(x, pending)
+            # the copies are equal: one stands for all until a sublayer's result has been written
+            stack, fresh, h = ctx.ws.alloc((self.streams, rows, width), torch.float32, keep=True), True, None
+        if h is None:
+            h = ctx.ws.alloc((rows, width), ctx.dtype)
+            kn.streams_step(x if fresh else stack, self.streams, read=read.weights, norm_weight=read.norm.weight,
+                            eps=read.norm.eps, h=h)
+        for i in range(self.subs):
+            y = self._result(self.mixer, (h, ctx, cache), ctx, width) if i == 0 else \
+                self._result(self.ffn, (h, ctx), ctx, width)
+            ahead = self.reads[i + 1] if i + 1 < self.subs else next_norm
+            if isinstance(ahead, StreamRead):
+                if ahead.streams != self.streams:
+                    ahead = None
+            elif not getattr(ahead, "deferrable", False):
+                ahead = None
+            more, h = {}, None
+            if ahead is not None:
+                norm = ahead.norm if isinstance(ahead, StreamRead) else ahead
+                h = ctx.ws.alloc((rows, width), ctx.dtype)
+                more = dict(read=ahead.weights if isinstance(ahead, StreamRead) else None, norm_weight=norm.weight,
+                            eps=norm.eps, h=h)
+            _, mix, out_w = self.links[i]
+            kn.streams_step(x if fresh else stack, self.streams, y=y, mix=mix, out_weights=out_w, out=stack, **more)
+            fresh = False
+        return Streams(stack, h, ahead if h is not None else None)

@@ -154,11 +154,11 @@ class GatedLinearUnit(FeedForward):
 @FEED_FORWARDS.register("mlp")
 class PlainFeedForward(FeedForward):
     """down(act(up(h))): two matrices, no gate and no biases; `activation` "gelu" (the exact one, with the error
-    function), "gelu_tanh", "silu" or "relu".  The activation reads the first product's 32-bit result."""
+    function), "gelu_tanh", "silu", "relu" or "relu2" (the square of relu).  The activation reads the first product's 32-bit result."""
 
     graph_safe = True
     takes_out = True
-    ACTIVATIONS = ("gelu", "gelu_tanh", "silu", "relu")
+    ACTIVATIONS = ("gelu", "gelu_tanh", "silu", "relu", "relu2")
 
     def __init__(self, width: int, inner: int, prefix: str, activation: str = "gelu",
                  names: Optional[Mapping[str, str]] = None) -> None:
@@ -193,7 +193,7 @@ class PlainFeedForward(FeedForward):
 
 @FEED_FORWARDS.register("moe")
 class MixtureOfExperts(FeedForward):
-    """`experts` small gated feed-forwards of which every token uses `top`, chosen by a router.
+    """`experts` small feed-forwards of which every token uses `top`, chosen by a router.
 
     Router: z = Wr h summed in 32-bit (h as the run holds it), s = sigmoid(z) in 32-bit; the `top` largest scores win (the lower index on a tie); an expert's
     weight is its score as it is (`renormalize` divides the chosen scores by their sum).  With `weight_input` the
@@ -202,7 +202,7 @@ class MixtureOfExperts(FeedForward):
     Expert (`activation` "clamped_swish"): g = min(Wg h, limit), u = clamp(Wu h, -limit, limit),
     y = g sigmoid(1.702 g) (u + 1), result Wd y; no biases.  Wg (s h) = s (Wg h), so the weight is applied to the
     32-bit results of the gate and up products, ahead of the clamps.  `activation` "silu": y = silu(Wg h) (Wu h),
-    no clamps.
+    no clamps.  `activation` "relu2": an expert has two matrices and no gate, y = relu(Wu h)^2 (the shared expert too).
 
     `correction`: a learned constant for every expert (`<prefix>.correction`) is added to the scores for the choice
     alone; the weights stay the scores.  `groups` / `keep`: the experts form `groups` equal groups of neighbours, a
@@ -211,7 +211,9 @@ class MixtureOfExperts(FeedForward):
     token with weight one, and is added.  `shared_gate`: the shared expert's result is multiplied by the sigmoid of
     one more projection of the input, a number a token (`<prefix>.shared.sg`, [1, width]).
 
-    `scoring` "softmax": s = softmax(z) over all the router's outputs in the place of the sigmoid.  `group_mark`
+    `scoring` "softmax": s = softmax(z) over all the router's outputs in the place of the sigmoid.  "softmax_chosen": the
+    `top` largest logits win and the weights are the softmax over these alone (no groups, correction or identity
+    experts).  `group_mark`
     "max": a group's mark is its largest choice score (the default, "top2", is the sum of its two largest); experts
     outside the kept groups cannot be chosen whatever their choice scores (which may be negative).  `renormalize_eps`
     is added to the chosen scores' sum before the division.  `identity`: so many more outputs of the router, behind
@@ -232,7 +234,7 @@ class MixtureOfExperts(FeedForward):
     #: rows from which a step that is no decoding step is sorted by expert
     sort_from_rows = 256
 
-    ACTIVATIONS = ("clamped_swish", "silu")
+    ACTIVATIONS = ("clamped_swish", "silu", "relu2")
 
     def __init__(self, width: int, experts: int, top: int, inner: int, prefix: str, limit: float = 0.0,
                  weight_input: bool = True, renormalize: bool = False, activation: str = "clamped_swish",
@@ -243,7 +245,7 @@ class MixtureOfExperts(FeedForward):
         self.scoring, self.group_mark, self.renormalize_eps = scoring, group_mark, float(renormalize_eps)
         self.identity, self.shared_gate = int(identity), bool(shared_gate)
         self.outputs = self.experts + self.identity  # what the router scores
-        if scoring not in ("sigmoid", "softmax") or group_mark not in ("top2", "max"):
+        if scoring not in ("sigmoid", "softmax", "softmax_chosen") or group_mark not in ("top2", "max"):
             raise ValueError(f"scoring is 'sigmoid' or 'softmax' ({scoring!r}), a group's mark 'top2' or 'max' ({group_mark!r})")
         if self.identity < 0 or (self.identity and weight_input):
             raise ValueError("identity experts: none or more, and the weight on the experts' results")
@@ -254,8 +256,14 @@ class MixtureOfExperts(FeedForward):
         self.groups, self.keep, self.shared_inner = int(groups), int(keep), int(shared_inner)
         if activation not in self.ACTIVATIONS:
             raise ValueError(f"unknown activation {activation!r}; known: {', '.join(self.ACTIVATIONS)}")
-        if self.shared_inner and activation != "silu":
-            raise ValueError("a shared expert is built for the 'silu' activation only")
+        self.gated = activation != "relu2"  # an expert has a gate matrix beside its up matrix
+        self.n_in = 2 if self.gated else 1
+        if self.shared_inner and activation == "clamped_swish":
+            raise ValueError("a shared expert is built for the 'silu' and 'relu2' activations only")
+        if not self.gated and (self.weight_input or self.shared_gate):
+            raise ValueError("experts without a gate take the weight on their results, and no gate on a shared expert")
+        if scoring == "softmax_chosen" and (correction or int(groups) > 1 or self.identity):
+            raise ValueError("a softmax over the chosen logits is not combined with a correction, groups or identity experts")
         if not 1 <= self.top <= self.outputs:
             raise ValueError(f"{top} of {self.outputs} experts cannot be chosen")
         if self.groups > 1:
@@ -279,17 +287,16 @@ class MixtureOfExperts(FeedForward):
 
     def tensor_specs(self) -> List[TensorSpec]:
         specs = []
+        ins = ("gate", "up") if self.gated else ("up",)
         for e in range(self.experts):
-            specs += [TensorSpec(self._name(e, "gate"), (self.inner, self.width)),
-                      TensorSpec(self._name(e, "up"), (self.inner, self.width)),
-                      TensorSpec(self._name(e, "down"), (self.width, self.inner))]
+            specs += [TensorSpec(self._name(e, key), (self.inner, self.width)) for key in ins]
+            specs.append(TensorSpec(self._name(e, "down"), (self.width, self.inner)))
         specs.append(TensorSpec(f"{self.prefix}.{self.n['router']}", (self.outputs, self.width)))
         if self.correction:
             specs.append(TensorSpec(f"{self.prefix}.{self.n['correction']}", (self.outputs,), kind=VECTOR32))
         if self.shared_inner:
-            specs += [TensorSpec(self._shared_name("gate"), (self.shared_inner, self.width)),
-                      TensorSpec(self._shared_name("up"), (self.shared_inner, self.width)),
-                      TensorSpec(self._shared_name("down"), (self.width, self.shared_inner))]
+            specs += [TensorSpec(self._shared_name(key), (self.shared_inner, self.width)) for key in ins]
+            specs.append(TensorSpec(self._shared_name("down"), (self.width, self.shared_inner)))
         if self.shared_gate:
             specs.append(TensorSpec(self._shared_name("shared_gate"), (1, self.width)))
         return specs
@@ -297,18 +304,20 @@ class MixtureOfExperts(FeedForward):
     def bind(self, tensors: Mapping[str, torch.Tensor], env: BuildEnv) -> None:
         super().bind(tensors, env)
         E = self.experts
-        gu = [tensors[self._name(e, w)] for e in range(E) for w in ("gate", "up")]
+        ins, n_in = ("gate", "up") if self.gated else ("up",), self.n_in
+        gu = [tensors[self._name(e, w)] for e in range(E) for w in ins]
         down = [tensors[self._name(e, "down")] for e in range(E)]
         ffs = self.shared_inner
         if ffs:  # the shared expert's rows and columns lie behind the routed experts'
-            gu += [tensors[self._shared_name(w)] for w in ("gate", "up")]
+            gu += [tensors[self._shared_name(w)] for w in ins]
             down.append(tensors[self._shared_name("down")])
         if len({m.dtype for m in gu + down}) != 1:
-            raise ValueError(f"{self._name(0, 'gate')}: the experts' matrices are stored in different dtypes")
-        # expert e's rows of the first matrix: [gate (ff) | up (ff)]; its columns of the second: e ff .. (e + 1) ff
+            raise ValueError(f"{self._name(0, 'up')}: the experts' matrices are stored in different dtypes")
+        # expert e's rows of the first matrix: [gate (ff) | up (ff)], or up alone; its columns of the second:
+        # e ff .. (e + 1) ff
         ff = self.inner
-        runs = [(e * 2 * ff, 2 * ff) for e in range(E)] + ([(E * 2 * ff, 2 * ffs)] if ffs else [])
-        whole = torch.cat(gu, dim=0).contiguous()  # [E * 2 ff (+ 2 ffs), width]
+        runs = [(e * n_in * ff, n_in * ff) for e in range(E)] + ([(E * n_in * ff, n_in * ffs)] if ffs else [])
+        whole = torch.cat(gu, dim=0).contiguous()  # [E * n_in ff (+ n_in ffs), width]
         self.w_gate_up = product_weight(env, whole)
         rows_of = getattr(env.kernels, "weight_rows", None)
         if self.w_gate_up is whole:
@@ -374,7 +383,9 @@ class MixtureOfExperts(FeedForward):
     def _unit(self, gu, act, ctx: StepContext) -> None:
         """The shared expert's activation (no routing; weight one, or the sigmoid of its gate's logit)."""
         gate = self._step[1]
-        if gate is not None:
+        if not self.gated:
+            ctx.kernels.activation(gu, act, self.activation)
+        elif gate is not None:
             ctx.kernels.glu(gu, act, "silu", row_gate=gate)
         else:
             ctx.kernels.glu(gu, act, "silu")
@@ -395,7 +406,7 @@ class MixtureOfExperts(FeedForward):
 
     def _shared(self, h, out, ctx: StepContext) -> None:
         kn, rows, ffs = ctx.kernels, h.shape[0], self.shared_inner
-        gu = ctx.ws.alloc((rows, 2 * ffs), torch.float32)
+        gu = ctx.ws.alloc((rows, self.n_in * ffs), torch.float32)
         project(kn, ctx, h, self.gate_up_of[-1], gu)
         act = ctx.ws.alloc((rows, ffs), ctx.dtype)
         self._unit(gu, act, ctx)
@@ -417,9 +428,14 @@ class MixtureOfExperts(FeedForward):
             return out
         # every row through all experts' columns (and the shared expert's behind them): the activations of the
         # experts that a row did not choose are zeros, so the second product adds the chosen ones and the shared one
-        gu = ctx.ws.alloc((rows, E * 2 * ff + 2 * ffs), torch.float32)
+        gu = ctx.ws.alloc((rows, self.n_in * (E * ff + ffs)), torch.float32)
         project(kn, ctx, h, self.w_gate_up, gu)
         act = ctx.ws.alloc((rows, E * ff + ffs), ctx.dtype)
+        if not self.gated:  # (one launch: the shared expert's columns pass with weight one)
+            kn.moe_act(gu, route, act, E, ff, self.activation, shared=ffs)
+            project(kn, ctx, act, self.w_down, out)
+            self._pass_on(h, out, ctx)
+            return out
         more = {"activation": self.activation} if self.activation != "clamped_swish" else {}
         kn.moe_glu(gu[:, : E * 2 * ff], route, act[:, : E * ff], E, ff, self.limit, self.weight_input, **more)
         if ffs:
@@ -445,15 +461,18 @@ class MixtureOfExperts(FeedForward):
             return
         hs = ctx.ws.alloc((pairs, self.width), h.dtype)
         kn.moe_gather(h, order, hs, total)
-        gu = ctx.ws.alloc((pairs, 2 * ff), torch.float32)
+        gu = ctx.ws.alloc((pairs, self.n_in * ff), torch.float32)
         at = 0
         for e, n in enumerate(n_of):
             if n:
                 project(kn, ctx, hs[at : at + n], self.gate_up_of[e], gu[at : at + n])
                 at += n
         act = ctx.ws.alloc((pairs, ff), ctx.dtype)
-        more = {"activation": self.activation} if self.activation != "clamped_swish" else {}
-        kn.moe_glu(gu[:total], weight[:total], act[:total], 1, ff, self.limit, self.weight_input, **more)
+        if self.gated:
+            more = {"activation": self.activation} if self.activation != "clamped_swish" else {}
+            kn.moe_glu(gu[:total], weight[:total], act[:total], 1, ff, self.limit, self.weight_input, **more)
+        else:
+            kn.moe_act(gu[:total], weight[:total], act[:total], 1, ff, self.activation)
         ys = ctx.ws.alloc((pairs, self.width), torch.float32)
         at = 0
         for e, n in enumerate(n_of):

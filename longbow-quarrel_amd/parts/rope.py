@@ -70,6 +70,18 @@ def rotary_magnitude(scaling: Optional[Mapping] = None) -> float:
     return 1.0
 
 
+def step_angles(ctx: StepContext, freqs: torch.Tensor, table: List[float]) -> torch.Tensor:
+    """cos and sin of every row's angles, float32 [rows, pairs, 2]: the same for every layer of a step that rotates with
+    these frequencies (`freqs` on the device, `table` the same numbers on the host), so computed once and shared."""
+    key = ("rope_cos_sin", tuple(table))
+    angles = ctx.shared.get(key)
+    if angles is None:
+        angles = ctx.ws.alloc((ctx.rows, len(table), 2), torch.float32, keep=True)
+        ctx.kernels.rope_table(freqs, ctx.row_pos, angles)
+        ctx.shared[key] = angles
+    return angles
+
+
 @POSITION_ENCODINGS.register("rope")
 class RotaryEncoding(PositionEncoding):
     graph_safe = True
@@ -85,15 +97,7 @@ class RotaryEncoding(PositionEncoding):
         self.rotary_frequencies = torch.tensor(self.table, dtype=torch.float64, device=env.device)
 
     def cos_sin(self, ctx: StepContext) -> torch.Tensor:
-        """cos and sin of every row's angles, float32 [rows, head_dim/2, 2]: the same for every layer
-        of a step that rotates with these frequencies, so it is computed once and shared."""
-        key = ("rope_cos_sin", tuple(self.table))
-        table = ctx.shared.get(key)
-        if table is None:
-            table = ctx.ws.alloc((ctx.rows, self.head_dim // 2, 2), torch.float32, keep=True)
-            ctx.kernels.rope_table(self.rotary_frequencies, ctx.row_pos, table)
-            ctx.shared[key] = table
-        return table
+        return step_angles(ctx, self.rotary_frequencies, self.table)
 
     def apply(self, q: torch.Tensor, k: torch.Tensor, ctx: StepContext) -> None:
         heads = q.shape[1] // self.head_dim

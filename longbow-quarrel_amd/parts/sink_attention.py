@@ -17,17 +17,22 @@ pass; `qk_norm_eps` then divides every query and key head by its root mean squar
 are taken in 32-bit on the product's 32-bit result, by one kernel that also leaves q, k and v in the dtype of the
 cache.
 
+`chunk` = c: position i sees only the keys of its own run of c positions, floor(i / c) = floor(j / c), counted from the
+start of the sequence.
+
 `probabilities="bfloat16"` says that a design lets the softmax's weights be rounded to bfloat16 as operands of their
 product with the values (the sums stay 32-bit): plain causal attention with keys and values of one size then runs, in
 a bfloat16 run, on the causal kernel of the matrix cores, several times as fast over a prompt.  The default keeps the
 weights 32-bit through that product.
 
-What a design may ask for beside these, each with a parameter (none of it together with a rotation or `qk_norm_eps`):
+What a design may ask for beside these, each with a parameter (none of the first five together with `qk_norm_eps`):
 * `qkv_bias`: biases on q, k and v (`<name>.b`); `out_bias`: one on the output projection (`<prefix>.o.b`).
 * `qk_norm` "head" or "row": RMS norm with a weight (`<prefix>.q.norm`, `<prefix>.k.norm`) on every head of q and k (the
-  weight is shared by the heads), or on all heads' entries of a row together; `value_norm`: every value head divided
-  by its root mean square, without a weight.  `norm_eps` for all of them.
-* `values_from_keys`: there is no Wv, the values are the keys as projected (with their bias, before their norm).
+  weight is shared by the heads), or on all heads' entries of a row together; "unit": every head of q and k divided by
+  its root mean square, no weight; `value_norm`: every value head divided by its root mean square, without a weight.
+  `norm_eps` for all of them.
+* `values_from_keys`: there is no Wv, the values are the keys as projected (with their bias, before rotation and norm).
+* `rotary` together with any of these: the rotation comes after the bias and before the norm (not with "row").
 * `temperature`: a stored number a head (`<prefix>.temp`) multiplies the scaled score; `softcap`: score <- softcap
   tanh(score / softcap) (0: not).
 * `log_bias`: r1_h ln(1 + r2_h n) is taken off the score of a key n positions back (`<prefix>.r1`, `.r2`, a number a
@@ -35,7 +40,7 @@ What a design may ask for beside these, each with a parameter (none of it togeth
   (`<prefix>.rel` [rows, heads], rows by `distance_rows`).
 * `entry_gate`: every entry of the heads' result times the sigmoid of one more projection of h (`<prefix>.g`, a row an
   entry).
-Biases, norms and the store into the cache are one kernel (`qkv_norm_store`) on the product's 32-bit result; what
+Biases, rotation, norms and the store into the cache are one kernel (`qkv_norm_store`) on the product's 32-bit result; what
 shapes a score and the gate are inside the attention kernel.
 
 All projections of h are one matrix product ([q | k | v | gate]).
@@ -49,17 +54,18 @@ import torch
 
 from .base import (MIXERS, POSITION_ENCODINGS, VECTOR32, BuildEnv, KVNeed, LayerCache, Mixer, PartSpec, StepContext,
                    TensorSpec, build_part, product_weight, project)
-from .rope import rotary_frequencies, rotary_magnitude
+from .rope import rotary_frequencies, rotary_magnitude, step_angles
 
 
 def split_scratch(ctx: StepContext, dtype, heads: int, kv_heads: int, key_dim: int, value_dim: int, block_size: int,
-                  window: int, keep_first: int) -> Dict[str, object]:
+                  window: int, keep_first: int, chunk: int = 0) -> Dict[str, object]:
     """The keywords with which `sink_attention` may share a decoding step's keys out over several workgroups a tile:
     the step's bound of the lengths and the scratch that the kernel object asks for (nothing where it asks for none)."""
     ask = getattr(ctx.kernels, "sink_attention_workspace", None)
     if ask is None or not ctx.decode:
         return {}
-    need = ask(dtype, ctx.rows, ctx.batch, heads, kv_heads, key_dim, value_dim, block_size, window, keep_first, ctx.max_len)
+    need = ask(dtype, ctx.rows, ctx.batch, heads, kv_heads, key_dim, value_dim, block_size, window, keep_first, ctx.max_len,
+               **({"chunk": chunk} if chunk else {}))
     return dict(max_len=ctx.max_len, workspace=ctx.ws.alloc((need,), torch.float32)) if need else {}
 
 
@@ -90,7 +96,7 @@ class SinkWindowAttention(Mixer):
                  probabilities: str = "float32", qkv_bias: bool = False, out_bias: bool = False,
                  qk_norm: Optional[str] = None, value_norm: bool = False, norm_eps: float = 0.0,
                  values_from_keys: bool = False, temperature: bool = False, softcap: float = 0.0, log_bias: bool = False,
-                 table_bias: Optional[Mapping] = None, entry_gate: bool = False) -> None:
+                 table_bias: Optional[Mapping] = None, entry_gate: bool = False, chunk: int = 0) -> None:
         if heads % kv_heads != 0:
             raise ValueError(f"{heads} heads cannot share {kv_heads} kv heads evenly")
         self.rot_dims, self.rot_interleaved, self.rot_magnitude, self.freq_table = 0, False, 1.0, []
@@ -108,26 +114,32 @@ class SinkWindowAttention(Mixer):
             self.freq_table = rotary_frequencies(self.rot_dims, float(rotary["base"]), scaling)
             self.rot_magnitude = rotary_magnitude(scaling)
         self.qk_norm_eps = None if qk_norm_eps is None else float(qk_norm_eps)
-        self.prepared = rotary is not None or qk_norm_eps is not None  # q, k and v pass the kernel named above
-        if self.prepared and head_gate:
+        if (rotary is not None or qk_norm_eps is not None) and head_gate:
             raise ValueError("a gate per head and a rotation or norm of q and k are not combined")
-        if qk_norm not in (None, "head", "row"):
-            raise ValueError(f"q and k are normed by 'head' or by 'row' (or not: None), found {qk_norm!r}")
+        if qk_norm not in (None, "head", "row", "unit"):
+            raise ValueError(f"q and k are normed by 'head', 'row' or 'unit' (or not: None), found {qk_norm!r}")
         self.qkv_bias, self.has_out_bias, self.qk_norm, self.value_norm = bool(qkv_bias), bool(out_bias), qk_norm, bool(value_norm)
         self.norm_eps, self.values_from_keys, self.temperature = float(norm_eps), bool(values_from_keys), bool(temperature)
         self.softcap, self.log_bias, self.entry_gate = float(softcap), bool(log_bias), bool(entry_gate)
         self.table_bias = None if table_bias is None else (int(table_bias["rows"]), float(table_bias["most"]))
         self.stored = bool(qkv_bias or qk_norm or value_norm or values_from_keys or entry_gate)  # by `qkv_norm_store`
         self.shaped = bool(temperature or softcap or log_bias or table_bias is not None or entry_gate)
-        if self.stored and (self.prepared or position is not None or head_gate):
-            raise ValueError("biases, weighted norms, values from keys or a gate an entry are not combined with a rotation, "
-                             "a unit norm of q and k or a gate a head")
+        if self.stored and (qk_norm_eps is not None or position is not None or head_gate):
+            raise ValueError("biases, weighted norms, values from keys or a gate an entry are not combined with a position "
+                             "part, `qk_norm_eps` or a gate a head")
+        if rotary is not None and qk_norm == "row":
+            raise ValueError("a norm over all heads of a row together is not combined with a rotation ahead of it")
+        # without any of those, q, k and v pass the kernel that rotates and norms them (`rotary_qkv`)
+        self.prepared = not self.stored and (rotary is not None or qk_norm_eps is not None)
         if self.values_from_keys and key_dim != value_dim:
             raise ValueError(f"values that are the keys are as wide as they are ({key_dim}, {value_dim})")
         if self.softcap < 0:
             raise ValueError("the cap on the scores must not be negative")
-        if window < 0 or keep_first < 0:
-            raise ValueError("window and keep_first must not be negative")
+        if window < 0 or keep_first < 0 or chunk < 0:
+            raise ValueError("window, keep_first and chunk must not be negative")
+        if chunk and keep_first:
+            raise ValueError("chunks keep no first tokens")
+        self.chunk = int(chunk)
         self.width, self.heads, self.kv_heads = int(width), int(heads), int(kv_heads)
         self.key_dim, self.value_dim = int(key_dim), int(value_dim)
         self.scale, self.window, self.keep_first = float(scale), int(window), int(keep_first)
@@ -167,7 +179,7 @@ class SinkWindowAttention(Mixer):
             specs.append(TensorSpec(nm[key], (width, self.width)))
             if self.qkv_bias and key != "gate":
                 specs.append(TensorSpec(nm[key] + ".b", (width,), kind=VECTOR32))
-        if self.qk_norm:
+        if self.qk_norm in ("head", "row"):
             whole = self.qk_norm == "row"
             specs += [TensorSpec(nm["q_norm"], (self.q_width if whole else self.key_dim,), kind=VECTOR32, init="around_one"),
                       TensorSpec(nm["k_norm"], (self.k_width if whole else self.key_dim,), kind=VECTOR32, init="around_one")]
@@ -193,7 +205,8 @@ class SinkWindowAttention(Mixer):
         if self.learned_sink:
             self.sink_w = tensors[self.names["sink"]].contiguous()
         get = lambda key, there: tensors[nm[key]].contiguous() if there else None
-        self.q_norm_w, self.k_norm_w = get("q_norm", self.qk_norm), get("k_norm", self.qk_norm)
+        weighted = self.qk_norm in ("head", "row")
+        self.q_norm_w, self.k_norm_w = get("q_norm", weighted), get("k_norm", weighted)
         self.in_bias = torch.cat([tensors[nm[key] + ".b"] for key, _ in self._projections() if key != "gate"]).contiguous() \
             if self.qkv_bias else None
         self.out_bias = tensors[nm["o"] + ".b"].contiguous() if self.has_out_bias else None
@@ -213,11 +226,12 @@ class SinkWindowAttention(Mixer):
 
     def cache_need(self) -> KVNeed:
         # a window that keeps first tokens still gives its middle blocks back
-        return KVNeed(self.kv_heads, self.key_dim, self.window, self.value_dim, self.keep_first if self.window else 0)
+        return KVNeed(self.kv_heads, self.key_dim, self.window, self.value_dim, self.keep_first if self.window else 0,
+                      self.chunk)
 
     def lengths_uneven(self, kernels, lengths) -> bool:
         ask = getattr(kernels, "decode_lengths_uneven", None)
-        plain = not (self.sink or self.head_gate or self.keep_first or self.window or self.shaped) and self.key_dim == self.value_dim \
+        plain = not (self.sink or self.head_gate or self.keep_first or self.window or self.chunk or self.shaped) and self.key_dim == self.value_dim \
             and self.probabilities == "bfloat16"
         return bool(ask(lengths)) if ask is not None and plain else False
 
@@ -225,7 +239,7 @@ class SinkWindowAttention(Mixer):
         """Whether this step's attention is the causal kernel's (`attention`): the design lets the probabilities be
         rounded to bfloat16 for their product with the values (that kernel's way; the general kernel keeps them
         32-bit), the mask and softmax are plain, and the kernel object runs the shape on its matrix cores."""
-        if self.probabilities != "bfloat16" or self.sink or self.head_gate or self.keep_first or self.shaped \
+        if self.probabilities != "bfloat16" or self.sink or self.head_gate or self.keep_first or self.chunk or self.shaped \
                 or self.key_dim != self.value_dim:
             return False
         ask = getattr(kn, "attention_on_matrix_cores", None)
@@ -248,8 +262,12 @@ class SinkWindowAttention(Mixer):
             n_qkv = total - (self.o_width if self.entry_gate else 0)
             place = dict(row_pos=ctx.row_pos, row_seq=ctx.row_seq, seq_slot=ctx.seq_slot, block_table=cache.block_table,
                          kcache=cache.k, vcache=cache.v, block_size=cache.block_size) if cache.write else {}
+            if self.rot_dims:
+                place.update(cos_sin=step_angles(ctx, self.freqs, self.freq_table), interleaved=self.rot_interleaved,
+                             magnitude=self.rot_magnitude)
             kn.qkv_norm_store(proj[:, :n_qkv], q, self.heads, self.kv_heads, self.key_dim, self.value_dim, self.norm_eps,
-                              bias=self.in_bias, q_weight=self.q_norm_w, k_weight=self.k_norm_w, norm_qk=self.qk_norm,
+                              bias=self.in_bias, q_weight=self.q_norm_w, k_weight=self.k_norm_w,
+                              norm_qk="head" if self.qk_norm == "unit" else self.qk_norm,
                               norm_v=self.value_norm, v_from_k=self.values_from_keys, **place)
             wide_gate = proj[:, n_qkv:] if self.entry_gate else None
         elif self.prepared:
@@ -290,9 +308,9 @@ class SinkWindowAttention(Mixer):
                           window=self.window, keep_first=self.keep_first, sink=self.sink, gate=gate,
                           decode=ctx.decode, **self.shape_kw, **({"wide_gate": wide_gate} if wide_gate is not None else {}),
                           **({"sink_values": self.sink_w} if self.learned_sink else {}),
-                          **split_scratch(ctx, q.dtype, self.heads, self.kv_heads, self.key_dim,
-                                                             self.value_dim, cache.block_size, self.window,
-                                                             self.keep_first))
+                          **({"chunk": self.chunk} if self.chunk else {}),
+                          **split_scratch(ctx, q.dtype, self.heads, self.kv_heads, self.key_dim, self.value_dim,
+                                          cache.block_size, self.window, self.keep_first, self.chunk))
         return self._project_out(ctx, att, out, leave_bias)
 
     def _project_out(self, ctx: StepContext, att: torch.Tensor, out: Optional[torch.Tensor], leave_bias: bool) -> torch.Tensor:

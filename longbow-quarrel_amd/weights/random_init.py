@@ -45,6 +45,9 @@ def random_tensors(specs: Sequence[TensorSpec], seed: int, dtype: torch.dtype, s
             continue
         if s.init == "around_one":
             t = torch.empty(s.shape, dtype=torch.float32, device=device).normal_(1.0, gain_spread, generator=gen)
+        elif s.init == "around_identity":
+            t = torch.empty(s.shape, dtype=torch.float32, device=device).normal_(0.0, gain_spread, generator=gen)
+            t += torch.eye(*s.shape, dtype=torch.float32, device=device)
         elif s.init == "zeros":
             t = torch.zeros(s.shape, dtype=torch.float32, device=device)
         elif s.init == "normal":

@@ -44,6 +44,10 @@ class CpuKernels:
         return 1
 
     @query
+    def linear_narrow_pieces(self, dtype, m, n, k):
+        return 1
+
+    @query
     def linear_fused_parts(self, dtype, m, n, k):
         return 0
 
@@ -153,6 +157,8 @@ class CpuKernels:
             return 0.5 * g * (1 + torch.tanh(math.sqrt(2 / math.pi) * (g + 0.044715 * g * g * g)))
         if activation == "gelu":
             return 0.5 * g * (1 + torch.erf(g * math.sqrt(0.5)))
+        if activation == "relu2":
+            return torch.clamp(g, min=0) ** 2
         raise ValueError(activation)
 
     def activation(self, x, out, activation):
@@ -163,7 +169,7 @@ class CpuKernels:
         g, u = gate_up[:, :inner].float(), gate_up[:, inner:].float()
         if bias is not None:
             g, u = g + bias[:inner], u + bias[inner:]
-        if activation == "gelu":
+        if activation in ("gelu", "relu2"):
             raise ValueError(activation)
         a = self._act(g, activation)
         if row_gate is not None:
@@ -184,7 +190,7 @@ class CpuKernels:
     def sink_attention(self, q, out, heads, kv_heads, key_dim, value_dim, row_pos, row_seq, seq_slot, block_table,
                        kcache, vcache, block_size, scale, window=0, keep_first=0, sink=True, gate=None, decode=False,
                        sink_values=None, maps=1, softcap=0.0, temp=None, log_bias=None, distance_bias=None,
-                       wide_gate=None):
+                       wide_gate=None, chunk=0):
         if maps > 1:  # a cached key row holds the keys of `maps` key heads side by side; they share the value head
             nb, g_heads, bs, wide = kcache.shape
             kcache = kcache.reshape(nb, g_heads, bs, maps, key_dim).permute(0, 1, 3, 2, 4).reshape(nb, kv_heads, bs, key_dim)
@@ -193,7 +199,7 @@ class CpuKernels:
             p = int(row_pos[r])
             slot = int(seq_slot[int(row_seq[r])])
             lo = p - window + 1 if (window > 0 and p >= window) else 0
-            ts = [t for t in range(p + 1) if t >= lo or t < keep_first]
+            ts = [t for t in range(p + 1) if (t >= lo or t < keep_first) and (not chunk or t // chunk == p // chunk)]
             kk = torch.stack([kcache[int(block_table[slot, t // block_size]), :, t % block_size, :] for t in ts]).float()
             vv = torch.stack([vcache[int(block_table[slot, t // block_size]), :, :, t % block_size] for t in ts]).float()
             for h in range(heads):
@@ -291,7 +297,8 @@ class CpuKernels:
         v = y.float() * gate if gate_first else y.float()
         v = v.reshape(rows, n // group, group)
         v = (v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps)).reshape(rows, n)
-        v = v * (weight if weight.numel() == n else weight.repeat(n // weight.numel()))
+        if weight is not None:
+            v = v * (weight if weight.numel() == n else weight.repeat(n // weight.numel()))
         out.copy_((v if gate_first else v * gate).to(out.dtype))
 
     def rmsnorm_mean(self, stack, weights, eps, out, biases=None):
@@ -348,7 +355,8 @@ class CpuKernels:
 
     def qkv_norm_store(self, src, q_out, heads, kv_heads, key_dim, value_dim, eps, bias=None, q_weight=None, k_weight=None,
                        norm_qk=None, norm_v=False, v_from_k=False, row_pos=None, row_seq=None, seq_slot=None,
-                       block_table=None, kcache=None, vcache=None, block_size=0):
+                       block_table=None, kcache=None, vcache=None, block_size=0, cos_sin=None, interleaved=False,
+                       magnitude=1.0):
         rows, qw, kw = src.shape[0], heads * key_dim, kv_heads * key_dim
         t = src.float() if bias is None else src.float() + bias
 
@@ -359,6 +367,8 @@ class CpuKernels:
 
         q, k = t[:, :qw], t[:, qw : qw + kw]
         v = k if v_from_k else t[:, qw + kw :]
+        if cos_sin is not None:
+            q, k = (self._turned(x, key_dim, cos_sin, interleaved, magnitude) for x in (q, k))
         if norm_qk:
             q = unit(q, q_weight, qw if norm_qk == "row" else key_dim)
             k = unit(k, k_weight, kw if norm_qk == "row" else key_dim)
@@ -368,6 +378,47 @@ class CpuKernels:
         if kcache is not None:
             self.kv_store(k.to(kcache.dtype), v.to(vcache.dtype), kv_heads, key_dim, value_dim, row_pos, row_seq, seq_slot,
                           block_table, kcache, vcache, block_size)
+
+    @staticmethod
+    def _turned(x, size, cos_sin, interleaved, magnitude):
+        rows, half = x.shape[0], cos_sin.shape[1]
+        v = x.reshape(rows, -1, size).clone()
+        c, s = cos_sin[:, None, :, 0] * magnitude, cos_sin[:, None, :, 1] * magnitude
+        first, second = (slice(0, 2 * half, 2), slice(1, 2 * half, 2)) if interleaved else (slice(0, half), slice(half, 2 * half))
+        a, b = v[..., first].clone(), v[..., second].clone()
+        v[..., first], v[..., second] = a * c - b * s, b * c + a * s
+        return v.reshape(rows, -1)
+
+    def decay_scan(self, q, k, v, powers, state, out, heads, key_dim, value_dim, k_scale, seq_slot, cu_rows, batch,
+                   activation=None, cos_sin=None, interleaved=False, magnitude=1.0):
+        if activation is not None:
+            q, k, v = (self._act(x, activation) for x in (q, k, v))
+        if cos_sin is not None:
+            q, k = (self._turned(x, key_dim, cos_sin, interleaved, magnitude) for x in (q, k))
+        decay = powers[:, 1][:, None, None]
+        for b in range(batch):
+            s = state[int(seq_slot[b])]  # [heads, value_dim, key_dim]
+            for r in range(int(cu_rows[b]), int(cu_rows[b + 1])):
+                kr, vr = k[r].reshape(heads, 1, key_dim) * k_scale, v[r].reshape(heads, value_dim, 1)
+                s.mul_(decay).add_(vr * kr)
+                out[r] = (s * q[r].reshape(heads, 1, key_dim)).sum(-1).reshape(-1)
+
+    def streams_step(self, src, streams, y=None, mix=None, out_weights=None, out=None, read=None, norm_weight=None, eps=0.0,
+                     h=None):
+        X = src.expand(streams, *src.shape) if src.dim() == 2 else src
+        if y is not None:
+            whole = y.sum(0) if y.dim() == 3 else y
+            X = torch.einsum("st,srw->trw", mix, X) + out_weights[:, None, None] * whole
+            out.copy_(X)
+        if h is not None:
+            u = X.sum(0) if read is None else torch.einsum("s,srw->rw", read, X)
+            h.copy_((u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * norm_weight).to(h.dtype))
+
+    def softcap(self, x, cap, factor=1.0):
+        x.copy_(cap * torch.tanh(x * factor / cap))
+
+    def sum_pieces(self, pieces, out):
+        out.copy_(pieces.sum(0).to(out.dtype))
 
     def selective_scan(self, x, dt, b_in, c_in, z, dt_bias, a_log, d_skip, state, out, seq_slot, cu_rows, batch):
         a = -torch.exp(a_log)
@@ -476,6 +527,13 @@ class CpuKernels:
 
     def moe_route(self, logits, route, top, renormalize=False, correction=None, groups=0, keep=0, scoring="sigmoid",
                   group_mark="top2", renormalize_eps=0.0, identity=None):
+        if scoring == "softmax_chosen":
+            route.fill_(-1.0)
+            for r in range(logits.shape[0]):
+                z = logits[r].tolist()
+                chosen = sorted(range(len(z)), key=lambda e: (-z[e], e))[:top]
+                route[r, chosen] = torch.softmax(logits[r, chosen].float(), 0)
+            return
         s = torch.sigmoid(logits.float()) if scoring == "sigmoid" else torch.softmax(logits.float(), -1)
         c = s + correction if correction is not None else s
         experts = s.shape[1]
@@ -520,6 +578,11 @@ class CpuKernels:
             y = y * w
         y = torch.where(w >= 0, y, torch.zeros_like(y))
         out.copy_(y.reshape(rows, experts * ff).to(out.dtype))
+
+    def moe_act(self, u, route, out, experts, ff, activation, shared=0):
+        w = route.float().reshape(-1, experts).clamp(min=0).repeat_interleave(ff, dim=1)
+        w = torch.cat([w, torch.ones(w.shape[0], shared)], dim=1)
+        out.copy_((self._act(u.float(), activation) * w).to(out.dtype))
 
     def moe_sort(self, route, counts, order, weight, place_of):
         rows, experts = route.shape

@@ -152,7 +152,8 @@ def test_missing_and_unexpected_tensors_are_named(tmp_path):
 def test_mechanisms_that_do_not_go_together_are_refused():
     from longbow_quarrel_amd.parts.sink_attention import SinkWindowAttention
     sizes = dict(width=8, heads=2, kv_heads=1, key_dim=4, value_dim=4, scale=1.0, prefix="x")
-    for more in (dict(qkv_bias=True, rotary={"dims": 4, "base": 10.0}), dict(entry_gate=True, head_gate=True),
+    for more in (dict(qk_norm="row", rotary={"dims": 4, "base": 10.0}),
+                 dict(qkv_bias=True, qk_norm_eps=1e-6), dict(entry_gate=True, head_gate=True),
                  dict(qk_norm="rows"), dict(values_from_keys=True, key_dim=4, value_dim=8), dict(softcap=-1.0)):
         with pytest.raises(ValueError):
             SinkWindowAttention(**{**sizes, **more})
