@@ -41,6 +41,10 @@ design of the same sizes (the closest: the same attention kernel and delta rule,
 `--design puzonex`: the same for the design of the selective scan, windowed attention with capped and biased scores, and
 attention whose values are its keys beside a matrix memory (per four layers two, one and one); beside the Llama shape
 and beside the Vafodra design of the same sizes (the closest: windowed attention with a sink beside a state-space scan).
+`--design tukedra`: the same for the design of linear attention with fixed decays and attention within chunks over four
+residual streams (per four layers lightning attention, retention, attention, lightning attention; experts of two
+matrices); beside the Llama shape and beside the Vupelorn design of the same sizes (the closest: gated linear attention,
+attention over the paged cache by the same kernel, a mixture of experts).
 """
 from __future__ import annotations
 
@@ -205,6 +209,28 @@ def puzonex_config(width: int, layers: int, vocab: int) -> dict:
     return {"architecture": "Puzonex", "layers": made, "norm": {"eps": 1e-5}, "vocab": vocab, "width": width}
 
 
+def tukedra_config(width: int, layers: int, vocab: int) -> dict:
+    """Layer sizes of a real model for the design.  Per four layers: lightning attention (heads of 128 x 128), retention
+    (half as many heads of 256 x 256), attention within chunks of 1 024 (heads of 128, a fourth as many key heads, 64
+    entries rotated under YaRN), lightning attention.  Four residual streams.  A gated unit of 3.5 times the width in the
+    first layer; elsewhere 8 experts of two matrices, 2 a token, beside a shared one, each 1.75 times the width (a token's
+    three together: the weights of that unit)."""
+    heads = width // 128
+    fading = lambda n: [1.0 - 2.0 ** (-5.0 - 3.0 * i / max(1, n - 1)) for i in range(n)]
+    lightning = {"heads": heads, "dim": 128, "vdim": 128, "decay": fading(heads)}
+    half = max(1, heads // 2)
+    retention = {"heads": half, "dim": 256, "vdim": 256, "decay": fading(half), "rot": {"base": 10000.0, "dims": 256}}
+    yarn = {"base": 10000.0, "dims": 64, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}
+    chunked = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+               "mask": {"size": 1024}, "rot": yarn}
+    kinds = (("lightning", lightning), ("retention", retention), ("attention", chunked), ("lightning", lightning))
+    dense = {"kind": "dense", "ff": width * 7 // 2}
+    moe = {"kind": "moe", "expert": {"ff": width * 7 // 4}, "shared": {"ff": width * 7 // 4}, "router": {"experts": 8, "top": 2}}
+    made = [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": moe if i else dense} for i in range(layers)]
+    return {"architecture": "Tukedra", "embedding": {"scale": 1.0}, "layers": made, "logit_scale": 1.0, "logit_softcap": 30.0,
+            "norm": {"eps": 1e-5}, "streams": 4, "vocab": vocab, "width": width}
+
+
 def design_run(args) -> int:
     import torch
 
@@ -223,8 +249,9 @@ def design_run(args) -> int:
                 "vupelorn": lambda: lq.VupelornConfig.from_dict(vupelorn_config(width, layers, vocab)),
                 "mifidra": lambda: lq.MifidraConfig.from_dict(mifidra_config(width, layers, vocab)),
                 "sofinex": lambda: lq.SofinexConfig.from_dict(sofinex_config(width, layers, vocab)),
-                "puzonex": lambda: lq.PuzonexConfig.from_dict(puzonex_config(width, layers, vocab))}
-        closest = {"mifidra": "vafodra", "sofinex": "mifidra", "puzonex": "vafodra"}.get(args.design)
+                "puzonex": lambda: lq.PuzonexConfig.from_dict(puzonex_config(width, layers, vocab)),
+                "tukedra": lambda: lq.TukedraConfig.from_dict(tukedra_config(width, layers, vocab))}
+        closest = {"mifidra": "vafodra", "sofinex": "mifidra", "puzonex": "vafodra", "tukedra": "vupelorn"}.get(args.design)
         beside = [(closest, made[closest]())] if closest else []
         for name, config in [(args.design, made[args.design]())] + beside + [("llama", lq.LlamaConfig.from_dict(llama))]:
             engine = lq.random_engine(config, seed=0, dtype=args.dtype, max_tokens=batch * 4096 + n_prefill + 64,
@@ -315,7 +342,7 @@ def main() -> int:
                     help="float32: the true 32-bit path (use --layers with the larger shapes)")
     ap.add_argument("--context", type=int, default=0,
                     help="tokens a sequence may hold (default: the shape's 8192); for decoding over longer prompts")
-    ap.add_argument("--design", choices=["vafodra", "vupelorn", "mifidra", "sofinex", "puzonex"], default=None,
+    ap.add_argument("--design", choices=["vafodra", "vupelorn", "mifidra", "sofinex", "puzonex", "tukedra"], default=None,
                     help="measure this design beside the Llama shape of equal size instead of the default workload")
     ap.add_argument("--design-widths", default="2048,4096", help="model widths of --design, with commas between them")
     args = ap.parse_args()

@@ -65,7 +65,7 @@ def random_engine(config: ModelConfig, seed: int, dtype: Union[str, torch.dtype]
     specs = model.tensor_specs()
     tensors = random_tensors(specs, seed, env.dtype, std, device=env.device)
     for s in specs:  # the same dtype rule as for files
-        if s.kind == "vector32":
+        if s.kind == "vector32" and s.name in tensors:
             tensors[s.name] = tensors[s.name].float()
     check_names_and_shapes(specs, {n: tuple(t.shape) for n, t in tensors.items()}, "random weights")
     model.bind(tensors, env, consume=True)
