@@ -45,20 +45,54 @@ __device__ inline float taken_in(const DecayArgs& a, const float* row, const flo
   return first ? v * c - m * s : v * c + m * s;
 }
 
-// Entries n .. n + 3 (zeros from `size` on).  FOURS: size and the row's place allow whole vectors.
-template <bool FOURS>
-__device__ inline float4 taken_in4(const DecayArgs& a, const float* row, const float* cs, int n, int size) {
-  if (FOURS && (cs == nullptr || n >= a.dims)) {
-    if (n >= size) return make_float4(0.f, 0.f, 0.f, 0.f);
-    const float4 v = *(const float4*)(row + n);
-    return make_float4(activate(v.x, a.act), activate(v.y, a.act), activate(v.z, a.act), activate(v.w, a.act));
+// How the chunks' kernels take q, k and v in.  The fast ways ask for whole vectors of four everywhere, have no branch
+// between their loads, so that a thread's loads are in flight together, and are made for what they name.
+enum { TAKE_ANY = 0, TAKE_SILU = 1, TAKE_HALF = 2 };  // any; silu and no rotation; half-split pairs and no activation
+
+// A quad of a head's row and what its rotation needs, as loaded.
+template <int TAKE>
+struct Quad {
+  float4 v, mate, c0, c1;
+};
+
+// Entries n .. n + 3 of a head's row of `size` entries (TAKE_ANY: of the row itself, without loads ahead).
+template <int TAKE>
+__device__ inline void load_quad(const DecayArgs& a, Quad<TAKE>& q, const float* row, const float* cs, int n, int size) {
+  if constexpr (TAKE == TAKE_ANY) return;
+  const int at = min(n, size - 4);
+  q.v = *(const float4*)(row + at);
+  if constexpr (TAKE == TAKE_HALF) {
+    const int half = a.dims >> 1, j = min(at < half ? at : at - half, half - 4);
+    q.mate = *(const float4*)(row + (at < half ? at + half : min(at, a.dims - 4) - half));
+    q.c0 = *(const float4*)(cs + 2 * j), q.c1 = *(const float4*)(cs + 2 * j + 4);
   }
-  float4 v;
-  v.x = n < size ? taken_in(a, row, cs, n) : 0.f;
-  v.y = n + 1 < size ? taken_in(a, row, cs, n + 1) : 0.f;
-  v.z = n + 2 < size ? taken_in(a, row, cs, n + 2) : 0.f;
-  v.w = n + 3 < size ? taken_in(a, row, cs, n + 3) : 0.f;
-  return v;
+}
+
+// What becomes of it (zeros from `size` on, and where `there` is false).
+template <int TAKE>
+__device__ inline float4 use_quad(const DecayArgs& a, const Quad<TAKE>& q, const float* row, const float* cs, int n, int size,
+                                  bool there) {
+  float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
+  if constexpr (TAKE == TAKE_ANY) {
+    if (!there) return o;
+    o.x = n < size ? taken_in(a, row, cs, n) : 0.f;
+    o.y = n + 1 < size ? taken_in(a, row, cs, n + 1) : 0.f;
+    o.z = n + 2 < size ? taken_in(a, row, cs, n + 2) : 0.f;
+    o.w = n + 3 < size ? taken_in(a, row, cs, n + 3) : 0.f;
+    return o;
+  } else {
+    if constexpr (TAKE == TAKE_SILU) {
+      o = make_float4(silu_f(q.v.x), silu_f(q.v.y), silu_f(q.v.z), silu_f(q.v.w));
+    } else {
+      const float sign = n < (a.dims >> 1) ? -a.mag : a.mag, m = a.mag;
+      o.x = q.v.x * (q.c0.x * m) + q.mate.x * (q.c0.y * sign);
+      o.y = q.v.y * (q.c0.z * m) + q.mate.y * (q.c0.w * sign);
+      o.z = q.v.z * (q.c1.x * m) + q.mate.z * (q.c1.y * sign);
+      o.w = q.v.w * (q.c1.z * m) + q.mate.w * (q.c1.w * sign);
+      if (n >= a.dims) o = q.v;
+    }
+    return there && n < size ? o : make_float4(0.f, 0.f, 0.f, 0.f);
+  }
 }
 
 // ---------------------------------------------------------------- token by token
@@ -95,6 +129,10 @@ __global__ __launch_bounds__(256) void decay_walk_kernel(DecayArgs a, int L) {
   for (int r = r0; r < r1; ++r) {
     const float* cs = a.cs != nullptr ? a.cs + (long long)r * a.dims : nullptr;
     const float *qr = a.q + (long long)r * a.ldq + h * N, *kr = a.k + (long long)r * a.ldk + h * N;
+    const float* vr = a.v + (long long)r * a.ldv + h * P;
+    float v[WALK];
+#pragma unroll
+    for (int w = 0; w < WALK; ++w) v[w] = vr[min(col[w], P - 1)];
     __syncthreads();
     for (int n = tid; n < NP; n += 256) {
       qs[n] = n < N ? taken_in(a, qr, cs, n) : 0.f;
@@ -103,14 +141,14 @@ __global__ __launch_bounds__(256) void decay_walk_kernel(DecayArgs a, int L) {
     __syncthreads();
 #pragma unroll
     for (int w = 0; w < WALK; ++w) {
-      const float v = col[w] < P ? activate(a.v[(long long)r * a.ldv + h * P + col[w]], a.act) : 0.f;
+      const float val = activate(v[w], a.act);
       float o = 0.f;
 #pragma unroll
       for (int e = 0; e < E; ++e)
 #pragma unroll
         for (int i = 0; i < VEC; ++i) {
           const int n = (e * L + l) * VEC + i;
-          S[w][e][i] = fmaf(decay, S[w][e][i], ks[n] * v);
+          S[w][e][i] = fmaf(decay, S[w][e][i], ks[n] * val);
           o = fmaf(S[w][e][i], qs[n], o);
         }
       for (int off = 1; off < L; off <<= 1) o += __shfl_xor(o, off, LQ_WAVE);
@@ -149,69 +187,104 @@ __device__ inline int chunk_rows(const DecayArgs& a, int c, int& r0, int& n) {
   return lo;
 }
 
-constexpr int SLICE = 128;  // value columns a workgroup at most
+constexpr int SLICE = 128;  // value columns a workgroup at most: two tiles of 16 a wavefront
 
-// The chunk's keys (scaled, times their decay to the chunk's end with `weigh`) and values, rows of 16 NS and of
-// 16 pt + PAD floats in LDS; entries and rows that are not there are zeros.
-template <int NS, bool FOURS>
-__device__ inline void stage_chunk(const DecayArgs& a, int h, int r0, int n, int p0, int pt, const float* pw, bool weigh,
-                                   float* kt, float* vt) {
-  constexpr int NP = 16 * NS;
-  for (int i = threadIdx.x; i < CHUNK * (NP / 4); i += 256) {
-    const int t = i / (NP / 4), e = (i - t * (NP / 4)) * 4;
-    float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
-    if (t < n) {
-      const float* cs = a.cs != nullptr ? a.cs + (long long)(r0 + t) * a.dims : nullptr;
-      v = taken_in4<FOURS>(a, a.k + (long long)(r0 + t) * a.ldk + h * a.N, cs, e, a.N);
-      const float f = weigh ? a.k_scale * pw[n - 1 - t] : a.k_scale;
-      v.x *= f, v.y *= f, v.z *= f, v.w *= f;
+// A chunk's q or k rows on their way in, as rows of 16 NS + PAD floats in LDS (entries and rows that are not there are
+// zeros), times `scale` and, with `pw`, the decay to the chunk's end.
+template <int NS, int TAKE>
+__device__ inline void stage_rows(const DecayArgs& a, const float* src, int ld, int h, int r0, int n, float scale,
+                                  const float* pw, float* to) {
+  constexpr int NP = 16 * NS, BATCH = NS < 4 ? NS : 4;  // quads whose loads are in flight together
+#pragma unroll 1
+  for (int i0 = 0; i0 < NS; i0 += BATCH) {
+    Quad<TAKE> quad[BATCH];
+    float f[BATCH];
+#pragma unroll
+    for (int k = 0; k < BATCH; ++k) {
+      const int i = (i0 + k) * 256 + threadIdx.x, t = i / (NP / 4), e = (i - t * (NP / 4)) * 4;
+      const long long r = r0 + min(t, n - 1);
+      load_quad<TAKE>(a, quad[k], src + r * ld + h * a.N, a.cs + r * a.dims, e, a.N);
+      f[k] = pw != nullptr ? scale * pw[max(n - 1 - t, 0)] : scale;
     }
-    *(float4*)(kt + t * (NP + PAD) + e) = v;
-  }
-  const int PW = 16 * pt;
-  for (int i = threadIdx.x; i < CHUNK * (PW / 4); i += 256) {
-    const int t = i / (PW / 4), e = (i - t * (PW / 4)) * 4;
-    float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
-    if (t < n) v = taken_in4<FOURS>(a, a.v + (long long)(r0 + t) * a.ldv + h * a.P, nullptr, p0 + e, a.P);
-    *(float4*)(vt + t * (PW + PAD) + e) = v;
+#pragma unroll
+    for (int k = 0; k < BATCH; ++k) {
+      const int i = (i0 + k) * 256 + threadIdx.x, t = i / (NP / 4), e = (i - t * (NP / 4)) * 4;
+      const long long r = r0 + min(t, n - 1);
+      float4 v = use_quad<TAKE>(a, quad[k], src + r * ld + h * a.N, a.cs != nullptr ? a.cs + r * a.dims : nullptr, e, a.N, t < n);
+      v.x *= f[k], v.y *= f[k], v.z *= f[k], v.w *= f[k];
+      *(float4*)(to + t * (NP + PAD) + e) = v;
+    }
   }
 }
 
-// What a chunk adds to the state: [P][N] = sum_j v_j (decay^(n - 1 - j) k_j)^T, in the chunk's place of the scratch.
-template <int NS, bool FOURS>
+// The chunk's values in column p of tokens 16 j + 4 g + e, straight from memory (a wavefront is alone in reading its
+// columns).
+template <int TAKE>
+__device__ inline void load_values(const DecayArgs& a, float (&v)[CHUNK / 16][4], int h, int r0, int n, int g, int p) {
+  const float* col = a.v + h * a.P + min(p, a.P - 1);
+#pragma unroll
+  for (int j = 0; j < CHUNK / 16; ++j)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[j][e] = col[(long long)(r0 + min(16 * j + 4 * g + e, n - 1)) * a.ldv];
+}
+template <int TAKE>
+__device__ inline void use_values(const DecayArgs& a, float (&v)[CHUNK / 16][4], int n, int g, int p) {
+#pragma unroll
+  for (int j = 0; j < CHUNK / 16; ++j)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const float x = TAKE == TAKE_SILU ? silu_f(v[j][e]) : TAKE == TAKE_HALF ? v[j][e] : activate(v[j][e], a.act);
+      v[j][e] = 16 * j + 4 * g + e < n && p < a.P ? x : 0.f;
+    }
+}
+
+// What a chunk adds to the state: [P][N] = sum_j v_j (decay^(n - 1 - j) k_j)^T, in the chunk's place of the scratch.  A
+// wavefront has two tiles of 16 columns of values, for all keys.
+template <int NS, int TAKE>
 __global__ __launch_bounds__(256) void decay_chunk_state_kernel(DecayArgs a) {
-  extern __shared__ __attribute__((aligned(16))) float lds[];
+  extern __shared__ __attribute__((aligned(16))) float kt[];
   constexpr int NP = 16 * NS;
   int r0, n;
   chunk_rows(a, blockIdx.x, r0, n);
   if (n <= 0) return;
-  const int h = blockIdx.y, p0 = blockIdx.z * SLICE, pt = (min(SLICE, a.P - p0) + 15) / 16, PW = 16 * pt;
-  float *kt = lds, *vt = lds + CHUNK * (NP + PAD);
-  stage_chunk<NS, FOURS>(a, h, r0, n, p0, pt, a.powers + h * (CHUNK + 1), true, kt, vt);
+  const int h = blockIdx.y, wave = threadIdx.x >> 6, lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
+  const int p0 = blockIdx.z * SLICE + 16 * wave;  // the first tile's columns; the second's lie 64 on
+  float v[2][CHUNK / 16][4];
+#pragma unroll
+  for (int t = 0; t < 2; ++t) load_values<TAKE>(a, v[t], h, r0, n, g, p0 + 64 * t + c);
+  stage_rows<NS, TAKE>(a, a.k, a.ldk, h, r0, n, a.k_scale, a.powers + h * (CHUNK + 1), kt);
+#pragma unroll
+  for (int t = 0; t < 2; ++t) use_values<TAKE>(a, v[t], n, g, p0 + 64 * t + c);
   __syncthreads();
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
+  if (p0 >= a.P) return;
+  const bool two = p0 + 64 < a.P;
   float* to = a.scratch + ((long long)blockIdx.x * a.heads + h) * a.P * a.N;
-  for (int t = wave; t < pt; t += 4) {
-    f32x4 acc[NS];
+  f32x4 acc[2][NS];
 #pragma unroll
-    for (int s = 0; s < NS; ++s) acc[s] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    for (int j = 0; j < CHUNK / 16; ++j)
+  for (int s = 0; s < NS; ++s) acc[0][s] = acc[1][s] = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int tok = 16 * j + 4 * g + e;
-        const float v = vt[tok * (PW + PAD) + 16 * t + c];
+  for (int j = 0; j < CHUNK / 16; ++j) {
+    if (16 * j >= n) break;
 #pragma unroll
-        for (int s = 0; s < NS; ++s)
-          acc[s] = __builtin_amdgcn_mfma_f32_16x16x4f32(v, kt[tok * (NP + PAD) + 16 * s + c], acc[s], 0, 0, 0);
+    for (int e = 0; e < 4; ++e) {
+      const float* kr = kt + (16 * j + 4 * g + e) * (NP + PAD) + c;
+#pragma unroll
+      for (int s = 0; s < NS; ++s) {
+        const float k = kr[16 * s];
+        acc[0][s] = __builtin_amdgcn_mfma_f32_16x16x4f32(v[0][j][e], k, acc[0][s], 0, 0, 0);
+        if (two) acc[1][s] = __builtin_amdgcn_mfma_f32_16x16x4f32(v[1][j][e], k, acc[1][s], 0, 0, 0);
       }
+    }
+  }
+#pragma unroll
+  for (int t = 0; t < 2; ++t)
 #pragma unroll
     for (int s = 0; s < NS; ++s)
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        const int p = p0 + 16 * t + 4 * g + e, m = 16 * s + c;
-        if (p < a.P && m < a.N) to[(long long)p * a.N + m] = acc[s][e];
+        const int p = p0 + 64 * t + 4 * g + e, m = 16 * s + c;
+        if (p < a.P && m < a.N) to[(long long)p * a.N + m] = acc[t][s][e];
       }
-  }
 }
 
 // In every chunk's place the state that the chunk starts from; the sequence's new state into the cache.
@@ -257,94 +330,114 @@ __global__ __launch_bounds__(256) void decay_chain_kernel(DecayArgs a) {
   if (chunks > 0) store(cached, S);
 }
 
-// A chunk's results.  Wavefront w has the rows 16 w .. + 15 of the chunk: the products of its queries with the keys up to
-// its own rows, 16 keys by 16 queries at a time, each times the decay between them, straight into the product with the
-// values; ahead of that the start state's share.
-template <int NS, int PT, bool FOURS>
+// A chunk's results, in two steps.  The scores first: wavefront w has the keys 16 w .. + 15 and makes their products with
+// the queries from its own rows on, 16 keys by 16 queries at a time, each times the decay between them, into LDS.  Then a
+// wavefront has two tiles of 16 columns of values, for all rows: the start state's share (an entry of the state is read
+// by one wavefront alone and meets all rows' queries), and the scores' product with the values.
+template <int NS, int TAKE>
 __global__ __launch_bounds__(256) void decay_chunk_out_kernel(DecayArgs a) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
-  constexpr int NP = 16 * NS, PW = 16 * PT;
+  constexpr int NP = 16 * NS, T = CHUNK / 16, SROW = CHUNK + PAD;
   __shared__ float pw[CHUNK + 1];
+  float *qt = lds, *sc = lds + CHUNK * (NP + PAD);  // queries [64][NP + PAD], scores [64][SROW]
   int r0, n;
   chunk_rows(a, blockIdx.x, r0, n);
   if (n <= 0) return;
-  const int h = blockIdx.y, p0 = blockIdx.z * PW;
-  float *kt = lds, *vt = lds + CHUNK * (NP + PAD);
+  const int h = blockIdx.y, wave = threadIdx.x >> 6, lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
   for (int i = threadIdx.x; i <= CHUNK; i += 256) pw[i] = a.powers[h * (CHUNK + 1) + i];
-  stage_chunk<NS, FOURS>(a, h, r0, n, p0, PT, nullptr, false, kt, vt);
-  __syncthreads();
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
-  if (16 * wave >= n) return;
-  const int i = 16 * wave + c;  // this lane's query row as an operand
-  float4 q[NS];
+  float4 k[NS];  // this wavefront's keys as an operand: key 16 wave + c, entries 16 s + 4 g .. + 3
   {
-    const int r = r0 + min(i, n - 1);
-    const float* cs = a.cs != nullptr ? a.cs + (long long)r * a.dims : nullptr;
-    const float* row = a.q + (long long)r * a.ldq + h * a.N;
+    const int t = 16 * wave + c;
+    const long long r = r0 + min(t, n - 1);
+    const float *row = a.k + r * a.ldk + h * a.N, *cs = a.cs != nullptr ? a.cs + r * a.dims : nullptr;
+    constexpr int BATCH = NS < 4 ? NS : 4;
 #pragma unroll
-    for (int s = 0; s < NS; ++s) q[s] = taken_in4<FOURS>(a, row, cs, 16 * s + 4 * g, a.N);
+    for (int s0 = 0; s0 < NS; s0 += BATCH) {
+      Quad<TAKE> quad[BATCH];
+#pragma unroll
+      for (int j = 0; j < BATCH; ++j) load_quad<TAKE>(a, quad[j], row, cs, 16 * (s0 + j) + 4 * g, a.N);
+#pragma unroll
+      for (int j = 0; j < BATCH; ++j) {
+        float4 x = use_quad<TAKE>(a, quad[j], row, cs, 16 * (s0 + j) + 4 * g, a.N, t < n);
+        x.x *= a.k_scale, x.y *= a.k_scale, x.z *= a.k_scale, x.w *= a.k_scale;
+        k[s0 + j] = x;
+      }
+    }
   }
-  f32x4 o[PT];  // o[d][e]: row 16 wave + 4 g + e, value column p0 + 16 d + c
-  const float* start = a.scratch + ((long long)blockIdx.x * a.heads + h) * a.P * a.N;
+  stage_rows<NS, TAKE>(a, a.q, a.ldq, h, r0, n, 1.f, nullptr, qt);
+  __syncthreads();
+  for (int i = wave; i < T; ++i) {
+    if (16 * i >= n) break;
+    f32x4 st = (f32x4){0.f, 0.f, 0.f, 0.f};  // st[e]: key 16 wave + 4 g + e with query 16 i + c
+    const float* qr = qt + (16 * i + c) * (NP + PAD) + 4 * g;
 #pragma unroll
-  for (int d = 0; d < PT; ++d) {
-    o[d] = (f32x4){0.f, 0.f, 0.f, 0.f};
-    const int p = p0 + 16 * d + c;
-    const float* col = start + (long long)min(p, a.P - 1) * a.N + 4 * g;
+    for (int s = 0; s < NS; ++s) {
+      const float4 q = *(const float4*)(qr + 16 * s);
+      st = __builtin_amdgcn_mfma_f32_16x16x4f32(k[s].x, q.x, st, 0, 0, 0);
+      st = __builtin_amdgcn_mfma_f32_16x16x4f32(k[s].y, q.y, st, 0, 0, 0);
+      st = __builtin_amdgcn_mfma_f32_16x16x4f32(k[s].z, q.z, st, 0, 0, 0);
+      st = __builtin_amdgcn_mfma_f32_16x16x4f32(k[s].w, q.w, st, 0, 0, 0);
+    }
+    const int back = 16 * (i - wave) + c - 4 * g;  // query minus key, at e = 0
+    float4 w;
+    w.x = back >= 0 ? st[0] * pw[back] : 0.f;
+    w.y = back >= 1 ? st[1] * pw[back - 1] : 0.f;
+    w.z = back >= 2 ? st[2] * pw[back - 2] : 0.f;
+    w.w = back >= 3 ? st[3] * pw[back - 3] : 0.f;
+    *(float4*)(sc + (16 * i + c) * SROW + 16 * wave + 4 * g) = w;
+  }
+  __syncthreads();
+  const float* start = a.scratch + ((long long)blockIdx.x * a.heads + h) * a.P * a.N;
+#pragma unroll 1
+  for (int d = 0; d < 2; ++d) {
+    const int p = blockIdx.z * SLICE + 16 * (wave + 4 * d) + c;
+    if (p - c >= a.P) break;
+    f32x4 o[T];  // o[i][e]: row 16 i + 4 g + e, value column p
+#pragma unroll
+    for (int i = 0; i < T; ++i) o[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const float* col = start + (long long)min(p, a.P - 1) * a.N;
+    float4 x[NS];
 #pragma unroll
     for (int s = 0; s < NS; ++s) {
       const int m = 16 * s + 4 * g;
-      float4 x;
-      if (FOURS) {
-        x = m < a.N ? *(const float4*)(col + 16 * s) : make_float4(0.f, 0.f, 0.f, 0.f);
+      if constexpr (TAKE != TAKE_ANY) {  // (the queries are zeros from N on; what meets them must be a number)
+        x[s] = *(const float4*)(col + min(m, a.N - 4));
       } else {
-        x.x = m < a.N ? col[16 * s] : 0.f, x.y = m + 1 < a.N ? col[16 * s + 1] : 0.f;
-        x.z = m + 2 < a.N ? col[16 * s + 2] : 0.f, x.w = m + 3 < a.N ? col[16 * s + 3] : 0.f;
+        x[s].x = m < a.N ? col[m] : 0.f, x[s].y = m + 1 < a.N ? col[m + 1] : 0.f;
+        x[s].z = m + 2 < a.N ? col[m + 2] : 0.f, x[s].w = m + 3 < a.N ? col[m + 3] : 0.f;
       }
-      o[d] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[s].x, x.x, o[d], 0, 0, 0);
-      o[d] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[s].y, x.y, o[d], 0, 0, 0);
-      o[d] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[s].z, x.z, o[d], 0, 0, 0);
-      o[d] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[s].w, x.w, o[d], 0, 0, 0);
     }
-  }
+    float v[T][4];
+    load_values<TAKE>(a, v, h, r0, n, g, p);
+    use_values<TAKE>(a, v, n, g, p);
 #pragma unroll
-  for (int e = 0; e < 4; ++e) {
-    const float f = pw[16 * wave + 4 * g + e + 1];
+    for (int s = 0; s < NS; ++s)
 #pragma unroll
-    for (int d = 0; d < PT; ++d) o[d][e] *= f;
-  }
-  for (int t = 0; t <= wave; ++t) {
-    f32x4 st = (f32x4){0.f, 0.f, 0.f, 0.f};  // st[e]: key 16 t + 4 g + e with query i
-    const float* kr = kt + (16 * t + c) * (NP + PAD) + 4 * g;
+      for (int i = 0; i < T; ++i) {
+        const float4 q = *(const float4*)(qt + (16 * i + c) * (NP + PAD) + 16 * s + 4 * g);
+        o[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(q.x, x[s].x, o[i], 0, 0, 0);
+        o[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(q.y, x[s].y, o[i], 0, 0, 0);
+        o[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(q.z, x[s].z, o[i], 0, 0, 0);
+        o[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(q.w, x[s].w, o[i], 0, 0, 0);
+      }
 #pragma unroll
-    for (int s = 0; s < NS; ++s) {
-      const float4 x = *(const float4*)(kr + 16 * s);
-      st = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, q[s].x, st, 0, 0, 0);
-      st = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, q[s].y, st, 0, 0, 0);
-      st = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, q[s].z, st, 0, 0, 0);
-      st = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, q[s].w, st, 0, 0, 0);
-    }
+    for (int i = 0; i < T; ++i) {
+      if (16 * i >= n) break;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int j = 16 * t + 4 * g + e;
-      st[e] = j <= i ? st[e] * pw[max(i - j, 0)] : 0.f;
-    }
+      for (int e = 0; e < 4; ++e) o[i][e] *= pw[16 * i + 4 * g + e + 1];
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const float* vr = vt + (16 * t + 4 * g + e) * (PW + PAD) + c;
+      for (int t = 0; t <= i; ++t) {
+        const float4 w = *(const float4*)(sc + (16 * i + c) * SROW + 16 * t + 4 * g);
+        o[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(w.x, v[t][0], o[i], 0, 0, 0);
+        o[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(w.y, v[t][1], o[i], 0, 0, 0);
+        o[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(w.z, v[t][2], o[i], 0, 0, 0);
+        o[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(w.w, v[t][3], o[i], 0, 0, 0);
+      }
 #pragma unroll
-      for (int d = 0; d < PT; ++d) o[d] = __builtin_amdgcn_mfma_f32_16x16x4f32(st[e], vr[16 * d], o[d], 0, 0, 0);
-    }
-  }
-#pragma unroll
-  for (int e = 0; e < 4; ++e) {
-    const int row = 16 * wave + 4 * g + e;
-    if (row >= n) continue;
-    float* to = a.out + (long long)(r0 + row) * a.ldo + h * a.P;
-#pragma unroll
-    for (int d = 0; d < PT; ++d) {
-      const int p = p0 + 16 * d + c;
-      if (p < a.P) to[p] = o[d][e];
+      for (int e = 0; e < 4; ++e) {
+        const int row = 16 * i + 4 * g + e;
+        if (row < n && p < a.P) a.out[(long long)(r0 + row) * a.ldo + h * a.P + p] = o[i][e];
+      }
     }
   }
 }
@@ -359,29 +452,22 @@ long long chunk_floats(int rows, int batch, int heads, int N, int P, int max_row
   return ((long long)rows / CHUNK + batch) * heads * ((long long)P * N);
 }
 
-template <int NS>
 bool large_lds(const void* kernel, int bytes) {
   return hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, bytes) == hipSuccess;
 }
 
-template <int NS, bool FOURS>
+template <int NS, int TAKE>
 int launch_chunks(const DecayArgs& a, hipStream_t stream) {
-  constexpr int NP = 16 * NS;
-  const int chunks = a.rows / CHUNK + a.batch;
-  const int pw = a.P < SLICE ? (a.P + 15) / 16 * 16 : SLICE;
-  const int lds_k = CHUNK * (NP + PAD) * 4;
-  constexpr int most = CHUNK * (NP + PAD + SLICE + PAD) * 4;
+  constexpr int rows_bytes = CHUNK * (16 * NS + PAD) * 4, out_bytes = rows_bytes + CHUNK * (CHUNK + PAD) * 4;
   static bool ready = false;
   if (!ready) {
-    LQ_REQUIRE(large_lds<NS>((const void*)decay_chunk_state_kernel<NS, FOURS>, most) &&
-                   large_lds<NS>((const void*)decay_chunk_out_kernel<NS, 2, FOURS>, most) &&
-                   large_lds<NS>((const void*)decay_chunk_out_kernel<NS, 4, FOURS>, most) &&
-                   large_lds<NS>((const void*)decay_chunk_out_kernel<NS, 8, FOURS>, most),
-               "decay_scan: %d bytes of LDS are not to be had", most);
+    LQ_REQUIRE(large_lds((const void*)decay_chunk_state_kernel<NS, TAKE>, rows_bytes) &&
+                   large_lds((const void*)decay_chunk_out_kernel<NS, TAKE>, out_bytes),
+               "decay_scan: %d bytes of LDS are not to be had", out_bytes);
     ready = true;
   }
-  decay_chunk_state_kernel<NS, FOURS><<<dim3(chunks, a.heads, lq_ceil_div(a.P, SLICE)), 256,
-                                        lds_k + CHUNK * (pw + PAD) * 4, stream>>>(a);
+  const dim3 grid(a.rows / CHUNK + a.batch, a.heads, lq_ceil_div(a.P, SLICE));
+  decay_chunk_state_kernel<NS, TAKE><<<grid, 256, rows_bytes, stream>>>(a);
   LQ_CHECK_LAUNCH("decay_scan(chunk states)");
   const long long PN = (long long)a.P * a.N;
   if (PN % 4 == 0 && (uintptr_t)a.state % 16 == 0 && (uintptr_t)a.scratch % 16 == 0)
@@ -389,23 +475,17 @@ int launch_chunks(const DecayArgs& a, hipStream_t stream) {
   else
     decay_chain_kernel<1><<<dim3(a.batch * a.heads, (unsigned)lq_ceil_div64(PN, 256)), 256, 0, stream>>>(a);
   LQ_CHECK_LAUNCH("decay_scan(chain)");
-#define LQ_DECAY_OUT(PT)                                                                                   \
-  decay_chunk_out_kernel<NS, PT, FOURS><<<dim3(chunks, a.heads, lq_ceil_div(a.P, 16 * PT)), 256,             \
-                                          lds_k + CHUNK * (16 * PT + PAD) * 4, stream>>>(a)
-  if (a.P <= 32) LQ_DECAY_OUT(2);
-  else if (a.P <= 64) LQ_DECAY_OUT(4);
-  else LQ_DECAY_OUT(8);
-#undef LQ_DECAY_OUT
+  decay_chunk_out_kernel<NS, TAKE><<<grid, 256, out_bytes, stream>>>(a);
   LQ_CHECK_LAUNCH("decay_scan(chunk results)");
   return 0;
 }
 
-template <bool FOURS>
+template <int TAKE>
 int launch_chunks_by_keys(const DecayArgs& a, hipStream_t stream) {
-  if (a.N <= 32) return launch_chunks<2, FOURS>(a, stream);
-  if (a.N <= 64) return launch_chunks<4, FOURS>(a, stream);
-  if (a.N <= 128) return launch_chunks<8, FOURS>(a, stream);
-  return launch_chunks<16, FOURS>(a, stream);
+  if (a.N <= 32) return launch_chunks<2, TAKE>(a, stream);
+  if (a.N <= 64) return launch_chunks<4, TAKE>(a, stream);
+  if (a.N <= 128) return launch_chunks<8, TAKE>(a, stream);
+  return launch_chunks<16, TAKE>(a, stream);
 }
 
 }  // namespace
@@ -438,9 +518,12 @@ extern "C" int lq_decay_scan(const float* q, int ldq, const float* k, int ldk, c
   const long long need = scratch != nullptr ? chunk_floats(rows, batch, heads, N, P, max_rows) : 0;
   LQ_REQUIRE(need <= scratch_floats, "decay_scan: %lld floats of scratch for a step in chunks, %lld given", need, scratch_floats);
   if (need > 0) {
-    const bool fours = N % 4 == 0 && P % 4 == 0 && ldq % 4 == 0 && ldk % 4 == 0 && ldv % 4 == 0 && (uintptr_t)q % 16 == 0 &&
-                       (uintptr_t)k % 16 == 0 && (uintptr_t)v % 16 == 0 && (uintptr_t)scratch % 16 == 0;
-    return fours ? launch_chunks_by_keys<true>(a, stream) : launch_chunks_by_keys<false>(a, stream);
+    const bool fours = N % 4 == 0 && ldq % 4 == 0 && ldk % 4 == 0 && (uintptr_t)q % 16 == 0 && (uintptr_t)k % 16 == 0 &&
+                       (uintptr_t)scratch % 16 == 0;
+    if (fours && act == ACT_SILU && cos_sin == nullptr) return launch_chunks_by_keys<TAKE_SILU>(a, stream);
+    if (fours && act == ACT_NONE && cos_sin != nullptr && !interleaved && dims % 8 == 0 && (uintptr_t)cos_sin % 16 == 0)
+      return launch_chunks_by_keys<TAKE_HALF>(a, stream);
+    return launch_chunks_by_keys<TAKE_ANY>(a, stream);
   }
   const bool vec = N % 4 == 0 && (uintptr_t)state % 16 == 0;
   const int units = vec ? N / 4 : N;

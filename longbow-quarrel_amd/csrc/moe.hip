@@ -10,8 +10,7 @@ namespace {
 // the experts form that many equal groups of neighbours; a group's mark is the sum of its two largest choice scores
 // (of its one, in groups of one), and only experts of the `keep` groups with the largest marks (the lower index on a
 // tie) can be chosen.  `softmax`: s = softmax(z) over all E outputs in the sigmoid's place.  `mark_max`: a group's mark
-// is its largest choice score alone.  `softmax` 2: the `top` largest logits win and the weights are the softmax over these
-// alone (no correction, groups or identity experts).  `renorm_eps` is added to the chosen scores' sum before the division.  The last
+// is its largest choice score alone.  `renorm_eps` is added to the chosen scores' sum before the division.  The last
 // `n_ident` of the E outputs are experts without tensors: their weights go to `ident` [rows, n_ident] (-1: not
 // chosen) and `route` has the E - n_ident others.
 __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ z, int ldz, float* __restrict__ route,
@@ -27,23 +26,6 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
   float* out_ident = n_ident > 0 ? ident + (long long)r * n_ident : nullptr;
   auto out = [&](int e) -> float& { return e < R ? out_real[e] : out_ident[e - R]; };
   for (int e = 0; e < E; ++e) out(e) = -1.f;
-  if (softmax == 2) {
-    float first = 0.f, sum = 0.f;
-    for (int k = 0; k < top; ++k) {
-      int best = -1;
-      float bz = 0.f;
-      for (int e = 0; e < E; ++e)
-        if (out(e) < 0.f && (best < 0 || zr[e] > bz)) best = e, bz = zr[e];
-      if (best < 0) break;
-      if (k == 0) first = bz;
-      const float w = expf(bz - first);
-      out(best) = w == w ? w : 0.f;
-      sum += out(best);
-    }
-    for (int e = 0; e < E; ++e)
-      if (out(e) >= 0.f) out(e) /= sum;
-    return;
-  }
   float zmax = -INFINITY, inv_sum = 1.f;
   if (softmax) {
     for (int e = 0; e < E; ++e) zmax = fmaxf(zmax, zr[e]);
@@ -94,6 +76,54 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
   if (renorm && total > 0.f)
     for (int e = 0; e < E; ++e)
       if (out(e) >= 0.f) out(e) /= total;
+}
+
+// The `top` largest logits win (the lower index on a tie) and the weights are the softmax over these alone.  A wavefront a
+// row: lane l has the logits l, l + 64, ...; every round finds the largest that is left.
+constexpr int ROUTE_PER = 16;  // logits a lane at most
+
+__global__ __launch_bounds__(256) void moe_route_chosen_kernel(const float* __restrict__ z, int ldz, float* __restrict__ route,
+                                                               int rows, int E, int top) {
+  const int r = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (r >= rows) return;
+  float v[ROUTE_PER], w[ROUTE_PER];
+#pragma unroll
+  for (int j = 0; j < ROUTE_PER; ++j) {
+    const int e = lane + 64 * j;
+    v[j] = e < E ? z[(long long)r * ldz + e] : -INFINITY;
+    if (v[j] != v[j]) v[j] = -INFINITY;
+    w[j] = -1.f;
+  }
+  float first = 0.f, sum = 0.f;
+  for (int k = 0; k < top; ++k) {
+    float best = -INFINITY;
+    int at = 0x7fffffff;  // the best's index: among equals, and where nothing is a number, the lowest that is left
+#pragma unroll
+    for (int j = 0; j < ROUTE_PER; ++j) {
+      const int e = lane + 64 * j;
+      if (e < E && w[j] < 0.f && (at == 0x7fffffff || v[j] > best)) best = v[j], at = e;
+    }
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+      const float ob = __shfl_xor(best, off, LQ_WAVE);
+      const int oa = __shfl_xor(at, off, LQ_WAVE);
+      if (oa != 0x7fffffff && (at == 0x7fffffff || ob > best || (ob == best && oa < at))) best = ob, at = oa;
+    }
+    if (at == 0x7fffffff) break;
+    if (k == 0) first = best;
+    float share = expf(best - first);
+    if (share != share) share = 0.f;
+    sum += share;
+#pragma unroll
+    for (int j = 0; j < ROUTE_PER; ++j)
+      if (lane + 64 * j == at) w[j] = share;
+  }
+  const float inv = sum > 0.f ? 1.f / sum : 0.f;
+#pragma unroll
+  for (int j = 0; j < ROUTE_PER; ++j) {
+    const int e = lane + 64 * j;
+    if (e < E) route[(long long)r * E + e] = w[j] < 0.f ? -1.f : w[j] * inv;
+  }
 }
 
 // out[r, :] += h[r, :] * (the sum of the row's chosen identity experts' weights); weights [rows, n] (-1: not chosen)
@@ -264,6 +294,12 @@ extern "C" int lq_moe_route(const float* z, int ldz, float* route, int rows, int
   LQ_REQUIRE(n_ident >= 0 && n_ident < experts && (n_ident == 0 || ident != nullptr) && renorm_eps >= 0.f,
              "moe_route: %d identity experts of %d", n_ident, experts);
   LQ_REQUIRE(z && route, "moe_route: null pointer");
+  if (softmax == 2) {
+    LQ_REQUIRE(experts <= 64 * ROUTE_PER, "moe_route: %d experts (at most %d)", experts, 64 * ROUTE_PER);
+    moe_route_chosen_kernel<<<lq_ceil_div(rows, 4), 256, 0, stream>>>(z, ldz, route, rows, experts, top);
+    LQ_CHECK_LAUNCH("moe_route(softmax over the chosen)");
+    return 0;
+  }
   moe_route_kernel<<<lq_ceil_div(rows, 64), 64, 0, stream>>>(z, ldz, route, rows, experts, top, renormalize, correction,
                                                              groups, keep, softmax, mark_max, renorm_eps, ident, n_ident);
   LQ_CHECK_LAUNCH("moe_route");

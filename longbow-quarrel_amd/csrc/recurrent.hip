@@ -976,6 +976,53 @@ __global__ void gated_rmsnorm_kernel(const float* __restrict__ y, int ldy, const
   }
 }
 
+// The same for groups, strides and weights in fours on whole vectors: a thread keeps its entries in registers between the
+// sum of squares and the result, so a row is read once.  WAVE: a wavefront a (row, group), for groups of up to 512
+// columns; else a workgroup.
+template <typename T, bool WAVE, int KEEP>
+__global__ __launch_bounds__(256) void gated_rmsnorm4_kernel(const float* __restrict__ y, int ldy, const float* __restrict__ z,
+                                                             int ldz, const float* __restrict__ w, int wlen, float eps,
+                                                             int group, int groups, T* __restrict__ out, int ldo,
+                                                             int gate_first, int sigmoid_gate) {
+  __shared__ float red[16];
+  constexpr int STEP = WAVE ? 64 : 256;
+  const int gi = WAVE ? (int)(blockIdx.x * 4 + (threadIdx.x >> 6)) : (int)blockIdx.x, i0 = WAVE ? threadIdx.x & 63 : threadIdx.x;
+  if (gi >= groups) return;  // (WAVE alone: a whole wavefront)
+  const long long r = blockIdx.y;
+  const int c0 = gi * group, quads = group / 4;
+  const float4* yr = (const float4*)(y + r * ldy + c0);
+  const float4* zr = (const float4*)(z + r * ldz + c0);
+  auto gated = [&](float x) { return sigmoid_gate ? sigmoid_f(x) : silu_f(x); };
+  float4 v[KEEP], g[KEEP];
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < KEEP; ++j) {
+    const int i = i0 + j * STEP;
+    v[j] = i < quads ? yr[i] : make_float4(0.f, 0.f, 0.f, 0.f);
+    g[j] = i < quads ? zr[i] : make_float4(0.f, 0.f, 0.f, 0.f);
+  }
+#pragma unroll
+  for (int j = 0; j < KEEP; ++j) {
+    g[j].x = gated(g[j].x), g[j].y = gated(g[j].y), g[j].z = gated(g[j].z), g[j].w = gated(g[j].w);
+    if (gate_first) v[j].x *= g[j].x, v[j].y *= g[j].y, v[j].z *= g[j].z, v[j].w *= g[j].w;
+    ss = fmaf(v[j].x, v[j].x, fmaf(v[j].y, v[j].y, fmaf(v[j].z, v[j].z, fmaf(v[j].w, v[j].w, ss))));
+  }
+  const float inv = 1.f / sqrtf((WAVE ? wave_sum(ss) : block_sum(ss, red)) / group + eps);
+#pragma unroll
+  for (int j = 0; j < KEEP; ++j) {
+    const int i = i0 + j * STEP;
+    if (i >= quads) continue;
+    float4 x = make_float4(v[j].x * inv, v[j].y * inv, v[j].z * inv, v[j].w * inv);
+    if (w != nullptr) {
+      const int at = wlen >= groups * group ? c0 + 4 * i : (4 * i) % wlen;
+      const float4 wv = *(const float4*)(w + at);
+      x.x *= wv.x, x.y *= wv.y, x.z *= wv.z, x.w *= wv.w;
+    }
+    if (!gate_first) x.x *= g[j].x, x.y *= g[j].y, x.z *= g[j].z, x.w *= g[j].w;
+    store4<T>(out + r * ldo + c0 + 4 * i, x);
+  }
+}
+
 struct MeanInputs {
   const float* x[4];
   const float* w[4];
@@ -1304,7 +1351,35 @@ extern "C" int lq_gated_rmsnorm(const float* y, int ldy, const float* z, int ldz
   LQ_REQUIRE(ldy >= n && ldz >= n && ldo >= n, "gated_rmsnorm: a row stride is smaller than its row");
   LQ_REQUIRE(y && z && out, "gated_rmsnorm: null pointer");
   const int threads = group >= 1024 ? 256 : group > 64 ? 128 : 64;
-  for (int r0 = 0; r0 < rows; r0 += 65535) {
+  // everything in fours on whole vectors: the kernel that keeps a group in registers (the choice follows from the model's
+  // sizes and the buffers' alignment, which are the same in every step)
+  const int el = out_dtype == LQ_F32 ? 4 : 2, groups = n / group;
+  const bool fours = group % 4 == 0 && group <= 8192 && ldy % 4 == 0 && ldz % 4 == 0 && ldo % 4 == 0 && (w == nullptr || wlen % 4 == 0) &&
+                     (uintptr_t)y % 16 == 0 && (uintptr_t)z % 16 == 0 && (uintptr_t)w % 16 == 0 &&
+                     (uintptr_t)out % (4 * el) == 0 && (out_dtype == LQ_F32 || out_dtype == LQ_BF16);
+  for (int r0 = 0; fours && r0 < rows; r0 += 65535) {
+    const int nr = rows - r0 < 65535 ? rows - r0 : 65535;
+    const bool wave = group <= 512;
+    const dim3 grid(wave ? lq_ceil_div(groups, 4) : groups, nr);
+#define LQ_GATED4(T, WAVE, KEEP)                                                                                          \
+  gated_rmsnorm4_kernel<T, WAVE, KEEP><<<grid, 256, 0, stream>>>(y + (long long)r0 * ldy, ldy, z + (long long)r0 * ldz, ldz, w, \
+                                                                 wlen, eps, group, groups, (T*)out + (long long)r0 * ldo, ldo, \
+                                                                 gate_first, sigmoid_gate)
+#define LQ_GATED4_T(T)                               \
+  do {                                               \
+    if (group <= 256) LQ_GATED4(T, true, 1);         \
+    else if (wave) LQ_GATED4(T, true, 2);            \
+    else if (group <= 1024) LQ_GATED4(T, false, 1);  \
+    else if (group <= 2048) LQ_GATED4(T, false, 2);  \
+    else if (group <= 4096) LQ_GATED4(T, false, 4);  \
+    else LQ_GATED4(T, false, 8);                     \
+  } while (0)
+    if (out_dtype == LQ_F32) LQ_GATED4_T(float);
+    else LQ_GATED4_T(bf16_t);
+#undef LQ_GATED4_T
+#undef LQ_GATED4
+  }
+  for (int r0 = 0; !fours && r0 < rows; r0 += 65535) {
     const int nr = rows - r0 < 65535 ? rows - r0 : 65535;
     dim3 grid(n / group, nr);
     if (out_dtype == LQ_F32)

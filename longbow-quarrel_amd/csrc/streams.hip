@@ -31,20 +31,26 @@ constexpr int MAX_STREAMS = 16;
 template <typename T, int NS, int KEEP>
 __global__ __launch_bounds__(256) void streams_step4_kernel(StreamArgs a, T* __restrict__ h) {
   __shared__ float red[16];
-  __shared__ float coef[MAX_STREAMS * MAX_STREAMS + 2 * MAX_STREAMS];  // mix, out, read
   const int S = NS > 0 ? NS : a.S;
-  float *mix = coef, *out_w = coef + S * S, *read_w = out_w + S;
-  for (int i = threadIdx.x; i < S * S + 2 * S; i += 256) {
-    float v;
-    if (i < S * S) v = a.y != nullptr ? a.mix[i] : 0.f;
-    else if (i < S * S + S) v = a.y != nullptr ? a.out_w[i - S * S] : 0.f;
-    else v = a.read_w != nullptr ? a.read_w[i - S * S - S] : 1.f;
-    coef[i] = v;
+  constexpr int XS = NS > 0 ? NS : MAX_STREAMS;
+  // the weights are the same for all threads: read once, ahead of all stores (a known few of them into scalar registers)
+  __shared__ float mix_lds[NS > 0 ? 1 : MAX_STREAMS * MAX_STREAMS];
+  float mix_own[NS > 0 ? NS * NS : 1], out_w[XS], read_w[XS];
+  if constexpr (NS > 0) {
+#pragma unroll
+    for (int i = 0; i < NS * NS; ++i) mix_own[i] = a.y != nullptr ? a.mix[i] : 0.f;
+  } else {
+    for (int i = threadIdx.x; i < S * S; i += 256) mix_lds[i] = a.y != nullptr ? a.mix[i] : 0.f;
+    __syncthreads();
   }
-  __syncthreads();
+#pragma unroll
+  for (int t = 0; t < XS; ++t) {
+    out_w[t] = a.y != nullptr && t < S ? a.out_w[t] : 0.f;
+    read_w[t] = a.read_w != nullptr && t < S ? a.read_w[t] : 1.f;
+  }
+  auto mix = [&](int s, int t) { return NS > 0 ? mix_own[NS > 0 ? s * NS + t : 0] : mix_lds[NS > 0 ? 0 : s * S + t]; };
   const long long base = (long long)blockIdx.x * a.width;
   const int n4 = a.width >> 2;
-  constexpr int XS = NS > 0 ? NS : MAX_STREAMS;
   float4 u[KEEP];
   float ss = 0.f;
 #pragma unroll
@@ -69,7 +75,7 @@ __global__ __launch_bounds__(256) void streams_step4_kernel(StreamArgs a, T* __r
 #pragma unroll
         for (int s = 0; s < XS; ++s)
           if (s < S) {
-            const float m = mix[s * S + t];
+            const float m = mix(s, t);
             v.x = fmaf(m, x[s].x, v.x), v.y = fmaf(m, x[s].y, v.y), v.z = fmaf(m, x[s].z, v.z), v.w = fmaf(m, x[s].w, v.w);
           }
         const float o = out_w[t], r = read_w[t];

@@ -9,7 +9,7 @@ from typing import Dict, List, Mapping, Optional
 import torch
 
 from .base import (FEED_FORWARDS, VECTOR32, BuildEnv, FeedForward, NormedRows, StepContext, TensorSpec, product_weight, project,
-                   project_into, project_normed)
+                   project_delta, project_into, project_normed)
 
 
 @FEED_FORWARDS.register("swiglu")
@@ -394,6 +394,9 @@ class MixtureOfExperts(FeedForward):
         """The result in pieces [n, rows, width] that the caller adds: the routed experts' sum, and the shared
         expert's result where a step's rows were sorted by expert (otherwise one product adds both)."""
         rows = h.shape[0]
+        if not self._sorts(rows, ctx) and not self.gated:
+            out = self.forward(h, ctx)  # (whole, or in the pieces that its last product leaves)
+            return out, (1.0,) * (out.shape[0] if out.dim() == 3 else 1)
         if not (self.shared_inner and self._sorts(rows, ctx)):
             out = ctx.ws.alloc((1, rows, self.width), torch.float32)
             self.forward(h, ctx, out=out[0])
@@ -416,9 +419,11 @@ class MixtureOfExperts(FeedForward):
         kn = ctx.kernels
         rows, E, ff, ffs = h.shape[0], self.experts, self.inner, self.shared_inner
         route = self._route(h, ctx)
-        if out is None:
+        sorts = self._sorts(rows, ctx)
+        in_pieces = out is None and not self.gated and not sorts  # what the last product likes to leave
+        if out is None and not in_pieces:
             out = ctx.ws.alloc((rows, self.width), torch.float32)
-        if self._sorts(rows, ctx):
+        if sorts:
             self._sorted(h, route, out, ctx)
             self._pass_on(h, out, ctx)
             if ffs:
@@ -433,6 +438,10 @@ class MixtureOfExperts(FeedForward):
         act = ctx.ws.alloc((rows, E * ff + ffs), ctx.dtype)
         if not self.gated:  # (one launch: the shared expert's columns pass with weight one)
             kn.moe_act(gu, route, act, E, ff, self.activation, shared=ffs)
+            if in_pieces and not self.identity:
+                return project_delta(kn, ctx, act, self.w_down)
+            if out is None:
+                out = ctx.ws.alloc((rows, self.width), torch.float32)
             project(kn, ctx, act, self.w_down, out)
             self._pass_on(h, out, ctx)
             return out
