@@ -365,7 +365,7 @@ def test_every_learned_number_matters(cases, name, leaves):
     ("retention", lambda c: c["layers"][0]["mixer"]["rot"].update(base=101.0)),
     ("retention", lambda c: c["layers"][0]["mixer"]["rot"].update(dims=14)),
     ("chunked", lambda c: c["layers"][0]["mixer"].update(scale=0.31)),
-    ("chunked", lambda c: c["layers"][0]["mixer"]["rot"]["scaling"].update(factor=5.0)),
+    ("chunked", lambda c: c["layers"][0]["mixer"]["rot"]["scaling"].update(factor=6.0)),
     ("chunked", lambda c: c["layers"][0]["mixer"]["rot"]["scaling"].update(original=256)),
     ("experts", lambda c: c["layers"][0]["mlp"]["router"].update(top=3)),
     ("capped", lambda c: c["embedding"].update(scale=2.5)), ("capped", lambda c: c.update(logit_scale=1.75)),

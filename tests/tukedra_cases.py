@@ -29,7 +29,7 @@ def _retention(heads, dim, vdim, decay, rot, mlp):
                                            "rot": {"base": base, "dims": dims}}, "mlp": mlp}
 
 
-def _yarn(base, dims, factor=4.0, original=64, fast=8.0, slow=1.0):
+def _yarn(base, dims, factor=5.0, original=64, fast=8.0, slow=1.0):
     return {"base": base, "dims": dims, "scaling": {"factor": factor, "original": original, "fast": fast, "slow": slow}}
 
 
@@ -82,10 +82,10 @@ CFG_B = _config(97, 51, 1e-6, 1, [
 CFG_C = _config(1000, 256, 1e-5, 4, [
     _lightning(4, 64, 64, [0.9, 0.97, 0.99, 0.999], _dense(384)),
     _retention(2, 128, 128, [0.98, 0.999], (10000.0, 128), _moe(128, 8, 2, 128)),
-    _attention(8, 2, 64, 0.125, _yarn(10000.0, 32, 4.0, 256, 16.0, 1.0), _moe(64, 6, 3, 96), 100),
+    _attention(8, 2, 64, 0.14, _yarn(10000.0, 40, 3.0, 256, 16.0, 1.0), _moe(64, 6, 3, 96), 100),
     _lightning(2, 128, 32, [0.95, 0.9999], _moe(96, 4, 1, 64)),
     _attention(2, 1, 128, 0.1, _yarn(10000.0, 128), _dense(128), 192),
-], scale=0.5, logit_scale=0.5, softcap=20.0)
+], scale=0.6, logit_scale=0.7, softcap=20.0)
 # one mechanism a model: what fails here names its mechanism
 CFG_LIGHTNING = _config(60, 48, 1e-6, 1, [_lightning(3, 16, 24, [0.6, 0.95, 0.9995], None)])
 CFG_RETENTION = _config(60, 48, 1e-6, 1, [_retention(2, 20, 12, [0.8, 0.999], (100.0, 12), None)])
